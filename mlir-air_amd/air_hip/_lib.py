@@ -1,10 +1,11 @@
-"""ctypes binding of libw4a16_hip.so (declared in include/w4a16.h)."""
+"""ctypes bindings of libw4a16_hip.so (include/w4a16.h) and libdense_lm_hip.so (include/dense_lm.h)."""
 
 import ctypes
 import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 _LIB_PATH = os.path.join(os.path.dirname(_HERE), "lib", "libw4a16_hip.so")
+_DENSE_PATH = os.path.join(os.path.dirname(_HERE), "lib", "libdense_lm_hip.so")
 
 OK = 0
 ERR_NULL, ERR_SHAPE, ERR_GROUP, ERR_ALIGN, ERR_WORKSPACE, ERR_HIP, ERR_TUNE, ERR_TIMEOUT, ERR_TOO_LARGE, ERR_NOT_PREPARED = -1, -2, -3, -4, -5, -6, -7, -8, -9, -10
@@ -78,6 +79,61 @@ SYMBOLS = {
 }
 
 
+# ---- libdense_lm_hip.so: descriptor structs and symbols of include/dense_lm.h
+_i32, _i64 = ctypes.c_int32, ctypes.c_int64
+
+
+class Intake(ctypes.Structure):
+    _fields_ = [("mode", _i32), ("width", _i32), ("eps", _cf), ("scale", _cf), ("x", _vp), ("res", _vp), ("y", _vp), ("norm_w", _vp),
+                ("final_w", _vp), ("res_out", _vp), ("h_out", _vp), ("embed", _vp), ("token", _vp)]
+
+
+class Router(ctypes.Structure):
+    _fields_ = [("logits", _vp), ("correction", _vp), ("ld", _i32), ("experts", _i32), ("top", _i32), ("groups", _i32), ("keep", _i32)]
+
+
+class GemmArgs(ctypes.Structure):
+    _fields_ = [("a", _vp), ("w", _vp), ("out", _vp), ("lda", _i64), ("ldo", _i64), ("w_stride", _i64), ("tiles", _vp), ("order", _vp),
+                ("M", _i32), ("N", _i32), ("K", _i32), ("epilogue", _i32), ("n_tiles", _i32), ("gather", _i32), ("tile_rows", _i32)]
+
+
+class LatentShape(ctypes.Structure):
+    _fields_ = [("heads", _i32), ("dim", _i32), ("rot", _i32), ("vdim", _i32), ("rank", _i32), ("rot_pairs", _i32), ("true_rank", _i32),
+                ("scale", _cf)]
+
+
+class LatentRows(ctypes.Structure):
+    _fields_ = [("proj", _vp), ("lut", _vp), ("kv_norm", _vp), ("cache", _vp), ("pos_dev", _vp), ("ld", _i64), ("kv_off", _i32),
+                ("gate_off", _i32), ("M", _i32), ("pos", _i32), ("eps", _cf)]
+
+
+DENSE_SYMBOLS = {
+    "dlm_abi_version": (_ci, []),
+    "dlm_strerror": (ctypes.c_char_p, [_ci]),
+    "dlm_last_hip_error": (ctypes.c_char_p, []),
+    "dlm_gemv_keys": (_ci, [_ci, _ci]),
+    "dlm_gemv": (_ci, [_ci] + [_vp] * 5 + [_ci] * 3 + [_vp]),
+    "dlm_argmax": (_ci, [_vp, _ci] + [_vp] * 4),
+    "dlm_moe_gate_up_gemv": (_ci, [_ci] + [_vp] * 6 + [_ci, _ci, _vp]),
+    "dlm_moe_down_gemv": (_ci, [_ci] + [_vp] * 5 + [_ci] * 4 + [_vp]),
+    "dlm_moe_select": (_ci, [_vp, _ci, _vp, _vp, _vp]),
+    "dlm_moe_max_tiles": (_ci, [_ci] * 3),
+    "dlm_moe_plan": (_ci, [_vp] + [_ci] * 3 + [_vp] * 3),
+    "dlm_gemm_tile_rows": (_ci, [_ci] * 3),
+    "dlm_gemm": (_ci, [_ci, _vp, _vp]),
+    "dlm_embed_rows": (_ci, [_ci, _vp, _vp, _cf, _vp, _vp, _ci, _ci, _vp]),
+    "dlm_residual_norm_rows": (_ci, [_ci, _vp, _vp, _vp, _ci, _vp, _cf, _ci, _vp, _ci, _ci, _vp]),
+    "dlm_norm_rows": (_ci, [_ci, _vp, _vp, _vp, _cf, _ci, _vp, _ci, _ci, _vp]),
+    "dlm_latent_decode_supported": (_ci, [_ci, _vp]),
+    "dlm_latent_prefill_supported": (_ci, [_ci, _vp]),
+    "dlm_latent_prepare": (_ci, [_ci, _vp, _vp, _vp]),
+    "dlm_latent_prefill": (_ci, [_ci, _vp, _vp, _vp, _i64, _vp, _vp, _i64, _vp]),
+    "dlm_latent_absorb": (_ci, [_ci] + [_vp] * 5),
+    "dlm_latent_decode": (_ci, [_ci, _vp, _vp, _vp, _ci, _vp, _vp, _vp]),
+    "dlm_latent_combine": (_ci, [_ci, _vp, _vp, _ci] + [_vp] * 5 + [_i64, _vp]),
+}
+
+
 class LibraryNotBuiltError(RuntimeError):
     pass
 
@@ -85,16 +141,58 @@ class LibraryNotBuiltError(RuntimeError):
 class W4A16Error(RuntimeError):
     """A C-ABI call returned a negative code."""
 
+    library = "w4a16"
+
     def __init__(self, code, message):
-        super().__init__(f"w4a16 error {code}: {message}")
+        super().__init__(f"{self.library} error {code}: {message}")
         self.code = code
 
 
+class DenseLmError(W4A16Error):
+    """The same from libdense_lm_hip.so."""
+
+    library = "dense_lm"
+
+
 _lib = None
+_dense = None
 
 
 def library_path():
     return _LIB_PATH
+
+
+def _bind(path, symbols):
+    lib = ctypes.CDLL(path)
+    for name, (restype, argtypes) in symbols.items():
+        fn = getattr(lib, name)
+        fn.restype = restype
+        fn.argtypes = argtypes
+    return lib
+
+
+def load_dense_library():
+    """Load the library of the dense-weight models; raises LibraryNotBuiltError when it is missing."""
+    global _dense
+    if _dense is None:
+        if not os.path.exists(_DENSE_PATH):
+            raise LibraryNotBuiltError(f"{_DENSE_PATH} is missing: build it with `python mlir-air_amd/build.py --only dense_lm` "
+                                       "(there is no CPU fallback)")
+        lib = _bind(_DENSE_PATH, DENSE_SYMBOLS)
+        if lib.dlm_abi_version() != 1:
+            raise LibraryNotBuiltError(f"{_DENSE_PATH}: ABI version {lib.dlm_abi_version()} != 1, rebuild")
+        _dense = lib
+    return _dense
+
+
+def check_dense(code):
+    """Raise DenseLmError for a negative return code of a dlm_ call."""
+    if code != OK:
+        lib = load_dense_library()
+        msg = lib.dlm_strerror(code).decode()
+        if code == ERR_HIP:
+            msg += ": " + lib.dlm_last_hip_error().decode()
+        raise DenseLmError(code, msg)
 
 
 def load_library():
@@ -107,11 +205,7 @@ def load_library():
             f"{_LIB_PATH} is missing: build it with `python mlir-air_amd/build.py` "
             "(there is no CPU fallback for the W4A16 kernels)"
         )
-    lib = ctypes.CDLL(_LIB_PATH)
-    for name, (restype, argtypes) in SYMBOLS.items():
-        fn = getattr(lib, name)
-        fn.restype = restype
-        fn.argtypes = argtypes
+    lib = _bind(_LIB_PATH, SYMBOLS)
     if lib.w4a16_abi_version() != 1:
         raise LibraryNotBuiltError(f"{_LIB_PATH}: ABI version {lib.w4a16_abi_version()} != 1, rebuild")
     _lib = lib

@@ -16,7 +16,7 @@ import dataclasses
 import numpy as np
 import torch
 
-from . import ops, weights as wmod
+from . import generation, ops, weights as wmod
 
 
 def generate_rope_lut(config, seq_len=2048, device="cuda"):
@@ -234,32 +234,81 @@ def generate(prompt_tokens, layers, embed_table, final_norm, lm_head, config, ro
     Without `on_token` the whole decode loop runs on the device (decode_greedy) and the ids come back once; tokens
     after an end-of-sequence id are computed and dropped.  With `on_token(token_id)` every token is brought to the
     host as it is produced (the reference's streaming mode) and the loop stops at an end-of-sequence id."""
-    seq_len = len(prompt_tokens)
-    max_seq = seq_len + n_tokens
-    if rope_lut.shape[0] < max_seq:
-        raise ValueError(f"the RoPE table has {rope_lut.shape[0]} rows, the run needs {max_seq}")
-    kv_cache = new_kv_cache(config, max_seq, device=embed_table.device)
-    ids = torch.as_tensor(list(prompt_tokens), dtype=torch.int32, device=embed_table.device)
-    _, first = prefill(ids, layers, embed_table, final_norm, lm_head, config, kv_cache, rope_lut)
-    eos = set(int(t) for t in eos_token_ids)
-    if on_token is None:
-        rest = decode_greedy(first, n_tokens, layers, embed_table, final_norm, lm_head, config, kv_cache, seq_len, rope_lut)
-        ops.check_health()
-        out = [int(first.item())] + [int(t) for t in rest.cpu().tolist()]
-        for i in range(1, len(out)):
-            if out[i] in eos:
-                return out[:i + 1]
+    model = LlamaModel(config, layers, embed_table, final_norm, lm_head, rope_lut)
+    return generation.generate(model, prompt_tokens, n_tokens, eos_token_ids, on_token)
+
+
+class LlamaCache:
+    """KV caches of one sequence and its length."""
+
+    def __init__(self, config, capacity, device):
+        self.kv = new_kv_cache(config, capacity, device)
+        self.capacity, self.pos = capacity, 0
+
+    def reset(self):
+        self.pos = 0
+
+
+class LlamaModel(generation.CausalLM):
+    """The int4 Llama behind the interface of the token loop (generation.CausalLM)."""
+
+    def __init__(self, config, layers, embed_table, final_norm, lm_head, rope_lut=None):
+        self.config, self.layers, self.embed_table, self.final_norm, self.lm_head = config, layers, embed_table, final_norm, lm_head
+        self.rope_lut = rope_lut
+        self.vocab, self.device = config.vocab_size, embed_table.device
+
+    @classmethod
+    def load(cls, path, config_json, dtype=torch.bfloat16, device="cuda"):
+        """An AutoAWQ checkpoint directory."""
+        if dtype != torch.bfloat16:
+            raise generation.UnsupportedDtype("the int4 Llama kernels compute in bfloat16 with fp32 accumulation only")
+        config = wmod.LlamaConfig.from_hf(config_json)
+        host = wmod.load_weights_awq(path, config)
+
+        def dev(bits):
+            return torch.from_numpy(np.ascontiguousarray(bits).view(np.int16)).to(device).view(torch.bfloat16)
+
+        embed = dev(host.embed_table)
+        head = embed if host.lm_head is host.embed_table else dev(host.lm_head)
+        return cls(config, [prepare_layer(l, device) for l in host.layers], embed, dev(host.final_norm), head)
+
+    def new_cache(self, max_tokens):
+        if self.rope_lut is None:
+            self.rope_lut = generate_rope_lut(self.config, max_tokens, self.device)
+        elif self.rope_lut.shape[0] < max_tokens:
+            raise ValueError(f"the RoPE table has {self.rope_lut.shape[0]} rows, the run needs {max_tokens}")
+        return LlamaCache(self.config, max_tokens, self.device)
+
+    def prefill(self, cache, tokens):
+        ids = torch.as_tensor(list(tokens), dtype=torch.int32, device=self.device)
+        logits, best = prefill(ids, self.layers, self.embed_table, self.final_norm, self.lm_head, self.config, cache.kv, self.rope_lut)
+        cache.pos = len(tokens)
+        return logits, best
+
+    def decode_token(self, cache, token):
+        out = decode_token(token, self.layers, self.embed_table, self.final_norm, self.lm_head, self.config, cache.kv, cache.pos, self.rope_lut,
+                           return_argmax=True)
+        cache.pos += 1
         return out
-    tok = int(first.item())
-    out = [tok]
-    on_token(tok)
-    for i in range(n_tokens):
-        _, best = decode_token(tok, layers, embed_table, final_norm, lm_head, config, kv_cache, seq_len + i, rope_lut,
-                               return_argmax=True)
+
+    def decode_greedy(self, cache, first, n_tokens):
+        out = decode_greedy(first, n_tokens, self.layers, self.embed_table, self.final_norm, self.lm_head, self.config, cache.kv, cache.pos,
+                            self.rope_lut)
+        cache.pos += n_tokens
+        return out
+
+    def step(self, cache, tokens, want):
+        """The prompt pass starts at position 0 and gives the last position's logits; any other portion goes token by
+        token."""
+        if cache.pos == 0 and len(tokens) > 1 and all(w == len(tokens) - 1 for w in want):
+            logits, _ = self.prefill(cache, tokens)
+            return logits.reshape(1, -1).expand(len(want), -1)
+        rows = {}
+        for i, t in enumerate(tokens):
+            logits, _ = self.decode_token(cache, int(t))
+            if i in want:
+                rows[i] = logits
+        return torch.stack([rows[w] for w in want]) if want else torch.empty((0, self.vocab), device=self.device)
+
+    def check_health(self):
         ops.check_health()
-        tok = int(best.item())
-        out.append(tok)
-        on_token(tok)
-        if tok in eos:
-            break
-    return out

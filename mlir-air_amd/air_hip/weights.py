@@ -44,6 +44,14 @@ class LlamaConfig:
     def kv_dim(self):
         return self.n_kv_heads * self.head_dim
 
+    @classmethod
+    def from_hf(cls, c):
+        """From the parsed config.json of a HuggingFace Llama checkpoint."""
+        heads, emb = c["num_attention_heads"], c["hidden_size"]
+        return cls(n_layers=c["num_hidden_layers"], emb_dim=emb, n_heads=heads, head_dim=c.get("head_dim") or emb // heads,
+                   n_kv_heads=c.get("num_key_value_heads") or heads, hidden_dim=c["intermediate_size"], vocab_size=c["vocab_size"],
+                   rope_base=float(c.get("rope_theta", 10000.0)), rms_eps=float(c.get("rms_norm_eps", 1e-6)))
+
 
 # HF AutoAWQ Linear suffix -> field name (llama32_1b_int4_weights.py:58-66)
 HF_AWQ_LINEARS = {
@@ -116,25 +124,39 @@ def check_linear(name, qweight, qzeros, scales, group_size):
                          f"are not an AutoAWQ gemm linear with group size {group_size}")
 
 
+class SafetensorsDir:
+    """Tensors of a local checkpoint directory by name, whichever shard holds them."""
+
+    def __init__(self, path):
+        from safetensors import safe_open
+
+        self._open = safe_open
+        self.files = resolve_safetensor_files(path)
+        self._shard_of = {}   # tensor name -> the shard that holds it
+        for file in self.files:
+            with safe_open(file, framework="pt") as f:
+                self._shard_of.update((key, file) for key in f.keys())
+
+    def __contains__(self, key):
+        return key in self._shard_of
+
+    def tensor(self, key, what="weight", hint=""):
+        path = self._shard_of.get(key)
+        if path is None:
+            raise KeyError(f"{what} {key} is in none of the {len(self.files)} safetensors shard(s){hint}")
+        with self._open(path, framework="pt") as f:
+            return f.get_tensor(key)
+
+
 def load_weights_awq(model_name_or_path, config: Optional[LlamaConfig] = None, group_size=awq.GROUP) -> LlamaWeights:
     """Load a local HuggingFace AutoAWQ Llama checkpoint."""
-    from safetensors import safe_open
-
     if config is None:
         config = LlamaConfig()
-    files = resolve_safetensor_files(model_name_or_path)
-    shard_of = {}   # tensor name -> the shard that holds it
-    for path in files:
-        with safe_open(path, framework="pt") as f:
-            shard_of.update((key, path) for key in f.keys())
+    shards = SafetensorsDir(model_name_or_path)
 
     def tensor(key, what="weight"):
-        path = shard_of.get(key)
-        if path is None:
-            hint = "; the directory holds no qweight / qzeros / scales triple under that name, so it was not written by AutoAWQ" if what == "AWQ tensor" else ""
-            raise KeyError(f"{what} {key} is in none of the {len(files)} safetensors shard(s){hint}")
-        with safe_open(path, framework="pt") as f:
-            return f.get_tensor(key)
+        hint = "; the directory holds no qweight / qzeros / scales triple under that name, so it was not written by AutoAWQ" if what == "AWQ tensor" else ""
+        return shards.tensor(key, what, hint)
 
     embed_table = _bf16_bits(tensor("model.embed_tokens.weight"))
     if embed_table.shape != (config.vocab_size, config.emb_dim):
@@ -164,7 +186,7 @@ def load_weights_awq(model_name_or_path, config: Optional[LlamaConfig] = None, g
         layers.append(LayerWeights(**fields))
 
     final_norm = _bf16_bits(tensor("model.norm.weight"))
-    lm_head = _bf16_bits(tensor("lm_head.weight")) if "lm_head.weight" in shard_of else embed_table
+    lm_head = _bf16_bits(tensor("lm_head.weight")) if "lm_head.weight" in shards else embed_table
     return LlamaWeights(embed_table=embed_table, layers=layers, final_norm=final_norm, lm_head=lm_head)
 
 

@@ -1,12 +1,16 @@
-"""Build libw4a16_hip.so (gfx950) in-tree with hipcc.
+"""Build the HIP libraries (gfx950) in-tree with hipcc.
 
-    python mlir-air_amd/build.py [-j JOBS]
+    python mlir-air_amd/build.py [-j JOBS] [--only NAME ...]
 
-Output: mlir-air_amd/lib/libw4a16_hip.so.  Cross-compiles without a GPU.
+Output: mlir-air_amd/lib/libw4a16_hip.so (int4 weights) and mlir-air_amd/lib/libdense_lm_hip.so (dense weights).  Each
+stands alone, so a program that serves one kind of model builds only what it needs (`ensure`).  Cross-compiles without a
+GPU.
 """
 
 import argparse
 import concurrent.futures
+import contextlib
+import fcntl
 import os
 import subprocess
 import sys
@@ -15,8 +19,18 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 OBJ_DIR = os.path.join(HERE, "build")
 LIB_DIR = os.path.join(HERE, "lib")
-LIB_PATH = os.path.join(LIB_DIR, "libw4a16_hip.so")
-SOURCES = ["capi.hip", "dequant.hip", "stream.hip", "gemv_ws.hip", "gemm_ws.hip", "gemm_wsk.hip", "gemm.hip", "attention.hip", "q4nx.hip", "lm_head.hip", "prefill_block.hip", "prefill_attention.hip"]
+LIBRARIES = {
+    "w4a16": ["capi.hip", "dequant.hip", "stream.hip", "gemv_ws.hip", "gemm_ws.hip", "gemm_wsk.hip", "gemm.hip", "attention.hip", "q4nx.hip", "lm_head.hip", "prefill_block.hip", "prefill_attention.hip"],
+    "dense_lm": ["dense_capi.hip", "dense_gemv.hip", "dense_gemm.hip", "rows.hip", "moe.hip", "latent_attention.hip", "latent_prefill.hip"],
+}
+SOURCES = [s for sources in LIBRARIES.values() for s in sources]
+
+
+def lib_path(name):
+    return os.path.join(LIB_DIR, f"lib{name}_hip.so")
+
+
+LIB_PATH = lib_path("w4a16")
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = [
@@ -35,9 +49,9 @@ FLAGS = [
 ]
 
 
-# Per-file flags.  The prompt-pass attention takes maxima over MFMA results: without the promise that they are not
+# Per-file flags.  The prompt-pass attentions take maxima over MFMA results: without the promise that they are not
 # NaN the compiler canonicalises every one of them first (one more VALU instruction per score).
-FILE_FLAGS = {"prefill_attention.hip": ["-fno-honor-nans"]}
+FILE_FLAGS = {"prefill_attention.hip": ["-fno-honor-nans"], "latent_prefill.hip": ["-fno-honor-nans"]}
 
 
 def _compile(src, extra):
@@ -53,24 +67,48 @@ def _compile(src, extra):
     return obj, out
 
 
-def build(jobs=4, extra=(), verbose=False):
+def build(jobs=4, extra=(), verbose=False, only=None):
+    """Compile and link the libraries named in `only` (default: all); returns the path of the last one."""
+    names = list(only or LIBRARIES)
     os.makedirs(OBJ_DIR, exist_ok=True)
     os.makedirs(LIB_DIR, exist_ok=True)
+    sources = [s for name in names for s in LIBRARIES[name]]
     with concurrent.futures.ThreadPoolExecutor(max_workers=jobs) as pool:
-        results = list(pool.map(lambda s: _compile(s, list(extra)), SOURCES))
-    for _, out in results:
+        results = dict(zip(sources, pool.map(lambda s: _compile(s, list(extra)), sources)))
+    for _, out in results.values():
         if out.strip() and verbose:
             print(out)
-    objs = [o for o, _ in results]
-    subprocess.check_call([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_PATH, *objs])
-    return LIB_PATH
+    for name in names:
+        objs = [results[s][0] for s in LIBRARIES[name]]
+        tmp = f"{lib_path(name)}.{os.getpid()}"   # renamed when whole: nobody loads half a library
+        subprocess.check_call([HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", tmp, *objs])
+        os.replace(tmp, lib_path(name))
+    return lib_path(names[-1])
+
+
+@contextlib.contextmanager
+def _lock():
+    os.makedirs(OBJ_DIR, exist_ok=True)
+    with open(os.path.join(OBJ_DIR, ".lock"), "w") as f:
+        fcntl.flock(f, fcntl.LOCK_EX)
+        yield
+
+
+def ensure(name, jobs=8):
+    """The library `name`, built first if there is none (one builder at a time)."""
+    if not os.path.exists(lib_path(name)):
+        with _lock():
+            if not os.path.exists(lib_path(name)):
+                build(jobs, only=[name])
+    return lib_path(name)
 
 
 if __name__ == "__main__":
     ap = argparse.ArgumentParser()
     ap.add_argument("-j", type=int, default=4)
     ap.add_argument("-v", action="store_true")
+    ap.add_argument("--only", nargs="*", choices=list(LIBRARIES), help="build these libraries only")
     ap.add_argument("--save-temps", action="store_true", help="keep ISA (.s) files under build/")
     a = ap.parse_args()
     extra = ["-save-temps=obj"] if a.save_temps else []
-    print(build(a.j, extra, a.v or True))
+    print(build(a.j, extra, a.v or True, a.only))

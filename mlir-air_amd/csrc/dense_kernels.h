@@ -1,0 +1,124 @@
+// Internal launch interface between the C ABI of the dense-weight library (dense_capi.hip) and its kernel files.
+// dtype: 0 = bf16, 1 = float, of weights and activations (`void *`); residual, norms, router logits are always fp32.
+#pragma once
+
+#include <hip/hip_runtime.h>
+#include <stddef.h>
+#include <stdint.h>
+
+namespace w4a16 {
+
+enum : int { kBf16 = 0, kF32 = 1 };
+inline size_t elem_bytes(int dtype) { return dtype == kF32 ? 4 : 2; }
+
+// What a one-token product reads as its input vector.
+enum : int {
+    kIntakePlain = 0,      // x
+    kIntakeResidual = 1,   // res + y / rms(y) * norm_w, also left in res_out (and h_out)
+    kIntakeEmbed = 2,      // embed[*token] * scale, also left in res_out (and h_out)
+    kIntakeFinal = 3,      // the norm final_w of (res + y / rms(y) * norm_w), or of res without y
+};
+struct RowIntake {
+    int mode = kIntakePlain;
+    const void *x = nullptr;
+    const float *res = nullptr, *y = nullptr, *norm_w = nullptr, *final_w = nullptr;
+    float eps = 0.f;
+    int width = 0;         // elements that count in the mean (the rest of K is zero padding)
+    float *res_out = nullptr;
+    void *h_out = nullptr;
+    const void *embed = nullptr;
+    const int32_t *token = nullptr;
+    float scale = 1.f;
+};
+// y[N] = W[N, K] x[K]; out in the element type, or fp32 in out_f32.  keys (4 per workgroup): argmax keys of the
+// first n_valid rows.
+hipError_t launch_dense_gemv(int dtype, const void *w, const RowIntake &in, void *out, float *out_f32, unsigned long long *keys,
+                             int n_valid, int K, int N, hipStream_t stream);
+int dense_gemv_blocks(int K, int N);   // workgroups of that launch; it writes four keys per workgroup
+// token[0] = argmax from the keys; position[0] += 1; history[position] = token (each optional)
+hipError_t launch_argmax_keys(const unsigned long long *keys, int n, int32_t *token, int32_t *position, int32_t *history,
+                              hipStream_t stream);
+
+// Experts of one token or of many.
+struct Router {
+    const float *logits = nullptr;      // [tokens, ld]
+    const float *correction = nullptr;  // [experts]
+    int ld = 0, experts = 0, top = 0, groups = 1, keep = 1;
+};
+constexpr int kMaxExperts = 1024, kMaxTop = 32;
+// one token: h[top, ff] = silu(gate x) * (up x) of the chosen experts; ids and weights of the choice are left for the
+// second product, y[width] = sum_s weight_s down_s h_s
+hipError_t launch_moe_gate_up_gemv(int dtype, const Router &r, const void *x, const void *w_gate_up, void *h, int32_t *ids, float *weights,
+                                   int K, int ff, hipStream_t stream);
+hipError_t launch_moe_down_gemv(int dtype, const void *h, const void *w_down, const int32_t *ids, const float *weights, float *y, int top,
+                                int ff, int N, hipStream_t stream);
+// many tokens
+hipError_t launch_moe_select(const Router &r, int tokens, int32_t *ids, float *weights, hipStream_t stream);
+// entries (token * top + slot) sorted by expert, and the row tiles of `bm` entries that the grouped product runs over:
+// tiles[i] = {expert (-1: none), first sorted entry, entries, 0}
+int moe_max_tiles(int entries, int experts, int bm);
+hipError_t launch_moe_plan(const int32_t *ids, int entries, int experts, int bm, int32_t *order, int32_t *tiles, hipStream_t stream);
+
+// Products over many rows: out[M, N] = A[M, K] W[N, K]^T.
+enum : int { kOutElem = 0, kOutF32 = 1, kOutSwiglu = 2 };   // swiglu: W holds 16 gate rows, 16 up rows, ...; out is [M, N / 2]
+struct GemmArgs {
+    const void *a = nullptr, *w = nullptr;
+    void *out = nullptr;
+    int M = 0, N = 0, K = 0;
+    long lda = 0, ldo = 0;
+    int epilogue = kOutElem;
+    // grouped (experts): rows are sorted entries, tiles from launch_moe_plan
+    const int32_t *tiles = nullptr, *order = nullptr;
+    int n_tiles = 0;       // tiles in the table
+    int gather = 0;        // > 0: A row of an entry = entry / gather, out row = sorted place; 0: A row = sorted place, out row = entry
+    long w_stride = 0;     // elements from one expert's W to the next
+};
+int dense_gemm_tile_rows(int dtype, int rows, int N);   // rows of the tile the launch will use (what launch_moe_plan gets as bm)
+hipError_t launch_dense_gemm(int dtype, const GemmArgs &g, int tile_rows, hipStream_t stream);
+
+hipError_t launch_embed_rows(int dtype, const int32_t *tokens, const void *embed, float scale, float *res, void *h, int M, int width,
+                             hipStream_t stream);
+// res += y / rms(y) * norm_w per row; h = res in the element type.  With weights (experts): y is [M * top, width] in the
+// element type and the row is sum_s weights[m, s] y[m * top + s]; otherwise y is fp32 [M, width].
+hipError_t launch_residual_norm_rows(int dtype, float *res, const void *y, const float *weights, int top, const float *norm_w, float eps,
+                                     int true_width, void *h, int M, int width, hipStream_t stream);
+// out[i] = norm of res[rows[i]] (rows nullptr: i)
+hipError_t launch_norm_rows(int dtype, const float *res, const int32_t *rows, const float *norm_w, float eps, int true_width, void *out, int n,
+                            int width, hipStream_t stream);
+
+// Latent attention.  Sizes are the padded ones; a cache row is [latent kv_rank | rotated key part rot].
+struct LatentShape {
+    int heads, dim, rot, vdim, rank;    // padded sizes (dim, rot, vdim multiples of 32, rank of 64)
+    int rot_pairs;                      // pairs that are rotated (true rot / 2)
+    int true_rank;                      // elements in the mean of the latent's norm
+    float scale;
+};
+struct LatentRows {
+    const void *proj = nullptr;         // [M, ld]: q per head [dim | rot], then (with_kv) latent | key part, then the gate
+    long ld = 0;
+    int kv_off = -1;                    // column of the latent, -1: the layer has none
+    int gate_off = 0;
+    const float *lut = nullptr;         // [positions, rot_pairs, 2]: cos, sin
+    const float *kv_norm = nullptr;
+    float eps = 0.f;
+    void *cache = nullptr;              // [rows, rank + rot]
+    int M = 0;
+    const int32_t *pos_dev = nullptr;   // position of the first row, on the device ...
+    int pos = 0;                        // ... or here
+};
+// rotates q in place and appends the cache rows
+hipError_t launch_latent_prepare(int dtype, const LatentShape &s, const LatentRows &r, hipStream_t stream);
+// appends the cache rows and writes the queries against the latent: qa[M * heads, rank + rot]
+hipError_t launch_latent_absorb(int dtype, const LatentShape &s, const LatentRows &r, const void *w_uk, void *qa, hipStream_t stream);
+// attention of qa over the cache, split along the keys; then merge, value projection and gate: out[M, ldo]
+hipError_t launch_latent_decode(int dtype, const LatentShape &s, const LatentRows &r, const void *qa, int nsplit, float *part_o, float *part_ml,
+                                hipStream_t stream);
+hipError_t launch_latent_combine(int dtype, const LatentShape &s, const LatentRows &r, int nsplit, const float *part_o, const float *part_ml,
+                                 const float *sink, const void *w_uv, void *out, long ldo, hipStream_t stream);
+bool latent_decode_supported(int dtype, const LatentShape &s);
+// causal attention on per-head keys and values kv[T, ldkv] (keys of all heads, then values of all heads)
+hipError_t launch_latent_prefill(int dtype, const LatentShape &s, const LatentRows &r, const void *kv, long ldkv, const float *sink, void *out,
+                                 long ldo, hipStream_t stream);
+bool latent_prefill_supported(int dtype, const LatentShape &s);
+
+}  // namespace w4a16

@@ -1,0 +1,439 @@
+// Latent attention over the cache for gfx950: the cache holds, per token, one normed latent (rank) and one rotated key part
+// (rot) shared by all heads; keys and values of a head are linear in the latent.
+//
+//   latent_prepare   rotates the queries of many rows in place and appends their cache rows (long portions; keys and values
+//                    are then expanded per head and latent_prefill.hip attends)
+//   latent_absorb    appends the cache rows and moves the key projection to the query side: qa = W_uk^T q_unrotated per head,
+//                    followed by the rotated part, so that a score is one product of length rank + rot with a cache row
+//   latent_decode    attention of all rows and heads over the cached rows: HBM-bound on the cache, which is read once per
+//                    16 (row, head) pairs; both products on MFMA, keys split over workgroups
+//   latent_combine   merges the splits with the sink, applies the value projection of the head to the merged latent and the
+//                    output gate
+//
+// Positions count from `pos`, which may lie on the device (a captured decode step advances it there).
+#include "dense.h"
+#include "dense_kernels.h"
+
+namespace w4a16 {
+
+namespace {
+
+constexpr int kLatThreads = 256;
+
+template <class T>
+struct LatentArgs {
+    LatentShape s;
+    const T *proj;
+    long ld;
+    int kv_off, gate_off;
+    const float *lut, *kv_norm;
+    float eps;
+    T *cache;
+    int M;
+    const int32_t *pos_dev;
+    int pos;
+};
+
+template <class T>
+__device__ __forceinline__ int first_position(const LatentArgs<T> &p) { return p.pos_dev ? p.pos_dev[0] : p.pos; }
+
+// neighbouring pairs rotated: (u, v) -> (u cos - v sin, v cos + u sin)
+template <class T>
+__device__ __forceinline__ void rotate_pair(const T *src, T *dst, const float *lut) {
+    const float u = to_float(src[0]), v = to_float(src[1]), c = lut[0], s = lut[1];
+    dst[0] = from_float<T>(u * c - v * s);
+    dst[1] = from_float<T>(v * c + u * s);
+}
+
+// The cache row of token m: by one workgroup.  Padding columns of the projections are zeros and stay zeros.
+template <class T>
+__device__ __forceinline__ void append_row(const LatentArgs<T> &p, int m, int position, float *red) {
+    const T *src = p.proj + (size_t)m * p.ld + p.kv_off;
+    T *dst = p.cache + (size_t)position * (p.s.rank + p.s.rot);
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < p.s.rank; i += kLatThreads) {
+        const float v = to_float(src[i]);
+        ss = fmaf(v, v, ss);
+    }
+    ss = wave_reduce<false>(ss);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+    __syncthreads();
+    const float rstd = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)p.s.true_rank + p.eps);
+    for (int i = threadIdx.x; i < p.s.rank; i += kLatThreads) dst[i] = from_float<T>(to_float(src[i]) * rstd * p.kv_norm[i]);
+    for (int i = threadIdx.x; i < p.s.rot / 2; i += kLatThreads) {
+        T *d = dst + p.s.rank + 2 * i;
+        if (i < p.s.rot_pairs) rotate_pair(src + p.s.rank + 2 * i, d, p.lut + ((size_t)position * p.s.rot_pairs + i) * 2);
+        else d[0] = d[1] = from_float<T>(0.f);
+    }
+}
+
+// one workgroup per token
+template <class T>
+__global__ void __launch_bounds__(kLatThreads) latent_prepare_kernel(const LatentArgs<T> p) {
+    __shared__ float red[4];
+    const int m = blockIdx.x, position = first_position(p) + m;
+    const int n = p.s.heads * p.s.rot_pairs, qd = p.s.dim + p.s.rot;
+    T *q = const_cast<T *>(p.proj) + (size_t)m * p.ld;
+    for (int i = threadIdx.x; i < n; i += kLatThreads) {
+        const int h = i / p.s.rot_pairs, j = i % p.s.rot_pairs;
+        T *v = q + h * qd + p.s.dim + 2 * j;
+        rotate_pair(v, v, p.lut + ((size_t)position * p.s.rot_pairs + j) * 2);
+    }
+    if (p.kv_off >= 0) append_row(p, m, position, red);
+}
+
+// blockIdx.y = token; blockIdx.x = head * blocks of 128 latent columns, then (with a latent of its own) the cache row
+template <class T>
+__global__ void __launch_bounds__(kLatThreads) latent_absorb_kernel(const LatentArgs<T> p, const T *w_uk, T *qa, int rank_blocks) {
+    __shared__ float part[16][128 + 4];
+    __shared__ float red[4];
+    __shared__ float qs[1024];
+    const int m = blockIdx.y, position = first_position(p) + m, tid = threadIdx.x;
+    if ((int)blockIdx.x == p.s.heads * rank_blocks) {
+        append_row(p, m, position, red);
+        return;
+    }
+    const int h = blockIdx.x / rank_blocks, r0 = (blockIdx.x % rank_blocks) * 128;
+    const int qd = p.s.dim + p.s.rot, lq = p.s.rank + p.s.rot;
+    const T *q = p.proj + (size_t)m * p.ld + h * qd;
+    T *out = qa + ((size_t)m * p.s.heads + h) * lq;
+    const int col = r0 + 8 * (tid & 15), dg = tid >> 4;
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int i = tid; i < p.s.dim; i += kLatThreads) qs[i] = to_float(q[i]);
+    __syncthreads();
+    if (col < p.s.rank) {
+        const T *w = w_uk + ((size_t)h * p.s.dim + dg) * p.s.rank + col;
+        for (int d = dg; d < p.s.dim; d += 64) {       // dim is a multiple of 32: two or four rows at a time
+            Vec8<T> v[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = d + 16 * j < p.s.dim ? load8(w + (size_t)(d - dg + 16 * j) * p.s.rank) : zero8<T>();
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                float f[8];
+                unpack8(v[j], f);
+                const float x = d + 16 * j < p.s.dim ? qs[d + 16 * j] : 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) acc[e] = fmaf(x, f[e], acc[e]);
+            }
+        }
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) part[dg][8 * (tid & 15) + e] = acc[e];
+    __syncthreads();
+    if (tid < 128 && r0 + tid < p.s.rank) {
+        float s = 0.f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) s += part[i][tid];
+        out[r0 + tid] = from_float<T>(s);
+    }
+    if (r0 == 0) {
+        for (int i = tid; i < p.s.rot / 2; i += kLatThreads) {
+            T *d = out + p.s.rank + 2 * i;
+            if (i < p.s.rot_pairs) rotate_pair(q + p.s.dim + 2 * i, d, p.lut + ((size_t)position * p.s.rot_pairs + i) * 2);
+            else d[0] = d[1] = from_float<T>(0.f);
+        }
+    }
+}
+
+// Keys of one split of the cached rows, in whole blocks: the same split is found by latent_decode and latent_combine.
+__host__ __device__ __forceinline__ int keys_per_split(int total, int nsplit, int kb) {
+    const int blocks = (total + kb - 1) / kb;
+    return (blocks + nsplit - 1) / nsplit * kb;
+}
+
+// blockIdx.x = split, blockIdx.y = 16 rows (row = token * heads + head).  CT: 16-column tiles of the latent per wave.
+template <class T, int KB, int CT>
+__global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const LatentArgs<T> p, const T *qa, int nsplit, float *part_o, float *part_ml) {
+    extern __shared__ __attribute__((aligned(16))) char latent_lds[];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int ql = lane & 15, g = lane >> 4;
+    const int lq = p.s.rank + p.s.rot, pitch = lq + 16 / (int)sizeof(T), rows = p.M * p.s.heads, row0 = blockIdx.y * 16;
+    constexpr int SP = KB + 4, PP = KB + 8;       // pitches of the scores and of the probabilities
+    T *tile = reinterpret_cast<T *>(latent_lds);  // [KB][pitch]
+    T *qt = tile + KB * pitch;                    // [16][pitch]
+    T *pt = qt + 16 * pitch;                      // [16][PP]
+    float *st = reinterpret_cast<float *>(pt + 16 * PP);   // [16][SP]
+    float *al = st + 16 * SP;                     // [16] rescaling factors of the block
+
+    const int pos0 = first_position(p), total = pos0 + p.M;
+    const int per = keys_per_split(total, nsplit, KB);
+    const int k0 = blockIdx.x * per;
+    const int last_row = row0 + 15 < rows ? row0 + 15 : rows - 1;
+    const int seen = pos0 + last_row / p.s.heads + 1;          // keys that any of these rows sees
+    const int k1 = k0 + per < seen ? k0 + per : seen;
+
+    const int chunks = lq / 8;
+    for (int c = tid; c < 16 * chunks; c += kLatThreads) {
+        const int r = c / chunks, e = 8 * (c % chunks);
+        const int row = row0 + r < rows ? row0 + r : rows - 1;
+        store8(qt + r * pitch + e, load8(qa + (size_t)row * lq + e));
+    }
+    // softmax threads: row tid / 16, keys (tid % 16) + 16 j of a block
+    const int srow = tid >> 4, skey = tid & 15;
+    const int row_of_mine = row0 + srow < rows ? row0 + srow : rows - 1;
+    const int my_limit = pos0 + row_of_mine / p.s.heads;       // last visible key
+    float m = kAttnNegBig, l = 0.f;
+    floatx4 o[CT];
+#pragma unroll
+    for (int c = 0; c < CT; ++c) o[c] = floatx4{0.f, 0.f, 0.f, 0.f};
+    const int tiles = p.s.rank / 16;
+    const float scale2 = p.s.scale * 1.4426950408889634f;
+
+    for (int kb = k0; kb < k1; kb += KB) {
+        for (int c = tid; c < KB * chunks; c += kLatThreads) {
+            const int r = c / chunks, e = 8 * (c % chunks);
+            const int key = kb + r < total ? kb + r : total - 1;
+            store8(tile + r * pitch + e, load8(p.cache + (size_t)key * lq + e));
+        }
+        __syncthreads();
+        for (int kt = wave; kt < KB / 16; kt += kLatThreads / 64) {
+            floatx4 s0 = floatx4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
+            const T *a = tile + (16 * kt + ql) * pitch + 8 * g, *b = qt + ql * pitch + 8 * g;
+            int k = 0;
+            for (; k + 64 <= lq; k += 64) {
+                s0 = mma32(load8(a + k), load8(b + k), s0);
+                s1 = mma32(load8(a + k + 32), load8(b + k + 32), s1);
+            }
+            if (k < lq) s0 = mma32(load8(a + k), load8(b + k), s0);
+            s0 += s1;
+            *reinterpret_cast<floatx4 *>(st + ql * SP + 16 * kt + 4 * g) = s0;   // keys 4 g .. of row ql
+        }
+        __syncthreads();
+        {
+            float v[KB / 16];
+            float top = kAttnNegBig;
+#pragma unroll
+            for (int j = 0; j < KB / 16; ++j) {
+                const int key = skey + 16 * j;
+                v[j] = kb + key <= my_limit ? st[srow * SP + key] * scale2 : kAttnNegBig;
+                top = fmaxf(top, v[j]);
+            }
+#pragma unroll
+            for (int d = 1; d < 16; d *= 2) top = fmaxf(top, __shfl_xor(top, d));
+            const float mn = fmaxf(m, top), alpha = exp2f(m - mn);
+            float sum = 0.f;
+#pragma unroll
+            for (int j = 0; j < KB / 16; ++j) {
+                const float e = v[j] > 0.5f * kAttnNegBig ? exp2f(v[j] - mn) : 0.f;
+                sum += e;
+                pt[srow * PP + skey + 16 * j] = from_float<T>(e);
+            }
+            l = l * alpha + row_sum16(sum);
+            m = mn;
+            if (skey == 0) al[srow] = alpha;
+        }
+        __syncthreads();
+        const float alpha = al[ql];
+        Vec8<T> pv[KB / 32];
+#pragma unroll
+        for (int t = 0; t < KB / 32; ++t) {
+            float a[4], b[4];
+            load4(pt + ql * PP + 32 * t + 4 * g, a);
+            load4(pt + ql * PP + 32 * t + 16 + 4 * g, b);
+            pv[t] = pair8<T>(floatx4{a[0], a[1], a[2], a[3]}, floatx4{b[0], b[1], b[2], b[3]});
+        }
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+            const int ct = wave + 4 * c;
+            if (ct < tiles) {
+                o[c] *= alpha;
+#pragma unroll
+                for (int t = 0; t < KB / 32; ++t) o[c] = mma32(column8(tile + 32 * t * pitch, pitch, 16 * ct), pv[t], o[c]);
+            }
+        }
+        __syncthreads();
+    }
+    if (k0 >= total) return;       // (the merge does not look at splits that start behind the last key)
+    if (row0 + ql < rows) {
+        float *dst = part_o + ((size_t)(row0 + ql) * nsplit + blockIdx.x) * p.s.rank + 4 * g;
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+            const int ct = wave + 4 * c;
+            if (ct < tiles) *reinterpret_cast<floatx4 *>(dst + 16 * ct) = o[c];
+        }
+    }
+    if (skey == 0 && row0 + srow < rows) {
+        float *ml = part_ml + ((size_t)(row0 + srow) * nsplit + blockIdx.x) * 2;
+        ml[0] = m;
+        ml[1] = l;
+    }
+}
+
+constexpr int kMaxSplits = 256, kValueRows = 32;
+
+// blockIdx.x = head * blocks of 32 value rows, blockIdx.y = token
+template <class T>
+__global__ void __launch_bounds__(kLatThreads) latent_combine_kernel(const LatentArgs<T> p, int nsplit, int kb, const float *part_o, const float *part_ml,
+                                                                     const float *sink, const T *w_uv, T *out, long ldo, int value_blocks) {
+    __shared__ float f[kMaxSplits];
+    __shared__ float red[8];
+    extern __shared__ __attribute__((aligned(16))) float merged[];   // [rank up to a multiple of 512]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int h = blockIdx.x / value_blocks, v0 = (blockIdx.x % value_blocks) * kValueRows, m = blockIdx.y;
+    const size_t row = (size_t)m * p.s.heads + h;
+    const int total = first_position(p) + p.M, per = keys_per_split(total, nsplit, kb);
+    const int active = (total + per - 1) / per;
+    const int rank = p.s.rank;
+
+    // factors of the splits in the log2 domain; the sink is one more term of the denominator
+    const float snk = sink[h] * 1.4426950408889634f;
+    float ms = kAttnNegBig, ls = 0.f;
+    if (tid < active) {
+        const float *ml = part_ml + (row * nsplit + tid) * 2;
+        ms = ml[0];
+        ls = ml[1];
+    }
+    float top = wave_reduce<true>(ms);
+    if (lane == 0) red[wave] = top;
+    __syncthreads();
+    top = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), snk);
+    const float fac = tid < active ? exp2f(ms - top) : 0.f;
+    const float part = wave_reduce<false>(fac * ls);
+    if (lane == 0) red[4 + wave] = part;
+    __syncthreads();
+    const float inv = 1.0f / (red[4] + red[5] + red[6] + red[7] + exp2f(snk - top));
+    f[tid] = fac * inv;
+    __syncthreads();
+    for (int r = 4 * tid; r < (rank + 511) / 512 * 512; r += 4 * kLatThreads) {
+        floatx4 s = floatx4{0.f, 0.f, 0.f, 0.f};
+        if (r < rank) {
+            const float *src = part_o + row * nsplit * rank + r;
+            for (int i = 0; i < active; ++i) s += *reinterpret_cast<const floatx4 *>(src + (size_t)i * rank) * f[i];
+        }
+        *reinterpret_cast<floatx4 *>(merged + r) = s;
+    }
+    __syncthreads();
+    for (int i = wave; i < kValueRows; i += kLatThreads / 64) {
+        const int v = v0 + i;
+        if (v >= p.s.vdim) break;
+        const T *w = w_uv + ((size_t)h * p.s.vdim + v) * rank;
+        float acc = 0.f;
+        for (int k = 8 * lane; k < rank; k += 512) {
+            float wf[8];
+            unpack8(load8(w + k), wf);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc = fmaf(wf[e], merged[k + e], acc);
+        }
+        acc = wave_reduce<false>(acc);
+        if (lane == 0) {
+            const float gate = to_float(p.proj[(size_t)m * p.ld + p.gate_off + h * p.s.vdim + v]);
+            out[(size_t)m * ldo + h * p.s.vdim + v] = from_float<T>(acc * sigmoid_f32(gate));
+        }
+    }
+}
+
+template <class T>
+LatentArgs<T> args_of(const LatentShape &s, const LatentRows &r) {
+    LatentArgs<T> a;
+    a.s = s;
+    a.proj = static_cast<const T *>(r.proj);
+    a.ld = r.ld;
+    a.kv_off = r.kv_off;
+    a.gate_off = r.gate_off;
+    a.lut = r.lut;
+    a.kv_norm = r.kv_norm;
+    a.eps = r.eps;
+    a.cache = static_cast<T *>(r.cache);
+    a.M = r.M;
+    a.pos_dev = r.pos_dev;
+    a.pos = r.pos;
+    return a;
+}
+
+template <class T>
+size_t decode_lds(const LatentShape &s, int kb) {
+    const size_t pitch = s.rank + s.rot + 16 / sizeof(T);
+    return ((kb + 16) * pitch + 16 * (kb + 8)) * sizeof(T) + (16 * (kb + 4) + 16) * sizeof(float);
+}
+constexpr size_t kLdsLimit = 160 * 1024;
+
+template <class T>
+constexpr int decode_block() { return sizeof(T) == 2 ? 64 : 32; }
+
+// keys per block: fewer where a block of the usual size does not fit in LDS (0: not at all)
+template <class T>
+int decode_kb(const LatentShape &s) {
+    if (s.rank > 1024) return 0;
+    int kb = decode_block<T>();
+    while (kb >= 32 && decode_lds<T>(s, kb) > kLdsLimit) kb /= 2;
+    return kb >= 32 ? kb : 0;
+}
+
+template <class T>
+hipError_t decode(const LatentShape &s, const LatentRows &r, const void *qa, int nsplit, float *part_o, float *part_ml, hipStream_t stream) {
+    const LatentArgs<T> a = args_of<T>(s, r);
+    const int kb = decode_kb<T>(s);
+    const size_t lds = decode_lds<T>(s, kb);
+    const dim3 grid(nsplit, (r.M * s.heads + 15) / 16);
+    auto run = [&](auto kernel) {
+        if (lds > 48 * 1024) {
+            const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            if (e != hipSuccess) return e;
+        }
+        hipLaunchKernelGGL(kernel, grid, dim3(kLatThreads), lds, stream, a, static_cast<const T *>(qa), nsplit, part_o, part_ml);
+        return hipGetLastError();
+    };
+    const int ct = (s.rank / 16 + 3) / 4;
+    if (kb == 64) {
+        if (ct <= 2) return run(&latent_decode_kernel<T, 64, 2>);
+        if (ct <= 4) return run(&latent_decode_kernel<T, 64, 4>);
+        if (ct <= 8) return run(&latent_decode_kernel<T, 64, 8>);
+        return run(&latent_decode_kernel<T, 64, 16>);
+    }
+    if (kb == 32) {
+        if (ct <= 2) return run(&latent_decode_kernel<T, 32, 2>);
+        if (ct <= 4) return run(&latent_decode_kernel<T, 32, 4>);
+        if (ct <= 8) return run(&latent_decode_kernel<T, 32, 8>);
+        return run(&latent_decode_kernel<T, 32, 16>);
+    }
+    return hipErrorInvalidValue;
+}
+
+template <class T>
+hipError_t absorb(const LatentShape &s, const LatentRows &r, const void *w_uk, void *qa, hipStream_t stream) {
+    const int blocks = (s.rank + 127) / 128;
+    const dim3 grid(s.heads * blocks + (r.kv_off >= 0), r.M);
+    hipLaunchKernelGGL(latent_absorb_kernel<T>, grid, dim3(kLatThreads), 0, stream, args_of<T>(s, r), static_cast<const T *>(w_uk), static_cast<T *>(qa),
+                       blocks);
+    return hipGetLastError();
+}
+
+template <class T>
+hipError_t combine(const LatentShape &s, const LatentRows &r, int nsplit, const float *part_o, const float *part_ml, const float *sink, const void *w_uv,
+                   void *out, long ldo, hipStream_t stream) {
+    const int blocks = (s.vdim + kValueRows - 1) / kValueRows;
+    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3(s.heads * blocks, r.M), dim3(kLatThreads), (size_t)(s.rank + 511) / 512 * 512 * sizeof(float),
+                       stream, args_of<T>(s, r), nsplit, decode_kb<T>(s), part_o, part_ml, sink, static_cast<const T *>(w_uv), static_cast<T *>(out), ldo,
+                       blocks);
+    return hipGetLastError();
+}
+
+}  // namespace
+
+bool latent_decode_supported(int dtype, const LatentShape &s) {
+    return s.dim <= 1024 && (dtype == kF32 ? decode_kb<float>(s) : decode_kb<bf16>(s)) != 0;
+}
+
+hipError_t launch_latent_prepare(int dtype, const LatentShape &s, const LatentRows &r, hipStream_t stream) {
+    if (dtype == kF32) hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(r.M), dim3(kLatThreads), 0, stream, args_of<float>(s, r));
+    else hipLaunchKernelGGL(latent_prepare_kernel<bf16>, dim3(r.M), dim3(kLatThreads), 0, stream, args_of<bf16>(s, r));
+    return hipGetLastError();
+}
+
+hipError_t launch_latent_absorb(int dtype, const LatentShape &s, const LatentRows &r, const void *w_uk, void *qa, hipStream_t stream) {
+    return dtype == kF32 ? absorb<float>(s, r, w_uk, qa, stream) : absorb<bf16>(s, r, w_uk, qa, stream);
+}
+
+hipError_t launch_latent_decode(int dtype, const LatentShape &s, const LatentRows &r, const void *qa, int nsplit, float *part_o, float *part_ml,
+                                hipStream_t stream) {
+    return dtype == kF32 ? decode<float>(s, r, qa, nsplit, part_o, part_ml, stream) : decode<bf16>(s, r, qa, nsplit, part_o, part_ml, stream);
+}
+
+hipError_t launch_latent_combine(int dtype, const LatentShape &s, const LatentRows &r, int nsplit, const float *part_o, const float *part_ml,
+                                 const float *sink, const void *w_uv, void *out, long ldo, hipStream_t stream) {
+    return dtype == kF32 ? combine<float>(s, r, nsplit, part_o, part_ml, sink, w_uv, out, ldo, stream)
+                         : combine<bf16>(s, r, nsplit, part_o, part_ml, sink, w_uv, out, ldo, stream);
+}
+
+}  // namespace w4a16
