@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the MI355X W4A16 path.  One JSON line on stdout.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload gemv|probe|gemv_awq|dequant|gemm16|gemm64|gemm64_down|gemm16_awq|prefill|prefill_awq|ffn|ffn_awq|block|block_awq|layer|layer_awq|q4nx_gemv|q4nx_gemm16|q4nx_prefill|lm_head|decode_1b|decode_8b|prefill_block|prefill_block_awq|prefill_1b|prefill_1b_awq|prefill_8b]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload gemv|probe|gemv_awq|dequant|gemm16|gemm64|gemm64_down|gemm16_awq|prefill|prefill_awq|ffn|ffn_awq|block|block_awq|layer|layer_awq|q4nx_gemv|q4nx_gemm16|q4nx_prefill|lm_head|decode_1b|decode_8b|prefill_block|prefill_block_awq|prefill_1b|prefill_1b_awq|prefill_8b|kuvonex]
 
 Default workload is the decode GEMV (x bf16 [1,4096], W int4 [4096 x 11008], group 128).
 A step is one launch of the hot path on synthetic inputs that are already resident in HBM.
@@ -626,6 +626,155 @@ def run_prefill_model(model="decode_1b", M=2048, reps=3, stream_order=True):
             "finite": bool(torch.isfinite(logits).all())}
 
 
+# Kuvonex layers (latent attention, mixture of experts, bf16 weights) beside int4 Llama layers of the same width, layer count,
+# vocabulary and feed-forward length per token (top x ff = hidden_dim).
+KUVONEX_SIZES = {
+    "w2048": dict(width=2048, layers=8, heads=16, dim=128, rot=64, vdim=128, rank=512, experts=64, top=8, groups=8, keep=4, ff=1024, vocab=32768,
+                  llama=dict(n_layers=8, emb_dim=2048, n_heads=32, head_dim=64, n_kv_heads=8, hidden_dim=8192, vocab_size=32768)),
+    "w4096": dict(width=4096, layers=4, heads=32, dim=128, rot=64, vdim=128, rank=512, experts=32, top=8, groups=4, keep=2, ff=1792, vocab=32768,
+                  llama=dict(n_layers=4, emb_dim=4096, n_heads=32, head_dim=128, n_kv_heads=8, hidden_dim=14336, vocab_size=32768)),
+}
+
+
+def random_kuvonex(size, dtype=None):
+    """A random-weight model of KUVONEX_SIZES[size]; every second layer attends over the layer before it."""
+    import torch
+
+    from air_hip import kuvonex
+
+    z = KUVONEX_SIZES[size]
+    mixer = dict(heads=z["heads"], dim=z["dim"], rot_dim=z["rot"], vdim=z["vdim"], kv_rank=z["rank"], scale=(z["dim"] + z["rot"]) ** -0.5,
+                 rot=dict(base=10000.0, dims=z["rot"]))
+    mlp = dict(kind="moe", expert=dict(ff=z["ff"]), router=dict(experts=z["experts"], top=z["top"], groups=dict(count=z["groups"], keep=z["keep"])))
+    layers = [dict(type="latent_attention", mixer=dict(mixer, kv_from=i - 1) if i % 2 else mixer, mlp=mlp) for i in range(z["layers"])]
+    cfg = kuvonex.KuvonexConfig.from_json(dict(vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-6), embedding=dict(scale=1.0), layers=layers))
+    g = torch.Generator(device="cuda")
+    g.manual_seed(7)
+
+    def tensor(name, shape):
+        t = torch.randn(shape, device="cuda", generator=g)
+        if "norm" in name:
+            return 1.0 + 0.1 * t
+        return t.mul_(1.0 if name == "embed" or len(shape) == 1 else shape[-1] ** -0.5).to(torch.bfloat16)
+
+    return kuvonex.KuvonexModel(cfg, tensor, dtype or torch.bfloat16)
+
+
+def random_llama(c, seed=5):
+    """A random-weight int4 Llama (stream-order weights) behind the same interface."""
+    import torch
+
+    from air_hip import decode, weights as wmod
+
+    cfg = wmod.LlamaConfig(**c)
+    E, H, nqkv = cfg.emb_dim, cfg.hidden_dim, (cfg.n_heads + 2 * cfg.n_kv_heads) * cfg.head_dim
+    g = torch.Generator(device="cuda")
+    g.manual_seed(seed)
+
+    def lin(K, N, s):
+        qw, qz, sc = make_weights(torch, K, N, s)
+        return qw, qz, (sc.float() * 0.05).to(torch.bfloat16)
+
+    def norm_w():
+        return (torch.randn((E,), device="cuda", generator=g) * 0.1 + 1.0).to(torch.bfloat16)
+
+    layers = [decode.DecodeLayer(attn_norm=norm_w(), ffn_norm=norm_w(), wqkv=lin(E, nqkv, 10 * i), wo=lin(E, E, 10 * i + 1), w_gate=lin(E, H, 10 * i + 2),
+                                 w_up=lin(E, H, 10 * i + 3), w_down=lin(H, E, 10 * i + 4)).with_stream() for i in range(cfg.n_layers)]
+    embed = torch.randn((cfg.vocab_size, E), device="cuda", generator=g).to(torch.bfloat16)
+    return decode.LlamaModel(cfg, layers, embed, norm_w(), embed)
+
+
+def time_model(model, prompt_len, steps, warmup, reps):
+    """(seconds of a prompt pass, seconds per decoded token behind it), each as one HIP graph on its own stream."""
+    import torch
+
+    stream = torch.cuda.Stream()
+    cache = model.new_cache(prompt_len + max(steps, warmup) + 1)
+    prompt = torch.randint(0, model.vocab, (prompt_len,), generator=torch.Generator().manual_seed(1)).tolist()
+
+    def timed(record, n):
+        graph = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(graph, stream=stream):
+            out = record()
+        graph.replay()
+        stream.synchronize()
+        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        e0.record(stream)
+        for _ in range(n):
+            graph.replay()
+        e1.record(stream)
+        torch.cuda.synchronize()
+        return e0.elapsed_time(e1) * 1e-3 / n, out
+
+    with torch.cuda.stream(stream):
+        cache.reset()
+        _, first = model.prefill(cache, prompt)
+        stream.synchronize()
+        ids = torch.tensor(prompt, dtype=torch.int32, device=model.device)
+
+        def whole_prompt():
+            cache.reset()
+            return model.prefill(cache, ids)
+
+        prefill_s, (logits, first) = timed(whole_prompt, reps)
+        cache.pos = prompt_len
+        model.decode_greedy(cache, first, warmup)
+
+        def tokens():
+            cache.pos = prompt_len
+            return model.decode_greedy(cache, first, steps)
+
+        decode_s, out = timed(tokens, 1)
+    return prefill_s, decode_s / steps, bool(torch.isfinite(logits).all()) and out.numel() == steps
+
+
+def kuvonex_costs(size, M, pos):
+    """(FLOPs of a prompt of M tokens, bytes of a decoded token at position pos) the algorithm needs."""
+    z = KUVONEX_SIZES[size]
+    W, H, R, T = z["width"], z["heads"], z["rank"], z["rot"]
+    own, shared = (z["layers"] + 1) // 2, z["layers"] // 2
+    proj = W * (H * (z["dim"] + T + 2 * z["vdim"]))                     # Q, gate, O
+    expand = H * (z["dim"] + z["vdim"]) * R
+    moe = 3 * W * z["ff"] * z["top"] + W * z["experts"]
+    dkv = W * (R + T)
+    weights = (own + shared) * (proj + expand + moe) + own * dkv
+    attn = (own + shared) * M * M * H * (z["dim"] + T + z["vdim"])      # causal half of 2 M^2
+    flops = 2 * M * weights + attn + 2 * W * z["vocab"]
+    return flops, 2 * (weights + W * z["vocab"]) + (own + shared) * 2 * pos * (R + T)
+
+
+def llama_costs(c, M, pos):
+    E, H, hd = c["emb_dim"], c["hidden_dim"], c["head_dim"]
+    nqkv = (c["n_heads"] + 2 * c["n_kv_heads"]) * hd
+    flops = c["n_layers"] * (2 * M * (E * nqkv + E * E + 3 * E * H) + 2 * M * M * hd * c["n_heads"]) + 2 * E * c["vocab_size"]
+    layer = weight_bytes(E, nqkv) + weight_bytes(E, E) + 2 * weight_bytes(E, H) + weight_bytes(H, E) + 2 * c["n_kv_heads"] * pos * hd * 2
+    return flops, c["n_layers"] * layer + 2 * c["vocab_size"] * E
+
+
+def run_kuvonex(steps, warmup, only=None, prompt_len=2048, llama=True):
+    """Prompt pass and greedy decode of the Kuvonex sizes and of the int4 Llama layers beside them."""
+    import torch
+
+    torch.cuda.set_device(0)
+    out = {}
+    for size in ([only] if only else KUVONEX_SIZES):
+        rows = {"kuvonex": (lambda: random_kuvonex(size), kuvonex_costs(size, prompt_len, prompt_len + steps // 2))}
+        if llama:
+            c = KUVONEX_SIZES[size]["llama"]
+            rows["llama_int4"] = (lambda: random_llama(c), llama_costs(c, prompt_len, prompt_len + steps // 2))
+        out[size] = {}
+        for name, (make, (flops, nbytes)) in rows.items():
+            model = make()
+            pre, dec, ok = time_model(model, prompt_len, steps, warmup, 3)
+            del model
+            torch.cuda.empty_cache()
+            out[size][name] = {"prefill_ms": pre * 1e3, "prefill_tokens_per_s": prompt_len / pre, "prefill_TFLOP/s": flops / pre / 1e12,
+                               "prefill_frac_mfma_peak": flops / pre / 1e12 / MFMA_BF16_PEAK_TFLOPS, "decode_us_per_token": dec * 1e6,
+                               "decode_tokens_per_s": 1 / dec, "decode_GB/s": nbytes / dec / 1e9, "decode_frac_hbm_peak": nbytes / dec / 1e9 / HBM_PEAK_GBS,
+                               "finite": ok}
+    return out
+
+
 def cpu_baseline(name, torch, w, x, outs, launch, stream):
     """The reference's NumPy path (restated in oracle/baseline.py) timed on this host's cores,
     on the same inputs as GPU launch 0; also used to sanity-check the GPU result."""
@@ -723,7 +872,9 @@ def main():
     ap.add_argument("--steps", type=int, default=200)
     ap.add_argument("--warmup", type=int, default=20)
     ap.add_argument("--workload", default="gemv", choices=list(CONFIGS) + ["decode_1b", "decode_8b", "prefill_block", "prefill_block_awq", "prefill_1b", "prefill_1b_awq",
-                                                             "prefill_8b"])
+                                                             "prefill_8b", "kuvonex"])
+    ap.add_argument("--size", choices=list(KUVONEX_SIZES), help="--workload kuvonex: this size only")
+    ap.add_argument("--no-llama", action="store_true", help="--workload kuvonex: without the int4 Llama layers beside it")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-extra", action="store_true", help="skip the short runs of the other configs")
     ap.add_argument("--copy-probe", action="store_true",
@@ -750,6 +901,21 @@ def main():
         dst.copy_(src)
         torch.cuda.synchronize()
         del src, dst
+    if a.workload == "kuvonex":
+        steps, warmup = min(a.steps, 64), min(a.warmup, 4)
+        r = run_kuvonex(steps, warmup, a.size, llama=not a.no_llama)
+        size, first = next(iter(r.items()))
+        k = first["kuvonex"]
+        print(json.dumps({
+            "metric": f"Kuvonex decode tokens/s, size {size}, batch 1", "value": k["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
+            "warmup": warmup, "ms_per_step": k["decode_us_per_token"] * 1e-3, "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+            "dtype": "bf16 weights and activations, fp32 residual and accumulate", "data": "synthetic (random weights of the architecture, random prompt)",
+            "config": {"workload": "prompt pass of 2048 tokens, then greedy decode behind it", "sizes": {s: KUVONEX_SIZES[s] for s in r},
+                       "timing": "one HIP graph of the pass / of all token steps, events on the launch stream"},
+            "roofline": {"bound": "hbm", "achieved": k["decode_GB/s"], "peak": HBM_PEAK_GBS, "unit": "GB/s", "frac": k["decode_frac_hbm_peak"],
+                         "traffic": None, "avg_launch_us": k["decode_us_per_token"]},
+            "sizes": r}))
+        return
     if a.workload in ("prefill_1b", "prefill_1b_awq", "prefill_8b"):
         model = "decode_8b" if a.workload == "prefill_8b" else "decode_1b"
         r = run_prefill_model(model, 2048, max(1, min(a.steps, 5)), stream_order=not a.workload.endswith("_awq"))

@@ -280,7 +280,7 @@ class LlamaModel(generation.CausalLM):
         return LlamaCache(self.config, max_tokens, self.device)
 
     def prefill(self, cache, tokens):
-        ids = torch.as_tensor(list(tokens), dtype=torch.int32, device=self.device)
+        ids = tokens if isinstance(tokens, torch.Tensor) else torch.as_tensor(list(tokens), dtype=torch.int32, device=self.device)
         logits, best = prefill(ids, self.layers, self.embed_table, self.final_norm, self.lm_head, self.config, cache.kv, self.rope_lut)
         cache.pos = len(tokens)
         return logits, best

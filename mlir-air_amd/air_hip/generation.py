@@ -26,7 +26,7 @@ class CausalLM:
         raise NotImplementedError
 
     def prefill(self, cache, tokens):
-        """Run a prompt; (fp32 logits [vocab] of its last position, greedy next token as a device int32 [1])."""
+        """Run a prompt (ints, or ids on the device); (fp32 logits [vocab] of its last position, greedy next token as a device int32 [1])."""
         raise NotImplementedError
 
     def decode_token(self, cache, token):

@@ -305,6 +305,8 @@ class KuvonexModel(generation.CausalLM):
         return res
 
     def _ids(self, tokens):
+        if isinstance(tokens, torch.Tensor):   # already on the device: the caller answers for the range
+            return tokens.to(device=self.device, dtype=torch.int32).contiguous()
         tokens = [int(t) for t in tokens]
         if not tokens or min(tokens) < 0 or max(tokens) >= self.vocab:
             raise ValueError(f"token ids must lie in 0 .. {self.vocab - 1}")

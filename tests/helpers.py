@@ -41,3 +41,68 @@ def assert_bf16_close(actual_bits, want_f64, ulps=1.0, atol=0.0, what=""):
     assert not bad.any(), (
         f"{what}: {int(bad.sum())}/{bad.size} elements outside {ulps} bf16 ulp + {atol}; "
         f"worst err {err.max():.4g} at {np.unravel_index(np.argmax(err - tol), err.shape)}")
+
+
+# ---- Kuvonex ------------------------------------------------------------------------------------------------------------
+def kuvonex_layer(heads=3, dim=24, rot_dim=8, vdim=40, kv_rank=56, kv_from=None, base=500.0, scale=None, mlp=None):
+    """One entry of `layers` of a Kuvonex config.json.  mlp: (experts, top, groups, keep, ff) or None."""
+    mixer = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
+             "scale": (dim + rot_dim) ** -0.5 if scale is None else scale, "rot": {"base": base, "dims": rot_dim}}
+    if kv_from is not None:
+        mixer["kv_from"] = kv_from
+    if mlp is not None:
+        experts, top, groups, keep, ff = mlp
+        mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}}}
+    return {"type": "latent_attention", "mixer": mixer, "mlp": mlp}
+
+
+def kuvonex_config(layers, vocab=67, width=72, eps=1e-5, embed_scale=1.7):
+    return {"architecture": "Kuvonex", "vocab": vocab, "width": width, "norm": {"eps": eps}, "embedding": {"scale": embed_scale}, "layers": layers}
+
+
+def kuvonex_weights(config, seed=0):
+    """Random weights as float32 arrays that hold bf16 values, by checkpoint name."""
+    from air_hip import kuvonex
+
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in kuvonex.tensor_shapes(kuvonex.KuvonexConfig.from_json(config)).items():
+        if name.endswith("norm") or name.endswith("norm1") or name.endswith("norm2"):
+            v = 1.0 + 0.3 * rng.standard_normal(shape)
+        elif name.endswith("sink"):
+            v = 1.5 * rng.standard_normal(shape)
+        elif name.endswith("correction"):
+            v = -0.6 + 0.5 * rng.standard_normal(shape)    # choice scores of either sign
+        elif name == "embed":
+            v = rng.standard_normal(shape) * 0.6
+        else:
+            v = rng.standard_normal(shape) * shape[-1] ** -0.5
+            if name.endswith("router"):
+                v *= 2.0                                     # scores well apart
+        out[name] = bf16_bits_to_f32(f32_to_bf16_bits(v.astype(np.float32)))
+    return out
+
+
+def kuvonex_write(path, config, weights):
+    """The checkpoint directory (config.json, model.safetensors)."""
+    import json
+    import os
+
+    import torch
+    from safetensors.torch import save_file
+
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(config, f)
+    save_file({k: torch.from_numpy(v).to(torch.bfloat16).contiguous() for k, v in weights.items()}, os.path.join(path, "model.safetensors"))
+    return str(path)
+
+
+# Layers that differ in every size, one without a feed-forward, one that attends over an earlier layer's cache with other
+# head sizes than its source; groups of one, of two and no grouping at all.
+KUVONEX_MIXED = kuvonex_config([
+    kuvonex_layer(mlp=(12, 3, 3, 2, 40)),
+    kuvonex_layer(heads=2, dim=40, rot_dim=12, vdim=16, kv_rank=72, base=90.0),
+    kuvonex_layer(heads=5, dim=16, rot_dim=8, vdim=24, kv_rank=56, kv_from=0, scale=0.31, mlp=(6, 2, 6, 3, 72)),
+    kuvonex_layer(heads=1, dim=8, rot_dim=12, vdim=8, kv_rank=72, base=90.0, kv_from=1, mlp=(4, 2, 1, 1, 8)),
+], vocab=67, width=72)
