@@ -655,6 +655,8 @@ def random_kuvonex(size, dtype=None):
         t = torch.randn(shape, device="cuda", generator=g)
         if "norm" in name:
             return 1.0 + 0.1 * t
+        if name.endswith("correction"):
+            return 0.02 * t                      # experts used about equally
         return t.mul_(1.0 if name == "embed" or len(shape) == 1 else shape[-1] ** -0.5).to(torch.bfloat16)
 
     return kuvonex.KuvonexModel(cfg, tensor, dtype or torch.bfloat16)

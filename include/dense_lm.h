@@ -77,7 +77,7 @@ int dlm_moe_gate_up_gemv(int dtype, const dlm_router *r, const void *x, const vo
 int dlm_moe_down_gemv(int dtype, const void *h, const void *w_down, const int32_t *ids, const float *weights, float *y, int top,
                       int experts, int ff, int N, void *stream);
 /* Many tokens: ids, weights [tokens, top]; then the entries token * top + slot sorted by expert (order[tokens * top]) and
- * their row tiles (int32 [dlm_moe_max_tiles(..), 4]). */
+ * their row tiles (int32 [dlm_moe_max_tiles(..) + 1, 4]; the last row holds the number of tiles in use). */
 int dlm_moe_select(const dlm_router *r, int tokens, int32_t *ids, float *weights, void *stream);
 int dlm_moe_max_tiles(int entries, int experts, int tile_rows);
 int dlm_moe_plan(const int32_t *ids, int entries, int experts, int tile_rows, int32_t *order, int32_t *tiles, void *stream);
@@ -90,9 +90,10 @@ typedef struct {
     void *out;
     int64_t lda, ldo, w_stride;
     const int32_t *tiles, *order;
-    int32_t M, N, K, epilogue, n_tiles, gather, tile_rows;   /* tile_rows: dlm_gemm_tile_rows(dtype, rows per matrix, N) */
+    int32_t M, N, K, epilogue, n_tiles, gather, tile_rows;   /* tile_rows: dlm_gemm_tile_rows, or 32, 128, 256 */
 } dlm_gemm_args;
-int dlm_gemm_tile_rows(int dtype, int rows, int N);
+/* Rows of A per tile for `rows` rows (experts: the mean number) with each of `matrices` matrices of N rows. */
+int dlm_gemm_tile_rows(int dtype, int rows, int N, int matrices);
 int dlm_gemm(int dtype, const dlm_gemm_args *g, void *stream);
 
 int dlm_embed_rows(int dtype, const int32_t *tokens, const void *embed, float scale, float *res, void *h, int M, int width, void *stream);

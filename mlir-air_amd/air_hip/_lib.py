@@ -119,7 +119,7 @@ DENSE_SYMBOLS = {
     "dlm_moe_select": (_ci, [_vp, _ci, _vp, _vp, _vp]),
     "dlm_moe_max_tiles": (_ci, [_ci] * 3),
     "dlm_moe_plan": (_ci, [_vp] + [_ci] * 3 + [_vp] * 3),
-    "dlm_gemm_tile_rows": (_ci, [_ci] * 3),
+    "dlm_gemm_tile_rows": (_ci, [_ci] * 4),
     "dlm_gemm": (_ci, [_ci, _vp, _vp]),
     "dlm_embed_rows": (_ci, [_ci, _vp, _vp, _cf, _vp, _vp, _ci, _ci, _vp]),
     "dlm_residual_norm_rows": (_ci, [_ci, _vp, _vp, _vp, _ci, _vp, _cf, _ci, _vp, _ci, _ci, _vp]),

@@ -145,7 +145,7 @@ def gemm(a, w, out_f32=False, lda=None, rows=None, out=None):
     if out is None:
         out = torch.empty((M, N), dtype=torch.float32 if out_f32 else w.dtype, device=w.device)
     g = _lib.GemmArgs(a=_ptr(a), w=_ptr(w), out=_ptr(out), lda=lda, ldo=N, M=M, N=N, K=K, epilogue=OUT_F32 if out_f32 else OUT_ELEM,
-                      tile_rows=lib.dlm_gemm_tile_rows(dtype_code(w), M, N))
+                      tile_rows=lib.dlm_gemm_tile_rows(dtype_code(w), M, N, 1))
     _lib.check_dense(lib.dlm_gemm(dtype_code(w), ctypes.byref(g), _stream()))
     return out
 
@@ -252,10 +252,10 @@ def moe_rows(h, logits, router, w_gate_up, w_down):
     M, dev, dt = h.shape[0], h.device, dtype_code(h)
     ids, wts = moe_select(logits, router)
     entries = M * top
-    tile_rows = 32 if entries <= 48 * E else 128   # by the mean number of rows of an expert
+    tile_rows = lib.dlm_gemm_tile_rows(dt, entries // E, max(ff2, N), E)
     n_tiles = lib.dlm_moe_max_tiles(entries, E, tile_rows)
     order = torch.empty((entries,), dtype=torch.int32, device=dev)
-    tiles = torch.empty((n_tiles, 4), dtype=torch.int32, device=dev)
+    tiles = torch.empty((n_tiles + 1, 4), dtype=torch.int32, device=dev)
     _lib.check_dense(lib.dlm_moe_plan(_ptr(ids), entries, E, tile_rows, _ptr(order), _ptr(tiles), _stream()))
     act = torch.empty((entries, ff), dtype=h.dtype, device=dev)
     out = torch.empty((entries, N), dtype=h.dtype, device=dev)
@@ -330,11 +330,11 @@ def latent_attention_rows(spec, proj, kv_off, gate_off, lut, kv_norm, eps, cache
     return out
 
 
-def latent_splits(spec, M, total, dtype):
-    """How many workgroups share the keys of 16 rows: enough for the chip, at most one per block of keys."""
-    kb = 64 if dtype == torch.bfloat16 else 32
-    tiles = (M * spec.heads + 15) // 16
-    return max(1, min(128, 512 // tiles, (total + kb - 1) // kb))
+def latent_splits(spec, M, total):
+    """How many workgroups share the keys of 16 rows.  A workgroup's time grows with its blocks of 32 keys, the merge's with
+    the splits and rows: the square root balances them (constant measured at 16, 32 and 128 heads, 2k to 128k keys)."""
+    rows, blocks = M * spec.heads, (total + 31) // 32
+    return max(1, min(256, 512 // ((rows + 15) // 16), blocks, round((512 * blocks / rows) ** 0.5)))
 
 
 def latent_attention_absorbed(spec, proj, kv_off, gate_off, lut, kv_norm, eps, cache, pos, w_ukv, sink, pos_dev=None, nsplit=None):
@@ -349,7 +349,7 @@ def latent_attention_absorbed(spec, proj, kv_off, gate_off, lut, kv_norm, eps, c
         raise ValueError("latent attention: the key / value projection has another shape")
     w_uk, w_uv = w_ukv[:spec.heads * spec.dim_p], w_ukv[spec.heads * spec.dim_p:]
     if nsplit is None:
-        nsplit = latent_splits(spec, M, pos + M, proj.dtype)
+        nsplit = latent_splits(spec, M, pos + M)
     rows = M * spec.heads
     qa = torch.empty((rows, spec.cache_width), dtype=proj.dtype, device=dev)
     part_o = torch.empty((rows, nsplit, spec.rank_p), dtype=torch.float32, device=dev)

@@ -277,7 +277,7 @@ class KuvonexModel(generation.CausalLM):
                 proj, res, _ = dense.gemv_embed(token, self.embed, c.embed_scale, l.w_in)
             else:
                 proj, res, _ = dense.gemv_residual(r, l.w_in)
-            nsplit = None if pos_dev is None else dense.latent_splits(l.spec, 1, cache.capacity, self.dtype)
+            nsplit = None if pos_dev is None else dense.latent_splits(l.spec, 1, cache.capacity)
             attn = self._attend(l, proj, cache, pos, pos_dev, nsplit)
             y = dense.gemv(attn.reshape(-1), l.w_o, out_f32=True)
             r = dense.Residual(res, y, l.norm1, c.eps, c.width)

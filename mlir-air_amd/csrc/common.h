@@ -77,17 +77,30 @@ __device__ __forceinline__ float wave_reduce(float v) {
     return op(v, __shfl_xor(v, 32));
 }
 
-// Sum over the 16 lanes of a DPP row, every lane of the row receiving it (the four in-row steps of wave_reduce).
-__device__ __forceinline__ float row_sum16(float v) {
+// Maximum / sum over the 16 lanes of a DPP row, every lane of the row receiving it (the four in-row steps of wave_reduce).
+template <bool MAX>
+__device__ __forceinline__ float row_reduce16(float v) {
+    auto op = [](float a, float b) { return MAX ? fmaxf(a, b) : a + b; };
     auto dpp = [&](auto ctrl) {
         constexpr int CTRL = decltype(ctrl)::value;
-        v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true));
+        v = op(v, __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xF, 0xF, true)));
     };
     dpp(std::integral_constant<int, 0xB1>());    // quad_perm [1, 0, 3, 2]
     dpp(std::integral_constant<int, 0x4E>());    // quad_perm [2, 3, 0, 1]
     dpp(std::integral_constant<int, 0x141>());   // row_half_mirror
     dpp(std::integral_constant<int, 0x140>());   // row_mirror
     return v;
+}
+__device__ __forceinline__ float row_sum16(float v) { return row_reduce16<false>(v); }
+
+// max over the four lanes ql, ql + 16, ql + 32, ql + 48
+__device__ __forceinline__ float max_over_lane_groups(float v) {
+    const uint32_t u = __builtin_bit_cast(uint32_t, v);
+    const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);   // rows (0, 1) and (2, 3) exchanged
+    v = fmaxf(__builtin_bit_cast(float, (uint32_t)a[0]), __builtin_bit_cast(float, (uint32_t)a[1]));
+    const uint32_t w = __builtin_bit_cast(uint32_t, v);
+    const auto b = __builtin_amdgcn_permlane32_swap(w, w, false, false);   // halves exchanged
+    return fmaxf(__builtin_bit_cast(float, (uint32_t)b[0]), __builtin_bit_cast(float, (uint32_t)b[1]));
 }
 
 // silu(g) in the reference's tanh form (matvec_int4_swiglu_rms.py:512-514), fp32

@@ -151,7 +151,7 @@ int dlm_moe_plan(const int32_t *ids, int entries, int experts, int tile_rows, in
     return done(launch_moe_plan(ids, entries, experts, tile_rows, order, tiles, hs(stream)));
 }
 
-int dlm_gemm_tile_rows(int dtype, int rows, int N) { return dense_gemm_tile_rows(dtype, rows, N); }
+int dlm_gemm_tile_rows(int dtype, int rows, int N, int matrices) { return dense_gemm_tile_rows(dtype, rows, N, matrices); }
 
 int dlm_gemm(int dtype, const dlm_gemm_args *g, void *stream) {
     if (!g || !g->a || !g->w || !g->out) return DLM_ERR_NULL;

@@ -2,12 +2,14 @@
 // type, fp32 accumulation; plain, or grouped over the experts of a mixture (row tiles from moe_plan_kernel).
 //
 // Both operands have k contiguous, so a tile of either is a set of rows of 128 bytes per K-step (64 bf16 or 32 floats) and
-// goes global -> LDS without passing through registers (global_load_lds_dwordx4), double buffered: one wave instruction
+// goes global -> LDS without passing through registers (global_load_lds_dwordx4) into a ring of STAGES buffers, STAGES - 1
+// K-steps ahead (two where the tile is large; the small tile has little to multiply per step): one wave instruction
 // fills 1 KiB, 8 rows, lane l writing 16-byte slot l % 8 of row l / 8 and fetching chunk slot ^ row % 8, so that the operand
 // reads of 16 consecutive rows are spread over the banks without padding.  One barrier per K-step.  W is the first MFMA
 // operand: a lane then holds four consecutive n of one row m and stores them as one word.
 //
-// Row gathers cost nothing here: every lane of a copy has its own source row.
+// Row gathers cost nothing here: every lane of a copy has its own source row.  The waves of a SIMD differ in their rows, so
+// that a wave whose rows lie behind the end of an expert's run can leave the matrix pipe to the other.
 //
 // Requirements: K a multiple of 128 bytes of elements (the loader pads), N of 16.  Rows past M and N are read from the last
 // row and never stored.
@@ -33,7 +35,7 @@ struct GemmKernelArgs {
 };
 
 // BM x BN tile, WM x WN waves (m x n); GROUPED: expert row tiles
-template <class T, int BM, int BN, int WM, int WN, int EPI, bool GROUPED>
+template <class T, int BM, int BN, int WM, int WN, int STAGES, int EPI, bool GROUPED>
 __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKernelArgs<T> p) {
     constexpr int NW = WM * WN, KE = kRowBytes / sizeof(T), KS = KE / 32;
     constexpr int MT = BM / WM / 16, NT = BN / WN / 16;
@@ -44,25 +46,25 @@ __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKern
 
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int wm = wave % WM, wn = wave / WM;
+    const int wm = wave / WN, wn = wave % WN;
     const int ql = lane & 15, g = lane >> 4;
 
     // An XCD (blockIdx % 8) takes a contiguous range of tiles; in a band of four row panels the columns go by first, so
     // that the workgroups running together on one XCD share both operands in its L2.
-    const int total = p.tiles_m * p.tiles_n, per_xcd = (total + 7) / 8;
+    // (Experts: the launch covers the most tiles that there can be, the table's last row says how many there are.)
+    const int tiles_m = GROUPED ? p.tiles[4 * p.tiles_m] : p.tiles_m;
+    const int total = tiles_m * p.tiles_n, per_xcd = (total + 7) / 8;
     const int tile = (blockIdx.x & 7) * per_xcd + (blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per_xcd || tile >= total) return;
     const int band = tile / (4 * p.tiles_n), in_band = tile % (4 * p.tiles_n);
-    const int rows_in_band = p.tiles_m - 4 * band < 4 ? p.tiles_m - 4 * band : 4;
+    const int rows_in_band = tiles_m - 4 * band < 4 ? tiles_m - 4 * band : 4;
     const int tm = 4 * band + in_band % rows_in_band, tn = in_band / rows_in_band;
 
     const T *w = p.w;
     int m0 = tm * BM, m_end = p.M;
     if constexpr (GROUPED) {
         const int32_t *t = p.tiles + 4 * tm;
-        const int expert = t[0];
-        if (expert < 0) return;
-        w += (size_t)expert * p.w_stride;
+        w += (size_t)t[0] * p.w_stride;
         m0 = t[1];
         m_end = m0 + t[2];
     }
@@ -110,12 +112,24 @@ __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKern
         for (int i = 0; i < MT; ++i) acc[j][i] = floatx4{0.f, 0.f, 0.f, 0.f};
 
     const int steps = p.K / KE;
-    copy(0, 0);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // the copies write LDS behind the compiler's back
-    __syncthreads();
+    const bool idle = GROUPED && m0 + wm * (BM / WM) >= m_end;
+#pragma unroll
+    for (int i = 0; i < STAGES - 1; ++i)
+        if (i < steps) copy(i, i);
+    int buf = 0;
     for (int kt = 0; kt < steps; ++kt) {
-        if (kt + 1 < steps) copy((kt + 1) & 1, kt + 1);   // that buffer was last read before the barrier of the step before
-        const char *stage = gemm_lds + (kt & 1) * kStage;
+        // The copies write LDS behind the compiler's back: step kt's have landed once at most those of the STAGES - 2 steps
+        // after it are outstanding; this wave's reads of the step before have returned.  Then, behind the barrier, so have
+        // everybody's, and the buffer of the step before can be filled again.
+        if (STAGES > 2 && kt + STAGES - 2 < steps) asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"n"((STAGES - 2) * COPIES) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
+        const int next = buf == 0 ? STAGES - 1 : buf - 1;   // the buffer of the step before = of the step STAGES - 1 ahead
+        if (kt + STAGES - 1 < steps) copy(next, kt + STAGES - 1);
+        const char *stage = gemm_lds + buf * kStage;
+        buf = buf + 1 == STAGES ? 0 : buf + 1;
+        if (idle) continue;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
             Vec8<T> b[MT], a[NT];
@@ -128,8 +142,6 @@ __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKern
 #pragma unroll
                 for (int i = 0; i < MT; ++i) acc[j][i] = mma32(a[j], b[i], acc[j][i]);
         }
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();
     }
 
     // lane: row m = ... + ql, columns 4 g .. + 3 of each 16-column block
@@ -164,7 +176,7 @@ __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKern
     }
 }
 
-template <class T, int BM, int BN, int WM, int WN>
+template <class T, int BM, int BN, int WM, int WN, int STAGES>
 hipError_t launch_tile(const GemmArgs &g, hipStream_t stream) {
     GemmKernelArgs<T> p;
     p.a = static_cast<const T *>(g.a);
@@ -182,7 +194,7 @@ hipError_t launch_tile(const GemmArgs &g, hipStream_t stream) {
     p.tiles_m = g.tiles ? g.n_tiles : (g.M + BM - 1) / BM;
     p.tiles_n = (g.N + BN - 1) / BN;
     const int total = p.tiles_m * p.tiles_n, grid = (total + 7) / 8 * 8;
-    constexpr size_t lds = 2 * (size_t)(BM + BN) * kRowBytes;
+    constexpr size_t lds = STAGES * (size_t)(BM + BN) * kRowBytes;
     auto run = [&](auto kernel) {
         if (lds > 48 * 1024) {
             const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -192,27 +204,33 @@ hipError_t launch_tile(const GemmArgs &g, hipStream_t stream) {
         return hipGetLastError();
     };
     if (g.tiles)
-        return g.epilogue == kOutSwiglu ? run(&dense_gemm_kernel<T, BM, BN, WM, WN, kOutSwiglu, true>)
-                                        : run(&dense_gemm_kernel<T, BM, BN, WM, WN, kOutElem, true>);
-    return g.epilogue == kOutF32 ? run(&dense_gemm_kernel<T, BM, BN, WM, WN, kOutF32, false>)
-                                 : run(&dense_gemm_kernel<T, BM, BN, WM, WN, kOutElem, false>);
+        return g.epilogue == kOutSwiglu ? run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutSwiglu, true>)
+                                        : run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutElem, true>);
+    return g.epilogue == kOutF32 ? run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutF32, false>)
+                                 : run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutElem, false>);
 }
 
 }  // namespace
 
-// `rows`: rows per matrix (for experts: the mean number of entries of one)
-int dense_gemm_tile_rows(int dtype, int rows, int N) {
+// Rows of A per tile for a product of `rows` rows with each of `matrices` matrices.  Measured: full of work, the 256 x 256
+// kernel runs at 1.22 PFLOP/s with one workgroup per CU, the 128 x 128 one at 1.0 with two; each loses what its last round
+// of workgroups leaves idle.  Experts with enough rows take the large tile (their tiles are rarely full in either case).
+int dense_gemm_tile_rows(int dtype, int rows, int N, int matrices) {
     if (rows <= 48 || N < 96) return 32;
-    if (dtype == kBf16 && rows >= 192 && (long)((rows + 255) / 256) * ((N + 255) / 256) >= 96) return 256;
-    return 128;
+    if (dtype != kBf16) return 128;
+    if (matrices > 1) return rows >= 160 && N >= 256 ? 256 : 128;
+    const int t256 = ((rows + 255) / 256) * ((N + 255) / 256), t128 = ((rows + 127) / 128) * ((N + 127) / 128);
+    const float e256 = 1.22f * t256 / ((t256 + 255) / 256 * 256);
+    const float e128 = t128 < 512 ? 1.1f * t128 / 512 : (float)t128 / ((t128 + 255) / 256 * 256);
+    return e256 > e128 ? 256 : 128;
 }
 
 hipError_t launch_dense_gemm(int dtype, const GemmArgs &g, int tile_rows, hipStream_t stream) {
-    if (dtype == kF32) return tile_rows == 32 ? launch_tile<float, 32, 128, 1, 4>(g, stream) : launch_tile<float, 128, 128, 2, 2>(g, stream);
+    if (dtype == kF32) return tile_rows == 32 ? launch_tile<float, 32, 128, 1, 4, 4>(g, stream) : launch_tile<float, 128, 128, 2, 2, 2>(g, stream);
     switch (tile_rows) {
-        case 32: return launch_tile<bf16, 32, 128, 1, 4>(g, stream);
-        case 128: return launch_tile<bf16, 128, 128, 2, 2>(g, stream);
-        default: return launch_tile<bf16, 256, 256, 2, 4>(g, stream);
+        case 32: return launch_tile<bf16, 32, 128, 1, 4, 4>(g, stream);
+        case 128: return launch_tile<bf16, 128, 128, 2, 2, 2>(g, stream);
+        default: return launch_tile<bf16, 256, 256, 2, 4, 2>(g, stream);
     }
 }
 

@@ -55,7 +55,7 @@ hipError_t launch_moe_down_gemv(int dtype, const void *h, const void *w_down, co
 // many tokens
 hipError_t launch_moe_select(const Router &r, int tokens, int32_t *ids, float *weights, hipStream_t stream);
 // entries (token * top + slot) sorted by expert, and the row tiles of `bm` entries that the grouped product runs over:
-// tiles[i] = {expert (-1: none), first sorted entry, entries, 0}
+// tiles[i] = {expert, first sorted entry, entries, 0}, and behind the most tiles that there can be {number of tiles}
 int moe_max_tiles(int entries, int experts, int bm);
 hipError_t launch_moe_plan(const int32_t *ids, int entries, int experts, int bm, int32_t *order, int32_t *tiles, hipStream_t stream);
 
@@ -69,11 +69,11 @@ struct GemmArgs {
     int epilogue = kOutElem;
     // grouped (experts): rows are sorted entries, tiles from launch_moe_plan
     const int32_t *tiles = nullptr, *order = nullptr;
-    int n_tiles = 0;       // tiles in the table
+    int n_tiles = 0;       // the most tiles (moe_max_tiles)
     int gather = 0;        // > 0: A row of an entry = entry / gather, out row = sorted place; 0: A row = sorted place, out row = entry
     long w_stride = 0;     // elements from one expert's W to the next
 };
-int dense_gemm_tile_rows(int dtype, int rows, int N);   // rows of the tile the launch will use (what launch_moe_plan gets as bm)
+int dense_gemm_tile_rows(int dtype, int rows, int N, int matrices);   // rows of a tile (what launch_moe_plan gets as bm)
 hipError_t launch_dense_gemm(int dtype, const GemmArgs &g, int tile_rows, hipStream_t stream);
 
 hipError_t launch_embed_rows(int dtype, const int32_t *tokens, const void *embed, float scale, float *res, void *h, int M, int width,

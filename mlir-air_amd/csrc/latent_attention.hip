@@ -141,6 +141,36 @@ __host__ __device__ __forceinline__ int keys_per_split(int total, int nsplit, in
     return (blocks + nsplit - 1) / nsplit * kb;
 }
 
+// Rows of `chunks` times 8 elements that follow each other in memory -> LDS rows of another pitch, by the whole workgroup, in
+// batches of BATCH chunks per thread: every thread requests a batch before it stores the first of it.
+template <class T, int BATCH>
+struct RowCopy {
+    Vec8<T> v[BATCH];
+    // chunks first .. of the rows at `base`; from `limit` on (past the last row) the last chunk instead
+    __device__ __forceinline__ void request(const T *base, int first, int limit) {
+#pragma unroll
+        for (int i = 0; i < BATCH; ++i) {
+            const int n = first + (int)threadIdx.x + kLatThreads * i;
+            v[i] = load8(base + 8 * (n < limit ? n : limit - 1));
+        }
+    }
+    __device__ __forceinline__ void store(T *tile, int pitch, int chunks, int first, int count) const {
+        const int n0 = first + (int)threadIdx.x;
+        int r = n0 / chunks, c = n0 % chunks;
+        const int dr = kLatThreads / chunks, dc = kLatThreads % chunks;
+#pragma unroll
+        for (int i = 0; i < BATCH; ++i) {
+            if (n0 + kLatThreads * i < count) store8(tile + r * pitch + 8 * c, v[i]);
+            r += dr;
+            c += dc;
+            if (c >= chunks) {
+                c -= chunks;
+                ++r;
+            }
+        }
+    }
+};
+
 // blockIdx.x = split, blockIdx.y = 16 rows (row = token * heads + head).  CT: 16-column tiles of the latent per wave.
 template <class T, int KB, int CT>
 __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const LatentArgs<T> p, const T *qa, int nsplit, float *part_o, float *part_ml) {
@@ -153,8 +183,8 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
     T *tile = reinterpret_cast<T *>(latent_lds);  // [KB][pitch]
     T *qt = tile + KB * pitch;                    // [16][pitch]
     T *pt = qt + 16 * pitch;                      // [16][PP]
-    float *st = reinterpret_cast<float *>(pt + 16 * PP);   // [16][SP]
-    float *al = st + 16 * SP;                     // [16] rescaling factors of the block
+    float *st = reinterpret_cast<float *>(pt + 16 * PP);   // [parts][16][SP]
+    float *al = st + 4 / (KB / 16) * 16 * SP;     // [16] rescaling factors of the block
 
     const int pos0 = first_position(p), total = pos0 + p.M;
     const int per = keys_per_split(total, nsplit, KB);
@@ -164,10 +194,21 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
     const int k1 = k0 + per < seen ? k0 + per : seen;
 
     const int chunks = lq / 8;
-    for (int c = tid; c < 16 * chunks; c += kLatThreads) {
-        const int r = c / chunks, e = 8 * (c % chunks);
-        const int row = row0 + r < rows ? row0 + r : rows - 1;
-        store8(qt + r * pitch + e, load8(qa + (size_t)row * lq + e));
+    // A block of keys that is one batch travels to registers while the block before it is multiplied.
+    constexpr int BATCH = sizeof(T) == 2 ? 10 : 8;
+    RowCopy<T, BATCH> copy;
+    const int count = KB * chunks;
+    const bool one_batch = count <= BATCH * kLatThreads;
+    auto request = [&](int kb, int first) { copy.request(p.cache + (size_t)kb * lq, first, (total - kb < KB ? total - kb : KB) * chunks); };
+    if (k0 < k1) {
+        if (one_batch) request(k0, 0);
+        constexpr int QB = sizeof(T) == 2 ? 5 : 3;
+        RowCopy<T, QB> queries;
+        const int n = 16 * chunks, valid = (rows - row0 < 16 ? rows - row0 : 16) * chunks;
+        for (int first = 0; first < n; first += QB * kLatThreads) {
+            queries.request(qa + (size_t)row0 * lq, first, valid);
+            queries.store(qt, pitch, chunks, first, n);
+        }
     }
     // softmax threads: row tid / 16, keys (tid % 16) + 16 j of a block
     const int srow = tid >> 4, skey = tid & 15;
@@ -181,23 +222,30 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
     const float scale2 = p.s.scale * 1.4426950408889634f;
 
     for (int kb = k0; kb < k1; kb += KB) {
-        for (int c = tid; c < KB * chunks; c += kLatThreads) {
-            const int r = c / chunks, e = 8 * (c % chunks);
-            const int key = kb + r < total ? kb + r : total - 1;
-            store8(tile + r * pitch + e, load8(p.cache + (size_t)key * lq + e));
+        if (one_batch) {
+            copy.store(tile, pitch, chunks, 0, count);
+        } else {
+            for (int first = 0; first < count; first += BATCH * kLatThreads) {
+                request(kb, first);
+                copy.store(tile, pitch, chunks, first, count);
+            }
         }
         __syncthreads();
-        for (int kt = wave; kt < KB / 16; kt += kLatThreads / 64) {
+        if (one_batch && kb + KB < k1) request(kb + KB, 0);
+        {   // 16 keys per wave; with fewer key tiles than waves, several waves share one and each takes a part of the length
+            constexpr int PARTS = 4 / (KB / 16);
+            const int kt = wave % (KB / 16), part = wave / (KB / 16);
             floatx4 s0 = floatx4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
             const T *a = tile + (16 * kt + ql) * pitch + 8 * g, *b = qt + ql * pitch + 8 * g;
-            int k = 0;
-            for (; k + 64 <= lq; k += 64) {
-                s0 = mma32(load8(a + k), load8(b + k), s0);
-                s1 = mma32(load8(a + k + 32), load8(b + k + 32), s1);
+            const int steps = lq / 32, ks1 = steps * (part + 1) / PARTS;
+            int ks = steps * part / PARTS;
+            for (; ks + 2 <= ks1; ks += 2) {
+                s0 = mma32(load8(a + 32 * ks), load8(b + 32 * ks), s0);
+                s1 = mma32(load8(a + 32 * ks + 32), load8(b + 32 * ks + 32), s1);
             }
-            if (k < lq) s0 = mma32(load8(a + k), load8(b + k), s0);
+            if (ks < ks1) s0 = mma32(load8(a + 32 * ks), load8(b + 32 * ks), s0);
             s0 += s1;
-            *reinterpret_cast<floatx4 *>(st + ql * SP + 16 * kt + 4 * g) = s0;   // keys 4 g .. of row ql
+            *reinterpret_cast<floatx4 *>(st + part * 16 * SP + ql * SP + 16 * kt + 4 * g) = s0;   // keys 4 g .. of row ql
         }
         __syncthreads();
         {
@@ -206,16 +254,18 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
 #pragma unroll
             for (int j = 0; j < KB / 16; ++j) {
                 const int key = skey + 16 * j;
-                v[j] = kb + key <= my_limit ? st[srow * SP + key] * scale2 : kAttnNegBig;
+                float raw = st[srow * SP + key];
+#pragma unroll
+                for (int q = 1; q < 4 / (KB / 16); ++q) raw += st[q * 16 * SP + srow * SP + key];
+                v[j] = kb + key <= my_limit ? raw * scale2 : kAttnNegBig;
                 top = fmaxf(top, v[j]);
             }
-#pragma unroll
-            for (int d = 1; d < 16; d *= 2) top = fmaxf(top, __shfl_xor(top, d));
-            const float mn = fmaxf(m, top), alpha = exp2f(m - mn);
+            top = row_reduce16<true>(top);
+            const float mn = fmaxf(m, top), alpha = __builtin_amdgcn_exp2f(m - mn);
             float sum = 0.f;
 #pragma unroll
             for (int j = 0; j < KB / 16; ++j) {
-                const float e = v[j] > 0.5f * kAttnNegBig ? exp2f(v[j] - mn) : 0.f;
+                const float e = v[j] > 0.5f * kAttnNegBig ? __builtin_amdgcn_exp2f(v[j] - mn) : 0.f;
                 sum += e;
                 pt[srow * PP + skey + 16 * j] = from_float<T>(e);
             }
@@ -260,15 +310,16 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
     }
 }
 
-constexpr int kMaxSplits = 256, kValueRows = 32;
+constexpr int kMaxSplits = 256, kValueRows = 16;
+constexpr int kMergeThreads = 512, kMergeWaves = kMergeThreads / 64, kRowsPerWave = kValueRows / kMergeWaves;
 
-// blockIdx.x = head * blocks of 32 value rows, blockIdx.y = token
+// blockIdx.x = head * blocks of 16 value rows, blockIdx.y = token
 template <class T>
-__global__ void __launch_bounds__(kLatThreads) latent_combine_kernel(const LatentArgs<T> p, int nsplit, int kb, const float *part_o, const float *part_ml,
+__global__ void __launch_bounds__(kMergeThreads) latent_combine_kernel(const LatentArgs<T> p, int nsplit, int kb, const float *part_o, const float *part_ml,
                                                                      const float *sink, const T *w_uv, T *out, long ldo, int value_blocks) {
     __shared__ float f[kMaxSplits];
-    __shared__ float red[8];
-    extern __shared__ __attribute__((aligned(16))) float merged[];   // [rank up to a multiple of 512]
+    __shared__ float red[2 * kMergeWaves];
+    extern __shared__ __attribute__((aligned(16))) float merged[];   // [rank up to a multiple of 512], then [3][512]
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int h = blockIdx.x / value_blocks, v0 = (blockIdx.x % value_blocks) * kValueRows, m = blockIdx.y;
     const size_t row = (size_t)m * p.s.heads + h;
@@ -276,6 +327,11 @@ __global__ void __launch_bounds__(kLatThreads) latent_combine_kernel(const Laten
     const int active = (total + per - 1) / per;
     const int rank = p.s.rank;
 
+    // the first 512 columns of this wave's value rows are requested before anything is waited for
+    const T *w_row = w_uv + ((size_t)h * p.s.vdim + v0 + kRowsPerWave * wave) * rank;
+    Vec8<T> w_first[kRowsPerWave];
+#pragma unroll
+    for (int i = 0; i < kRowsPerWave; ++i) w_first[i] = 8 * lane < rank ? load8(w_row + (size_t)i * rank + 8 * lane) : zero8<T>();
     // factors of the splits in the log2 domain; the sink is one more term of the denominator
     const float snk = sink[h] * 1.4426950408889634f;
     float ms = kAttnNegBig, ls = 0.f;
@@ -287,39 +343,61 @@ __global__ void __launch_bounds__(kLatThreads) latent_combine_kernel(const Laten
     float top = wave_reduce<true>(ms);
     if (lane == 0) red[wave] = top;
     __syncthreads();
-    top = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), snk);
+    top = snk;
+#pragma unroll
+    for (int i = 0; i < kMergeWaves; ++i) top = fmaxf(top, red[i]);
     const float fac = tid < active ? exp2f(ms - top) : 0.f;
     const float part = wave_reduce<false>(fac * ls);
-    if (lane == 0) red[4 + wave] = part;
+    if (lane == 0) red[kMergeWaves + wave] = part;
     __syncthreads();
-    const float inv = 1.0f / (red[4] + red[5] + red[6] + red[7] + exp2f(snk - top));
-    f[tid] = fac * inv;
+    float den = exp2f(snk - top);
+#pragma unroll
+    for (int i = 0; i < kMergeWaves; ++i) den += red[kMergeWaves + i];
+    if (tid < kMaxSplits) f[tid] = fac / den;
     __syncthreads();
-    for (int r = 4 * tid; r < (rank + 511) / 512 * 512; r += 4 * kLatThreads) {
+    // merged latent: a thread adds every fourth split of four columns, the quarters meet in LDS
+    const int quarter = tid >> 7, col = 4 * (tid & 127);
+    float *piece = merged + (rank + 511) / 512 * 512;
+    constexpr int BATCH = 16;
+    for (int r0 = 0; r0 < rank; r0 += 512) {
+        const int r = r0 + col;
         floatx4 s = floatx4{0.f, 0.f, 0.f, 0.f};
         if (r < rank) {
             const float *src = part_o + row * nsplit * rank + r;
-            for (int i = 0; i < active; ++i) s += *reinterpret_cast<const floatx4 *>(src + (size_t)i * rank) * f[i];
+            for (int i = quarter; i < active; i += 4 * BATCH) {
+                floatx4 v[BATCH];
+#pragma unroll
+                for (int j = 0; j < BATCH; ++j) v[j] = *reinterpret_cast<const floatx4 *>(src + (size_t)(i + 4 * j < active ? i + 4 * j : i) * rank);
+#pragma unroll
+                for (int j = 0; j < BATCH; ++j) s += v[j] * (i + 4 * j < active ? f[i + 4 * j] : 0.f);
+            }
         }
-        *reinterpret_cast<floatx4 *>(merged + r) = s;
+        if (quarter > 0) *reinterpret_cast<floatx4 *>(piece + 512 * (quarter - 1) + col) = s;
+        __syncthreads();
+        if (quarter == 0) {
+#pragma unroll
+            for (int q = 0; q < 3; ++q) s += *reinterpret_cast<const floatx4 *>(piece + 512 * q + col);
+            *reinterpret_cast<floatx4 *>(merged + r) = s;
+        }
+        __syncthreads();
     }
-    __syncthreads();
-    for (int i = wave; i < kValueRows; i += kLatThreads / 64) {
-        const int v = v0 + i;
-        if (v >= p.s.vdim) break;
-        const T *w = w_uv + ((size_t)h * p.s.vdim + v) * rank;
+    float mine = 0.f;
+#pragma unroll
+    for (int i = 0; i < kRowsPerWave; ++i) {
         float acc = 0.f;
         for (int k = 8 * lane; k < rank; k += 512) {
             float wf[8];
-            unpack8(load8(w + k), wf);
+            unpack8(k < 512 ? w_first[i] : load8(w_row + (size_t)i * rank + k), wf);
 #pragma unroll
             for (int e = 0; e < 8; ++e) acc = fmaf(wf[e], merged[k + e], acc);
         }
         acc = wave_reduce<false>(acc);
-        if (lane == 0) {
-            const float gate = to_float(p.proj[(size_t)m * p.ld + p.gate_off + h * p.s.vdim + v]);
-            out[(size_t)m * ldo + h * p.s.vdim + v] = from_float<T>(acc * sigmoid_f32(gate));
-        }
+        mine = lane == i ? acc : mine;
+    }
+    if (lane < kRowsPerWave) {
+        const int v = h * p.s.vdim + v0 + kRowsPerWave * wave + lane;
+        const float gate = to_float(p.proj[(size_t)m * p.ld + p.gate_off + v]);
+        out[(size_t)m * ldo + v] = from_float<T>(mine * sigmoid_f32(gate));
     }
 }
 
@@ -344,12 +422,12 @@ LatentArgs<T> args_of(const LatentShape &s, const LatentRows &r) {
 template <class T>
 size_t decode_lds(const LatentShape &s, int kb) {
     const size_t pitch = s.rank + s.rot + 16 / sizeof(T);
-    return ((kb + 16) * pitch + 16 * (kb + 8)) * sizeof(T) + (16 * (kb + 4) + 16) * sizeof(float);
+    return ((kb + 16) * pitch + 16 * (kb + 8)) * sizeof(T) + (64 / kb * 16 * (kb + 4) + 16) * sizeof(float);
 }
 constexpr size_t kLdsLimit = 160 * 1024;
 
 template <class T>
-constexpr int decode_block() { return sizeof(T) == 2 ? 64 : 32; }
+constexpr int decode_block() { return 32; }
 
 // keys per block: fewer where a block of the usual size does not fit in LDS (0: not at all)
 template <class T>
@@ -375,12 +453,6 @@ hipError_t decode(const LatentShape &s, const LatentRows &r, const void *qa, int
         return hipGetLastError();
     };
     const int ct = (s.rank / 16 + 3) / 4;
-    if (kb == 64) {
-        if (ct <= 2) return run(&latent_decode_kernel<T, 64, 2>);
-        if (ct <= 4) return run(&latent_decode_kernel<T, 64, 4>);
-        if (ct <= 8) return run(&latent_decode_kernel<T, 64, 8>);
-        return run(&latent_decode_kernel<T, 64, 16>);
-    }
     if (kb == 32) {
         if (ct <= 2) return run(&latent_decode_kernel<T, 32, 2>);
         if (ct <= 4) return run(&latent_decode_kernel<T, 32, 4>);
@@ -403,7 +475,7 @@ template <class T>
 hipError_t combine(const LatentShape &s, const LatentRows &r, int nsplit, const float *part_o, const float *part_ml, const float *sink, const void *w_uv,
                    void *out, long ldo, hipStream_t stream) {
     const int blocks = (s.vdim + kValueRows - 1) / kValueRows;
-    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3(s.heads * blocks, r.M), dim3(kLatThreads), (size_t)(s.rank + 511) / 512 * 512 * sizeof(float),
+    hipLaunchKernelGGL(latent_combine_kernel<T>, dim3(s.heads * blocks, r.M), dim3(kMergeThreads), ((size_t)(s.rank + 511) / 512 * 512 + 3 * 512) * sizeof(float),
                        stream, args_of<T>(s, r), nsplit, decode_kb<T>(s), part_o, part_ml, sink, static_cast<const T *>(w_uv), static_cast<T *>(out), ldo,
                        blocks);
     return hipGetLastError();

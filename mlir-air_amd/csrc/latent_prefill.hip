@@ -7,9 +7,10 @@
 //   S^T[key, q] = K . Q^T      A = K rows from LDS, B = Q^T held in registers
 //   O^T[d, q]  += V^T . P^T    A = V^T (transposing LDS read), B = P^T built from the lane's own S^T registers
 // The D layout gives a lane keys 4 g .. + 3 of each 16-key block; the k slots of the second product are defined as exactly
-// those keys, so P never moves between lanes.  A workgroup is four waves on one head, QB blocks of 16 queries each, that
-// share the K and V rows going through LDS; the next block of keys travels global -> registers while one is multiplied.
-// The grid puts the longest rows first.  The running maximum may lag the true one by 2^8 (as in prefill_attention.hip), so
+// those keys, so P never moves between lanes.  Four waves of QB blocks of 16 queries each share the K and V rows going through
+// LDS; the next block of keys travels global -> registers while one is multiplied.  With SETS = 2 a second set of four waves
+// takes the odd key blocks for the same queries, and the two partial results are merged through LDS at the end: the longest
+// rows take half as long, and two waves share a SIMD.  The grid puts the longest rows first.  The running maximum may lag the true one by 2^8 (as in prefill_attention.hip), so
 // rescaling is rare; the row sum is a product with a row of ones.
 //
 // Head sizes that are common have kernels of their own (EXACT: everything unrolled); any other size runs on the next
@@ -21,8 +22,9 @@ namespace w4a16 {
 
 namespace {
 
-constexpr int kPfThreads = 256;
+constexpr int kSetThreads = 256;
 constexpr float kMasked = -1.0e30f;
+constexpr float kNoMax = -1.0e20f;   // "no score yet": far below any score, far above a masked one
 constexpr float kLazy = 8.0f;
 
 template <class T>
@@ -38,11 +40,6 @@ struct PrefillArgs {
     const float *sink;
 };
 
-__device__ __forceinline__ float max_of_lane_groups(float v) {   // over lanes ql, ql + 16, ql + 32, ql + 48
-    v = fmaxf(v, __shfl_xor(v, 16));
-    return fmaxf(v, __shfl_xor(v, 32));
-}
-
 template <class T>
 __device__ __forceinline__ Vec8<T> ones8();
 template <>
@@ -52,12 +49,14 @@ __device__ __forceinline__ Vec8<float> ones8<float>() { return {floatx4{1.f, 1.f
 
 // NQ: K-steps of 32 of a score; NV: 16-column tiles of the output; EXACT: the sizes are exactly these, otherwise at most
 // these.  blockIdx.z picks a range of 16 NV value columns.
-template <class T, int NQ, int NV, int QB, int KB, bool EXACT>
-__global__ void __launch_bounds__(kPfThreads) latent_prefill_kernel(const PrefillArgs<T> p) {
+// (EXACT addresses K and V rows with 32-bit offsets: the expanded matrix is smaller than 4 GiB.)
+template <class T, int NQ, int NV, int QB, int KB, int SETS, bool EXACT>
+__global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kernel(const PrefillArgs<T> p) {
     constexpr int NKK = KB / 16, NT = KB / 32, QW = 64 * QB;
     extern __shared__ __attribute__((aligned(16))) char pf_lds[];
-    const int tid = threadIdx.x, lane = tid & 63;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int tid = threadIdx.x & (kSetThreads - 1), lane = tid & 63;   // thread within its set
+    const int wave8 = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int set = SETS == 1 ? 0 : wave8 >> 2, wave = wave8 & 3;
     const int ql = lane & 15, g = lane >> 4;
     const int head = blockIdx.x, item = gridDim.y - 1 - blockIdx.y;
     const int qd = EXACT ? 32 * NQ : p.dim + p.rot;
@@ -65,7 +64,7 @@ __global__ void __launch_bounds__(kPfThreads) latent_prefill_kernel(const Prefil
     const int vd = EXACT ? 16 * NV : (p.vdim - vcol0 < 16 * NV ? p.vdim - vcol0 : 16 * NV);
     const int nq = qd / 32, nv = vd / 16;
     const int kp = qd + 16 / (int)sizeof(T), vp = vd + 32 / (int)sizeof(T);
-    T *kt = reinterpret_cast<T *>(pf_lds);
+    T *kt = reinterpret_cast<T *>(pf_lds) + set * KB * (kp + vp);
     T *vt = kt + KB * kp;
 
     const int pos0 = p.total - p.M;
@@ -89,58 +88,62 @@ __global__ void __launch_bounds__(kPfThreads) latent_prefill_kernel(const Prefil
 #pragma unroll
         for (int d = 0; d < NV; ++d) o[b][d] = floatx4{0.f, 0.f, 0.f, 0.f};
         l[b] = floatx4{0.f, 0.f, 0.f, 0.f};
-        m[b] = kMasked;
+        m[b] = kNoMax;
     }
 
     // a chunk is 8 elements of a row; the first dim of a K row come from the expanded matrix, the rest from the cache
+    const T *k_base = p.kv + (size_t)head * p.dim, *v_base = p.kv + p.v_off + (size_t)head * p.vdim + vcol0, *r_base = p.cache + p.rot_off;
+    auto at = [&](const T *base, int row, long ld, int e) -> Vec8<T> {
+        if constexpr (EXACT) return load8(reinterpret_cast<const T *>(reinterpret_cast<const char *>(base) + (uint32_t)(row * (uint32_t)ld + e) * (uint32_t)sizeof(T)));
+        return load8(base + (size_t)row * ld + e);
+    };
     auto k_chunk = [&](int kb, int c, int cpr) -> Vec8<T> {
         const int key = kb + c / cpr, e = 8 * (c % cpr);
-        const size_t row = key < p.total ? key : p.total - 1;
-        return e < p.dim ? load8(p.kv + row * p.ldkv + (size_t)head * p.dim + e) : load8(p.cache + row * p.ldc + p.rot_off + (e - p.dim));
+        const int row = key < p.total ? key : p.total - 1;
+        return e < p.dim ? at(k_base, row, p.ldkv, e) : at(r_base, row, p.ldc, e - p.dim);
     };
     auto v_chunk = [&](int kb, int c, int cpr) -> Vec8<T> {
         const int key = kb + c / cpr, e = 8 * (c % cpr);
-        const size_t row = key < p.total ? key : p.total - 1;
-        return load8(p.kv + row * p.ldkv + p.v_off + (size_t)head * p.vdim + vcol0 + e);
+        return at(v_base, key < p.total ? key : p.total - 1, p.ldkv, e);
     };
     constexpr int CK = 4 * NQ, CV = 2 * NV;                       // chunks per row (EXACT)
-    constexpr int NCK = EXACT ? KB * CK / kPfThreads : 1, NCV = EXACT ? KB * CV / kPfThreads : 1;
-    static_assert(!EXACT || (KB * CK % kPfThreads == 0 && KB * CV % kPfThreads == 0), "whole chunks per thread");
+    constexpr int NCK = EXACT ? KB * CK / kSetThreads : 1, NCV = EXACT ? KB * CV / kSetThreads : 1;
+    static_assert(!EXACT || (KB * CK % kSetThreads == 0 && KB * CV % kSetThreads == 0), "whole chunks per thread");
     Vec8<T> kreg[NCK], vreg[NCV];
     auto fetch = [&](int it) {
         if constexpr (EXACT) {
 #pragma unroll
-            for (int i = 0; i < NCK; ++i) kreg[i] = k_chunk(it * KB, tid + kPfThreads * i, CK);
+            for (int i = 0; i < NCK; ++i) kreg[i] = k_chunk(it * KB, tid + kSetThreads * i, CK);
 #pragma unroll
-            for (int i = 0; i < NCV; ++i) vreg[i] = v_chunk(it * KB, tid + kPfThreads * i, CV);
+            for (int i = 0; i < NCV; ++i) vreg[i] = v_chunk(it * KB, tid + kSetThreads * i, CV);
         }
     };
     auto stage = [&](int it) {
         if constexpr (EXACT) {
 #pragma unroll
             for (int i = 0; i < NCK; ++i) {
-                const int c = tid + kPfThreads * i;
+                const int c = tid + kSetThreads * i;
                 store8(kt + (c / CK) * kp + 8 * (c % CK), kreg[i]);
             }
 #pragma unroll
             for (int i = 0; i < NCV; ++i) {
-                const int c = tid + kPfThreads * i;
+                const int c = tid + kSetThreads * i;
                 store8(vt + (c / CV) * vp + 8 * (c % CV), vreg[i]);
             }
         } else {
             const int ck = qd / 8, cv = vd / 8;
-            for (int c = tid; c < KB * ck; c += kPfThreads) store8(kt + (c / ck) * kp + 8 * (c % ck), k_chunk(it * KB, c, ck));
-            for (int c = tid; c < KB * cv; c += kPfThreads) store8(vt + (c / cv) * vp + 8 * (c % cv), v_chunk(it * KB, c, cv));
+            for (int c = tid; c < KB * ck; c += kSetThreads) store8(kt + (c / ck) * kp + 8 * (c % ck), k_chunk(it * KB, c, ck));
+            for (int c = tid; c < KB * cv; c += kSetThreads) store8(vt + (c / cv) * vp + 8 * (c % cv), v_chunk(it * KB, c, cv));
         }
     };
 
-    fetch(0);
-    for (int it = 0; it < blocks; ++it) {
-        const int kb = it * KB;
-        stage(it);
+    if (set < blocks) fetch(set);
+    for (int it0 = 0; it0 < blocks; it0 += SETS) {
+        const int it = it0 + set, kb = it * KB;
+        if (it < blocks) stage(it);
         __syncthreads();
-        if (it + 1 < blocks) fetch(it + 1);
-        if (kb <= wave_last) {
+        if (it + SETS < blocks) fetch(it + SETS);
+        if (it < blocks && kb <= wave_last) {
             floatx4 s[NKK][QB];
 #pragma unroll
             for (int kk = 0; kk < NKK; ++kk) {
@@ -173,10 +176,10 @@ __global__ void __launch_bounds__(kPfThreads) latent_prefill_kernel(const Prefil
                     v = fmaxf(fmaxf(v, s[kk][b][0]), s[kk][b][1]);
                     v = fmaxf(fmaxf(v, s[kk][b][2]), s[kk][b][3]);
                 }
-                bm[b] = max_of_lane_groups(v);
+                bm[b] = max_over_lane_groups(v);
                 lag = lag || (bm[b] - m[b]) * p.scale_log2 > kLazy;
             }
-            if (__builtin_amdgcn_ballot_w64(lag) != 0) {   // (the first block always: key 0 is visible to every query)
+            if (__builtin_amdgcn_ballot_w64(lag) != 0) {   // (always at a query's first visible key)
 #pragma unroll
                 for (int b = 0; b < QB; ++b) {
                     const float mn = fmaxf(m[b], bm[b]);
@@ -214,6 +217,36 @@ __global__ void __launch_bounds__(kPfThreads) latent_prefill_kernel(const Prefil
         __syncthreads();
     }
 
+    if constexpr (SETS == 2) {   // the same wave and lane of the other set holds the same queries and output elements
+        constexpr int NREG = QB * (4 * NV + 2);
+        float *xch = reinterpret_cast<float *>(pf_lds) + wave * NREG * 64 + lane;
+        if (set == 1) {
+#pragma unroll
+            for (int b = 0; b < QB; ++b) {
+#pragma unroll
+                for (int d = 0; d < NV; ++d)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) xch[((b * NV + d) * 4 + r) * 64] = o[b][d][r];
+                xch[(4 * QB * NV + 2 * b) * 64] = m[b];
+                xch[(4 * QB * NV + 2 * b + 1) * 64] = l[b][0];
+            }
+        }
+        __syncthreads();
+        if (set == 1) return;
+#pragma unroll
+        for (int b = 0; b < QB; ++b) {
+            const float m1 = xch[(4 * QB * NV + 2 * b) * 64], l1 = xch[(4 * QB * NV + 2 * b + 1) * 64];
+            const float mm = fmaxf(m[b], m1);
+            const float f0 = __builtin_amdgcn_exp2f((m[b] - mm) * p.scale_log2), f1 = __builtin_amdgcn_exp2f((m1 - mm) * p.scale_log2);
+            m[b] = mm;
+            l[b][0] = l[b][0] * f0 + l1 * f1;
+#pragma unroll
+            for (int d = 0; d < NV; ++d)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[b][d][r] = o[b][d][r] * f0 + xch[((b * NV + d) * 4 + r) * 64] * f1;
+        }
+    }
+
     const float snk = p.sink[head] * 1.4426950408889634f;
 #pragma unroll
     for (int b = 0; b < QB; ++b) {
@@ -237,18 +270,20 @@ __global__ void __launch_bounds__(kPfThreads) latent_prefill_kernel(const Prefil
 
 constexpr size_t kLdsLimit = 160 * 1024;
 
-template <class T, int NQ, int NV, int QB, int KB, bool EXACT>
+template <class T, int NQ, int NV, int QB, int KB, int SETS, bool EXACT>
 hipError_t launch(const PrefillArgs<T> &p, hipStream_t stream) {
     const int vd = p.vdim < 16 * NV ? p.vdim : 16 * NV;
-    const size_t lds = (size_t)KB * ((p.dim + p.rot + 16 / sizeof(T)) + (vd + 32 / sizeof(T))) * sizeof(T);
+    size_t lds = (size_t)SETS * KB * ((p.dim + p.rot + 16 / sizeof(T)) + (vd + 32 / sizeof(T))) * sizeof(T);
+    const size_t exchange = SETS == 2 ? 4 * QB * (4 * NV + 2) * 64 * sizeof(float) : 0;
+    if (lds < exchange) lds = exchange;
     if (lds > kLdsLimit) return hipErrorInvalidValue;
-    auto kernel = &latent_prefill_kernel<T, NQ, NV, QB, KB, EXACT>;
+    auto kernel = &latent_prefill_kernel<T, NQ, NV, QB, KB, SETS, EXACT>;
     if (lds > 48 * 1024) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
     const int items = (p.M + 64 * QB - 1) / (64 * QB);
-    hipLaunchKernelGGL(kernel, dim3(p.heads, items, (p.vdim + 16 * NV - 1) / (16 * NV)), dim3(kPfThreads), lds, stream, p);
+    hipLaunchKernelGGL(kernel, dim3(p.heads, items, (p.vdim + 16 * NV - 1) / (16 * NV)), dim3(SETS * kSetThreads), lds, stream, p);
     return hipGetLastError();
 }
 
@@ -289,16 +324,18 @@ hipError_t launch_latent_prefill(int dtype, const LatentShape &s, const LatentRo
     const int nq = (s.dim + s.rot) / 32, nv = s.vdim / 16;
     if (dtype == kF32) {
         const PrefillArgs<float> p = args_of<float>(s, r, kv, ldkv, sink, out, ldo);
-        if (nq <= 4 && nv <= 4) return launch<float, 4, 4, 1, 32, false>(p, stream);
-        if (nq <= 8 && nv <= 8) return launch<float, 8, 8, 1, 32, false>(p, stream);
-        return launch<float, 16, 16, 1, 32, false>(p, stream);
+        if (nq <= 4 && nv <= 4) return launch<float, 4, 4, 1, 32, 1, false>(p, stream);
+        if (nq <= 8 && nv <= 8) return launch<float, 8, 8, 1, 32, 1, false>(p, stream);
+        return launch<float, 16, 16, 1, 32, 1, false>(p, stream);
     }
     const PrefillArgs<bf16> p = args_of<bf16>(s, r, kv, ldkv, sink, out, ldo);
-    if (nq == 6 && nv == 8) return launch<bf16, 6, 8, 2, 64, true>(p, stream);
-    if (nq == 3 && nv == 4) return launch<bf16, 3, 4, 2, 64, true>(p, stream);
-    if (nq <= 4 && nv <= 4) return launch<bf16, 4, 4, 1, 64, false>(p, stream);
-    if (nq <= 8 && nv <= 8) return launch<bf16, 8, 8, 1, 64, false>(p, stream);
-    return launch<bf16, 16, 16, 1, 32, false>(p, stream);
+    if ((double)p.total * ldkv * sizeof(bf16) < 4e9) {
+        if (nq == 6 && nv == 8) return launch<bf16, 6, 8, 2, 64, 2, true>(p, stream);
+        if (nq == 3 && nv == 4) return launch<bf16, 3, 4, 2, 64, 2, true>(p, stream);
+    }
+    if (nq <= 4 && nv <= 4) return launch<bf16, 4, 4, 1, 64, 1, false>(p, stream);
+    if (nq <= 8 && nv <= 8) return launch<bf16, 8, 8, 1, 64, 1, false>(p, stream);
+    return launch<bf16, 16, 16, 1, 32, 1, false>(p, stream);
 }
 
 }  // namespace w4a16

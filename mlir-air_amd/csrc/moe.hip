@@ -18,35 +18,45 @@ namespace {
 
 constexpr int kMoeWaves = 4, kMoeThreads = 64 * kMoeWaves;
 constexpr int kMoePiece = 512;
-constexpr int kPerLane = kMaxExperts / 64;
 
-// Called by one whole wavefront; choice: LDS scratch of r.experts floats, group: of r.groups floats (both of this wave).  ids / weights [top] may
-// be LDS or global.
+// Called by one whole wavefront, which owns experts lane + 64 j, j < PL; choice: LDS scratch of r.experts floats, group: of
+// r.groups floats (both of this wave).  ids / weights [top] may be LDS or global.
+template <int PL>
 __device__ __forceinline__ void choose_experts(const Router &r, const float *logits, float *choice, float *group, int32_t *ids,
                                                float *weights) {
     const int lane = threadIdx.x & 63;
     const int size = r.experts / r.groups;
-    for (int e = lane; e < r.experts; e += 64) choice[e] = sigmoid_f32(logits[e]) + r.correction[e];
-    __builtin_amdgcn_wave_barrier();
-    __threadfence_block();
-    for (int g = lane; g < r.groups; g += 64) {
-        float a = -INFINITY, b = -INFINITY;   // the two largest
-        for (int i = 0; i < size; ++i) {
-            const float v = choice[g * size + i];
-            b = fmaxf(b, fminf(a, v));
-            a = fmaxf(a, v);
-        }
-        group[g] = size > 1 ? a + b : a;
-    }
-    __builtin_amdgcn_wave_barrier();
-    __threadfence_block();
-    // choice keys of this lane's experts; those outside the kept groups count as minus infinity
-    unsigned long long key[kPerLane];
+    float score[PL], c[PL];
 #pragma unroll
-    for (int j = 0; j < kPerLane; ++j) {
+    for (int j = 0; j < PL; ++j) {
         const int e = lane + 64 * j;
-        key[j] = 0;
+        score[j] = 0.f;
+        c[j] = -INFINITY;
         if (e < r.experts) {
+            score[j] = sigmoid_f32(logits[e]);
+            c[j] = score[j] + r.correction[e];
+            choice[e] = c[j];
+        }
+    }
+    if (r.groups > 1) {
+        __builtin_amdgcn_wave_barrier();
+        __threadfence_block();
+        for (int g = lane; g < r.groups; g += 64) {
+            float a = -INFINITY, b = -INFINITY;   // the two largest
+            for (int i = 0; i < size; ++i) {
+                const float v = choice[g * size + i];
+                b = fmaxf(b, fminf(a, v));
+                a = fmaxf(a, v);
+            }
+            group[g] = size > 1 ? a + b : a;
+        }
+        __builtin_amdgcn_wave_barrier();
+        __threadfence_block();
+        // experts outside the kept groups count as minus infinity
+#pragma unroll
+        for (int j = 0; j < PL; ++j) {
+            const int e = lane + 64 * j;
+            if (e >= r.experts) continue;
             const int g = e / size;
             const float mine = group[g];
             int better = 0;
@@ -54,32 +64,44 @@ __device__ __forceinline__ void choose_experts(const Router &r, const float *log
                 const float v = group[o];
                 better += v > mine || (v == mine && o < g);
             }
-            const float c = better < r.keep ? choice[e] : -INFINITY;
-            key[j] = ((unsigned long long)order_key(c) << 32) | (0xFFFFFFFFu - (uint32_t)e);
+            if (better >= r.keep) c[j] = -INFINITY;
         }
     }
     for (int s = 0; s < r.top; ++s) {
-        unsigned long long best = 0;
+        float best = c[0];
 #pragma unroll
-        for (int j = 0; j < kPerLane; ++j) best = key[j] > best ? key[j] : best;
-        best = wave_max_u64(best);
-        const int e = (int)(0xFFFFFFFFu - (uint32_t)(best & 0xFFFFFFFFull));
+        for (int j = 1; j < PL; ++j) best = fmaxf(best, c[j]);
+        best = wave_reduce<true>(best);
+        bool found = false;   // wave-uniform; the lowest index among equals: the first j, its lowest lane
 #pragma unroll
-        for (int j = 0; j < kPerLane; ++j)
-            if (key[j] == best) key[j] = 0;
-        if (lane == 0) {
-            ids[s] = e;
-            weights[s] = sigmoid_f32(logits[e]);
+        for (int j = 0; j < PL; ++j) {
+            const unsigned long long hit = found ? 0ull : __ballot(c[j] == best);
+            if (hit) {
+                found = true;
+                if (lane == __builtin_ctzll(hit)) {
+                    ids[s] = lane + 64 * j;
+                    weights[s] = score[j];
+                    c[j] = -INFINITY;
+                }
+            }
         }
     }
 }
 
+template <class F>
+auto with_lanes(int experts, F f) {
+    if (experts <= 64) return f(std::integral_constant<int, 1>());
+    if (experts <= 256) return f(std::integral_constant<int, 4>());
+    return f(std::integral_constant<int, kMaxExperts / 64>());
+}
+
+template <int PL>
 __global__ void __launch_bounds__(kMoeThreads) moe_select_kernel(const Router r, int tokens, int32_t *ids, float *weights) {
     extern __shared__ float select_lds[];
     const int wave = threadIdx.x >> 6, t = blockIdx.x * kMoeWaves + wave;
     if (t >= tokens) return;   // whole waves leave; no workgroup barrier below
     float *mine = select_lds + wave * (r.experts + r.groups);
-    choose_experts(r, r.logits + (size_t)t * r.ld, mine, mine + r.experts, ids + (size_t)t * r.top, weights + (size_t)t * r.top);
+    choose_experts<PL>(r, r.logits + (size_t)t * r.ld, mine, mine + r.experts, ids + (size_t)t * r.top, weights + (size_t)t * r.top);
 }
 
 // One workgroup: sort the entries by expert (counting sort) and cut every expert's run into tiles of bm entries.
@@ -118,7 +140,7 @@ __global__ void __launch_bounds__(1024) moe_plan_kernel(const int32_t *ids, int 
             row[2] = n - i * bm < bm ? n - i * bm : bm;
             row[3] = 0;
         }
-    for (int i = tile0[1024] + t; i < max_tiles; i += 1024) tiles[4 * i] = -1;
+    if (t == 0) tiles[4 * max_tiles] = tile0[1024];
     count[t] = 0;
     __syncthreads();
     for (int i = t; i < entries; i += 1024) {
@@ -139,7 +161,7 @@ struct MoeGemv {
 };
 
 // h[slot] = silu(gate x) * (up x); blockIdx.y = slot; a wave owns P neighbouring gate rows and the matching up rows
-template <class T, int P, int U>
+template <class T, int P, int U, int PL>
 __global__ void __launch_bounds__(kMoeThreads) moe_gate_up_gemv_kernel(const MoeGemv<T> p) {
     extern __shared__ __attribute__((aligned(16))) char moe_lds[];
     __shared__ int32_t ids[kMaxTop];
@@ -148,7 +170,7 @@ __global__ void __launch_bounds__(kMoeThreads) moe_gate_up_gemv_kernel(const Moe
     T *xs = reinterpret_cast<T *>(moe_lds);
     float *scratch = reinterpret_cast<float *>(xs + kl);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, slot = blockIdx.y;
-    if (wave == 0) choose_experts(p.r, p.r.logits, scratch, scratch + p.r.experts, ids, weights);
+    if (wave == 0) choose_experts<PL>(p.r, p.r.logits, scratch, scratch + p.r.experts, ids, weights);
     else {
         for (int i = 8 * (tid - 64); i < p.K; i += 8 * (kMoeThreads - 64)) store8(xs + i, load8(p.x + i));
         for (int i = p.K + 8 * (tid - 64); i < kl; i += 8 * (kMoeThreads - 64)) store8(xs + i, zero8<T>());
@@ -276,7 +298,10 @@ hipError_t gate_up(const Router &r, const void *x, const void *w, void *h, int32
         hipLaunchKernelGGL(kernel, grid, block, lds, stream, p);
         return hipGetLastError();
     };
-    return P == 1 ? run(&moe_gate_up_gemv_kernel<T, 1, 4>) : run(&moe_gate_up_gemv_kernel<T, 2, 2>);
+    return with_lanes(r.experts, [&](auto pl) {
+        constexpr int PL = decltype(pl)::value;
+        return P == 1 ? run(&moe_gate_up_gemv_kernel<T, 1, 4, PL>) : run(&moe_gate_up_gemv_kernel<T, 2, 2, PL>);
+    });
 }
 
 template <class T>
@@ -314,8 +339,11 @@ hipError_t launch_moe_down_gemv(int dtype, const void *h, const void *w_down, co
 
 hipError_t launch_moe_select(const Router &r, int tokens, int32_t *ids, float *weights, hipStream_t stream) {
     const size_t lds = (size_t)kMoeWaves * (r.experts + r.groups) * sizeof(float);
-    hipLaunchKernelGGL(moe_select_kernel, dim3((tokens + kMoeWaves - 1) / kMoeWaves), dim3(kMoeThreads), lds, stream, r, tokens, ids, weights);
-    return hipGetLastError();
+    return with_lanes(r.experts, [&](auto pl) {
+        hipLaunchKernelGGL(moe_select_kernel<decltype(pl)::value>, dim3((tokens + kMoeWaves - 1) / kMoeWaves), dim3(kMoeThreads), lds, stream, r, tokens,
+                           ids, weights);
+        return hipGetLastError();
+    });
 }
 
 int moe_max_tiles(int entries, int experts, int bm) { return entries / bm + (entries < experts ? entries : experts); }

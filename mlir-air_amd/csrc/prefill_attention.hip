@@ -62,17 +62,6 @@ constexpr size_t attn_lds_bytes() {
 
 // (This file is compiled with -fno-honor-nans: otherwise every MFMA result is canonicalised before it enters a
 // maximum, one more instruction per score.  A NaN in the inputs gives unspecified output values.)
-__device__ __forceinline__ float max2(float a, float b) { return fmaxf(a, b); }
-
-// max over the four lanes ql, ql + 16, ql + 32, ql + 48
-__device__ __forceinline__ float max_over_lane_groups(float v) {
-    const uint32_t u = __builtin_bit_cast(uint32_t, v);
-    const auto a = __builtin_amdgcn_permlane16_swap(u, u, false, false);   // rows (0, 1) and (2, 3) exchanged
-    v = max2(__builtin_bit_cast(float, (uint32_t)a[0]), __builtin_bit_cast(float, (uint32_t)a[1]));
-    const uint32_t w = __builtin_bit_cast(uint32_t, v);
-    const auto b = __builtin_amdgcn_permlane32_swap(w, w, false, false);   // halves exchanged
-    return max2(__builtin_bit_cast(float, (uint32_t)b[0]), __builtin_bit_cast(float, (uint32_t)b[1]));
-}
 
 template <int HD, int HPW>
 __global__ void __launch_bounds__(512) prefill_attn_kernel(const PrefillAttnParams p) {
