@@ -130,22 +130,20 @@ class SafetensorsDir:
     def __init__(self, path):
         from safetensors import safe_open
 
-        self._open = safe_open
         self.files = resolve_safetensor_files(path)
-        self._shard_of = {}   # tensor name -> the shard that holds it
+        self._shard_of = {}   # tensor name -> the open shard that holds it
         for file in self.files:
-            with safe_open(file, framework="pt") as f:
-                self._shard_of.update((key, file) for key in f.keys())
+            f = safe_open(file, framework="pt")
+            self._shard_of.update((key, f) for key in f.keys())
 
     def __contains__(self, key):
         return key in self._shard_of
 
     def tensor(self, key, what="weight", hint=""):
-        path = self._shard_of.get(key)
-        if path is None:
+        shard = self._shard_of.get(key)
+        if shard is None:
             raise KeyError(f"{what} {key} is in none of the {len(self.files)} safetensors shard(s){hint}")
-        with self._open(path, framework="pt") as f:
-            return f.get_tensor(key)
+        return shard.get_tensor(key)
 
 
 def load_weights_awq(model_name_or_path, config: Optional[LlamaConfig] = None, group_size=awq.GROUP) -> LlamaWeights:

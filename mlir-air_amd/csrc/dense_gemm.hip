@@ -213,15 +213,15 @@ hipError_t launch_tile(const GemmArgs &g, hipStream_t stream) {
 }  // namespace
 
 // Rows of A per tile for a product of `rows` rows with each of `matrices` matrices.  Measured: full of work, the 256 x 256
-// kernel runs at 1.22 PFLOP/s with one workgroup per CU, the 128 x 128 one at 1.0 with two; each loses what its last round
-// of workgroups leaves idle.  Experts with enough rows take the large tile (their tiles are rarely full in either case).
+// kernel runs at 1.22 PFLOP/s with one workgroup per CU, the 128 x 128 one at 0.9 to 1.0 with two; each loses what its last
+// round of workgroups leaves idle.  Experts with enough rows take the large tile (their tiles are rarely full in either case).
 int dense_gemm_tile_rows(int dtype, int rows, int N, int matrices) {
     if (rows <= 48 || N < 96) return 32;
     if (dtype != kBf16) return 128;
     if (matrices > 1) return rows >= 160 && N >= 256 ? 256 : 128;
     const int t256 = ((rows + 255) / 256) * ((N + 255) / 256), t128 = ((rows + 127) / 128) * ((N + 127) / 128);
     const float e256 = 1.22f * t256 / ((t256 + 255) / 256 * 256);
-    const float e128 = t128 < 512 ? 1.1f * t128 / 512 : (float)t128 / ((t128 + 255) / 256 * 256);
+    const float e128 = t128 < 512 ? 1.1f * t128 / 512 : 0.88f * t128 / ((t128 + 255) / 256 * 256);
     return e256 > e128 ? 256 : 128;
 }
 
