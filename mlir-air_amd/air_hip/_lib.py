@@ -5,6 +5,7 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 _LIB_PATH = os.path.join(os.path.dirname(_HERE), "lib", "libw4a16_hip.so")
+DENSE_ABI = 2
 _DENSE_PATH = os.path.join(os.path.dirname(_HERE), "lib", "libdense_lm_hip.so")
 
 OK = 0
@@ -94,7 +95,8 @@ class Router(ctypes.Structure):
 
 class GemmArgs(ctypes.Structure):
     _fields_ = [("a", _vp), ("w", _vp), ("out", _vp), ("lda", _i64), ("ldo", _i64), ("w_stride", _i64), ("tiles", _vp), ("order", _vp),
-                ("M", _i32), ("N", _i32), ("K", _i32), ("epilogue", _i32), ("n_tiles", _i32), ("gather", _i32), ("tile_rows", _i32)]
+                ("M", _i32), ("N", _i32), ("K", _i32), ("epilogue", _i32), ("n_tiles", _i32), ("gather", _i32), ("tile_rows", _i32),
+                ("silu_begin", _i32), ("silu_end", _i32)]
 
 
 class LatentShape(ctypes.Structure):
@@ -105,6 +107,31 @@ class LatentShape(ctypes.Structure):
 class LatentRows(ctypes.Structure):
     _fields_ = [("proj", _vp), ("lut", _vp), ("kv_norm", _vp), ("cache", _vp), ("pos_dev", _vp), ("ld", _i64), ("kv_off", _i32),
                 ("gate_off", _i32), ("M", _i32), ("pos", _i32), ("eps", _cf)]
+
+
+class RowOutput(ctypes.Structure):
+    _fields_ = [("silu_begin", _i32), ("silu_end", _i32), ("gate", _i32)]
+
+
+class HeadShape(ctypes.Structure):
+    _fields_ = [("heads", _i32), ("kv_heads", _i32), ("dim", _i32), ("vdim", _i32), ("true_dim", _i32), ("window", _i32), ("ring", _i32),
+                ("scale", _cf), ("out_scale", _cf)]
+
+
+class HeadRows(ctypes.Structure):
+    _fields_ = [("proj", _vp), ("q_norm", _vp), ("k_norm", _vp), ("cache", _vp), ("pos_dev", _vp), ("ld", _i64), ("off", _i32), ("M", _i32),
+                ("pos", _i32), ("eps", _cf)]
+
+
+class ShortConvArgs(ctypes.Structure):
+    _fields_ = [("proj", _vp), ("w", _vp), ("history", _vp), ("factors", _vp), ("pos_dev", _vp), ("ld", _i64), ("k_heads", _i32), ("heads", _i32),
+                ("dim", _i32), ("vdim", _i32), ("taps", _i32), ("off", _i32), ("M", _i32), ("pos", _i32), ("q_scale", _cf), ("unit_eps", _cf)]
+
+
+class RecurrenceArgs(ctypes.Structure):
+    _fields_ = [("qkv", _vp), ("log2_decay", _vp), ("z", _vp), ("a_log", _vp), ("dt_bias", _vp), ("factors", _vp), ("beta", _vp), ("state", _vp),
+                ("pos_dev", _vp), ("ld", _i64), ("ld_beta", _i64), ("k_heads", _i32), ("heads", _i32), ("dim", _i32), ("vdim", _i32),
+                ("q_off", _i32), ("k_off", _i32), ("v_off", _i32), ("M", _i32), ("pos", _i32)]
 
 
 DENSE_SYMBOLS = {
@@ -124,6 +151,19 @@ DENSE_SYMBOLS = {
     "dlm_embed_rows": (_ci, [_ci, _vp, _vp, _cf, _vp, _vp, _ci, _ci, _vp]),
     "dlm_residual_norm_rows": (_ci, [_ci, _vp, _vp, _vp, _ci, _vp, _cf, _ci, _vp, _ci, _ci, _vp]),
     "dlm_norm_rows": (_ci, [_ci, _vp, _vp, _vp, _cf, _ci, _vp, _ci, _ci, _vp]),
+    "dlm_gemv_act": (_ci, [_ci] + [_vp] * 4 + [_ci, _ci, _vp]),
+    "dlm_add_norm_rows": (_ci, [_ci] + [_vp] * 4 + [_cf, _vp, _cf, _ci, _vp, _ci, _ci, _vp]),
+    "dlm_head_decode_supported": (_ci, [_ci, _vp]),
+    "dlm_head_prefill_supported": (_ci, [_ci, _vp]),
+    "dlm_head_prepare": (_ci, [_ci] + [_vp] * 4),
+    "dlm_head_prefill": (_ci, [_ci] + [_vp] * 4 + [_i64, _vp]),
+    "dlm_head_decode": (_ci, [_ci] + [_vp] * 3 + [_ci] + [_vp] * 3),
+    "dlm_head_merge": (_ci, [_ci, _vp, _vp, _ci] + [_vp] * 3 + [_i64, _vp]),
+    "dlm_short_conv": (_ci, [_ci] + [_vp] * 3),
+    "dlm_recurrence_steps": (_ci, [_ci] + [_vp] * 3),
+    "dlm_recurrence_chunk_bytes": (_sz, [_vp]),
+    "dlm_recurrence_chunks": (_ci, [_ci] + [_vp] * 4),
+    "dlm_gated_norm": (_ci, [_ci, _vp, _vp, _vp, _i64, _vp, _i64] + [_ci] * 4 + [_cf, _vp]),
     "dlm_latent_decode_supported": (_ci, [_ci, _vp]),
     "dlm_latent_prefill_supported": (_ci, [_ci, _vp]),
     "dlm_latent_prepare": (_ci, [_ci, _vp, _vp, _vp]),
@@ -179,8 +219,8 @@ def load_dense_library():
             raise LibraryNotBuiltError(f"{_DENSE_PATH} is missing: build it with `python mlir-air_amd/build.py --only dense_lm` "
                                        "(there is no CPU fallback)")
         lib = _bind(_DENSE_PATH, DENSE_SYMBOLS)
-        if lib.dlm_abi_version() != 1:
-            raise LibraryNotBuiltError(f"{_DENSE_PATH}: ABI version {lib.dlm_abi_version()} != 1, rebuild")
+        if lib.dlm_abi_version() != DENSE_ABI:
+            raise LibraryNotBuiltError(f"{_DENSE_PATH}: ABI version {lib.dlm_abi_version()} != {DENSE_ABI}, rebuild")
         _dense = lib
     return _dense
 

@@ -18,7 +18,10 @@ HEAD_PAD = 32    # parts of a head
 ROW_PAD = 16     # output lengths
 
 PLAIN, RESIDUAL, EMBED, FINAL = 0, 1, 2, 3
-OUT_ELEM, OUT_F32, OUT_SWIGLU = 0, 1, 2
+NORMED = 4
+OUT_ELEM, OUT_F32, OUT_SWIGLU, OUT_GEGLU = 0, 1, 2, 3
+GATE_NONE, GATE_SILU, GATE_GELU = 0, 1, 2
+STATE_PAD = 64   # a recurrence's query / key size
 
 
 def pad_to(n, k):
@@ -117,6 +120,42 @@ def gemv_final(r, final_w, w, keys=None, n_valid=0):
     return _gemv(w, intake, True, keys, n_valid, w.device)
 
 
+class Sum:
+    """The residual stream of one token in front of a sublayer that norms its input: fp32 `res`, and the previous sublayer's output
+    `y` (or None), still to be added; or, in front of the first layer, the embedding row of a token."""
+
+    __slots__ = ("res", "y", "token", "embed", "scale")
+
+    def __init__(self, res=None, y=None, token=None, embed=None, scale=1.0):
+        self.res, self.y, self.token, self.embed, self.scale = res, y, token, embed, scale
+
+
+def gemv_normed(s, norm_w, eps, width, w, silu=None, gate=GATE_NONE, out_f32=False, keys=None, n_valid=0, keep=True):
+    """The Sum `s` brought up to date, normed with norm_w, times W.  `silu`: a range of rows that silu is applied to; `gate`: W holds
+    interleaved gate and up rows (16 each) and the result is their gated half.  Returns (y, the sum fp32 [K] with `keep`)."""
+    lib = _lib.load_dense_library()
+    _need_cuda(norm_w, w)
+    _need_f32(s.res, s.y, norm_w)
+    N, K = w.shape
+    if norm_w.numel() != K or any(t is not None and t.numel() != K for t in (s.res, s.y)) or (s.embed is not None and s.embed.shape[1] != K):
+        raise ValueError(f"gemv_normed: the stream and the norm weight must have {K} elements")
+    _same("gemv_normed", w, s.embed)
+    if s.token is not None and s.token.dtype != torch.int32:
+        raise TypeError("gemv_normed takes an int32 token")
+    res = torch.empty((K,), dtype=torch.float32, device=w.device) if keep else None
+    intake = _lib.Intake(mode=NORMED, width=width, eps=eps, scale=s.scale, res=_opt(s.res), y=_opt(s.y), final_w=_ptr(norm_w), res_out=_opt(res),
+                         embed=_opt(s.embed), token=_opt(s.token))
+    if gate == GATE_NONE and silu is None:
+        return _gemv(w, intake, out_f32, keys, n_valid, w.device), res
+    if out_f32 or keys is not None:
+        raise ValueError("gemv_normed: activations come in the element type and without keys")
+    out = torch.empty((N // 2 if gate else N,), dtype=w.dtype, device=w.device)
+    begin, end = silu or (0, 0)
+    ro = _lib.RowOutput(silu_begin=begin, silu_end=end, gate=gate)
+    _lib.check_dense(lib.dlm_gemv_act(dtype_code(w), _ptr(w), ctypes.byref(intake), ctypes.byref(ro), _ptr(out), K, N, _stream()))
+    return out, res
+
+
 def new_keys(w):
     """Argmax keys of a one-token product with W."""
     n = _lib.load_dense_library().dlm_gemv_keys(w.shape[1], w.shape[0])
@@ -132,8 +171,8 @@ def argmax(keys, token=None, position=None, history=None):
     _lib.check_dense(lib.dlm_argmax(_ptr(keys), keys.numel(), _opt(token), _opt(position), _opt(history), _stream()))
 
 
-def gemm(a, w, out_f32=False, lda=None, rows=None, out=None):
-    """out[M, N] = A[M, K] W[N, K]^T; a: [M, >= K] with row stride `lda` (default: its width)."""
+def gemm(a, w, out_f32=False, lda=None, rows=None, out=None, silu=None, gate=GATE_NONE):
+    """out[M, N] = A[M, K] W[N, K]^T; a: [M, >= K] with row stride `lda` (default: its width).  `silu`, `gate` as in gemv_normed."""
     lib = _lib.load_dense_library()
     _need_cuda(w)
     _same("gemm", w, a)
@@ -142,12 +181,22 @@ def gemm(a, w, out_f32=False, lda=None, rows=None, out=None):
     lda = a.stride(0) if lda is None else lda
     if not a.is_cuda or a.stride(-1) != 1 or a.shape[1] < K or M > a.shape[0]:
         raise ValueError(f"gemm: A must be a GPU matrix with at least {K} columns and {M} rows")
+    width = N // 2 if gate else N
     if out is None:
-        out = torch.empty((M, N), dtype=torch.float32 if out_f32 else w.dtype, device=w.device)
-    g = _lib.GemmArgs(a=_ptr(a), w=_ptr(w), out=_ptr(out), lda=lda, ldo=N, M=M, N=N, K=K, epilogue=OUT_F32 if out_f32 else OUT_ELEM,
+        out = torch.empty((M, width), dtype=torch.float32 if out_f32 else w.dtype, device=w.device)
+    begin, end = silu or (0, 0)
+    epilogue = OUT_F32 if out_f32 else {GATE_NONE: OUT_ELEM, GATE_SILU: OUT_SWIGLU, GATE_GELU: OUT_GEGLU}[gate]
+    g = _lib.GemmArgs(a=a.data_ptr(), w=_ptr(w), out=_ptr(out), lda=lda, ldo=width, M=M, N=N, K=K, epilogue=epilogue, silu_begin=begin, silu_end=end,
                       tile_rows=lib.dlm_gemm_tile_rows(dtype_code(w), M, N, 1))
     _lib.check_dense(lib.dlm_gemm(dtype_code(w), ctypes.byref(g), _stream()))
     return out
+
+
+def product(a, w, out_f32=False):
+    """gemm, or the one-token product for a single row."""
+    if a.shape[0] == 1:
+        return gemv(a.reshape(-1), w, out_f32).reshape(1, -1)
+    return gemm(a, w, out_f32)
 
 
 def embed_rows(tokens, embed, scale):
@@ -176,6 +225,23 @@ def residual_norm_rows(res, y, norm_w, eps, width, dtype, weights=None):
     h = torch.empty((M, K), dtype=dtype, device=res.device)
     _lib.check_dense(lib.dlm_residual_norm_rows(dtype_code(dtype), _ptr(res), _ptr(y), _opt(weights), top, _ptr(norm_w), eps, width, _ptr(h), M, K,
                                                 _stream()))
+    return h
+
+
+def add_norm_rows(res, y, norm_w, eps, width, dtype, tokens=None, embed=None, scale=1.0):
+    """The residual rows brought up to date in place - res + y (y fp32 [M, K] or None), or with `tokens` the embedding rows times
+    `scale` - and their norm in the element type (None without norm_w)."""
+    lib = _lib.load_dense_library()
+    _need_cuda(res)
+    _need_f32(res, y, norm_w)
+    M, K = res.shape
+    if (y is not None and tuple(y.shape) != (M, K)) or (norm_w is not None and norm_w.numel() != K):
+        raise ValueError("add_norm_rows: shapes of the residual, y and the norm weight do not match")
+    if tokens is not None and (tokens.dtype != torch.int32 or tokens.numel() != M or embed.shape[1] != K or embed.dtype != dtype or y is not None):
+        raise ValueError("add_norm_rows: int32 tokens, one per row, and an embedding of the rows' width")
+    h = None if norm_w is None else torch.empty((M, K), dtype=dtype, device=res.device)
+    _lib.check_dense(lib.dlm_add_norm_rows(dtype_code(dtype), _ptr(res), _opt(y), _opt(tokens), _opt(embed), scale, _opt(norm_w), eps, width, _opt(h), M, K,
+                                           _stream()))
     return h
 
 
@@ -361,3 +427,161 @@ def latent_attention_absorbed(spec, proj, kv_off, gate_off, lut, kv_norm, eps, c
     _lib.check_dense(lib.dlm_latent_combine(dt, s, rr, nsplit, _ptr(part_o), _ptr(part_ml), _ptr(sink), _ptr(w_uv), _ptr(out), out.shape[1],
                                             _stream()))
     return out
+
+
+class HeadSpec:
+    """Sizes of one windowed attention of grouped heads: true and padded."""
+
+    __slots__ = ("heads", "kv_heads", "dim", "vdim", "window", "scale", "out_scale", "dim_p", "vdim_p")
+
+    def __init__(self, heads, kv_heads, dim, vdim, window, scale, out_scale=1.0):
+        self.heads, self.kv_heads, self.dim, self.vdim, self.window, self.scale, self.out_scale = heads, kv_heads, dim, vdim, window, scale, out_scale
+        self.dim_p, self.vdim_p = pad_to(dim, HEAD_PAD), pad_to(vdim, HEAD_PAD)
+
+    @property
+    def proj_width(self):
+        return (self.heads + self.kv_heads) * self.dim_p + self.kv_heads * self.vdim_p
+
+    def ring(self, capacity, portion):
+        """Cache rows for a sequence of `capacity` tokens that come in portions of at most `portion`."""
+        rows = capacity if portion is None else min(capacity, self.window - 1 + portion)
+        return pad_to(rows, 64)
+
+    def shape(self, ring):
+        return _lib.HeadShape(heads=self.heads, kv_heads=self.kv_heads, dim=self.dim_p, vdim=self.vdim_p, true_dim=self.dim,
+                              window=min(self.window, 1 << 30), ring=ring, scale=self.scale, out_scale=self.out_scale)
+
+    def decode_supported(self, dtype):
+        return bool(_lib.load_dense_library().dlm_head_decode_supported(dtype_code(dtype), ctypes.byref(self.shape(64))))
+
+    def prefill_supported(self, dtype):
+        return bool(_lib.load_dense_library().dlm_head_prefill_supported(dtype_code(dtype), ctypes.byref(self.shape(64))))
+
+
+def head_splits(spec, M, total):
+    """How many workgroups share the keys of 16 query rows of a key / value head: enough of them to fill the GPU twice, as far as
+    there are blocks of 32 keys."""
+    tiles = spec.kv_heads * ((M * (spec.heads // spec.kv_heads) + 15) // 16)
+    blocks = (min(total, spec.window + M - 1) + 31) // 32 + 1
+    return max(1, min(256, 512 // tiles, blocks))
+
+
+def head_attention(spec, proj, off, q_norm, k_norm, eps, cache, pos, out, pos_dev=None, nsplit=None, rows_form=False):
+    """Windowed attention of the rows of proj [M, ld] (q, k, v from column `off` on) at positions pos .. into the first columns of
+    out [M, ldo]; their keys and values are appended to cache [kv_heads, ring, dim + vdim].  rows_form: the kernel for many rows."""
+    lib = _lib.load_dense_library()
+    _need_cuda(cache, q_norm, k_norm)
+    _same("head attention", cache, proj, out)
+    _need_f32(q_norm, k_norm)
+    M, dt = proj.shape[0], dtype_code(proj)
+    if tuple(cache.shape[::2]) != (spec.kv_heads, spec.dim_p + spec.vdim_p) or out.shape[0] != M or proj.shape[1] < off + spec.proj_width:
+        raise ValueError("head attention: the cache, the projections or the output have another shape")
+    if q_norm.numel() != spec.dim_p or k_norm.numel() != spec.dim_p:
+        raise ValueError(f"head attention: the norm weights must have {spec.dim_p} elements")
+    s = spec.shape(cache.shape[1])
+    r = _lib.HeadRows(proj=proj.data_ptr(), q_norm=_ptr(q_norm), k_norm=_ptr(k_norm), cache=_ptr(cache), pos_dev=_opt(pos_dev), ld=proj.stride(0), off=off, M=M,
+                      pos=pos, eps=eps)
+    q = torch.empty((M * spec.heads, spec.dim_p), dtype=proj.dtype, device=proj.device)
+    s, r = ctypes.byref(s), ctypes.byref(r)
+    _lib.check_dense(lib.dlm_head_prepare(dt, s, r, _ptr(q), _stream()))
+    if rows_form:
+        _lib.check_dense(lib.dlm_head_prefill(dt, s, r, _ptr(q), out.data_ptr(), out.stride(0), _stream()))
+        return
+    if nsplit is None:
+        nsplit = head_splits(spec, M, pos + M)
+    part_o = torch.empty((M * spec.heads, nsplit, spec.vdim_p), dtype=torch.float32, device=proj.device)
+    part_ml = torch.empty((M * spec.heads, nsplit, 2), dtype=torch.float32, device=proj.device)
+    _lib.check_dense(lib.dlm_head_decode(dt, s, r, _ptr(q), nsplit, _ptr(part_o), _ptr(part_ml), _stream()))
+    _lib.check_dense(lib.dlm_head_merge(dt, s, r, nsplit, _ptr(part_o), _ptr(part_ml), out.data_ptr(), out.stride(0), _stream()))
+
+
+class StateSpec:
+    """Sizes of one linear recurrence over a matrix state per head: true and padded."""
+
+    __slots__ = ("heads", "k_heads", "dim", "vdim", "dim_p", "vdim_p")
+
+    def __init__(self, heads, k_heads, dim, vdim):
+        self.heads, self.k_heads, self.dim, self.vdim = heads, k_heads, dim, vdim
+        self.dim_p, self.vdim_p = pad_to(dim, STATE_PAD), pad_to(vdim, HEAD_PAD)
+
+    @property
+    def qk_width(self):
+        return self.k_heads * self.dim_p
+
+    @property
+    def v_width(self):
+        return self.heads * self.vdim_p
+
+    @property
+    def channels(self):
+        return 2 * self.qk_width + self.v_width
+
+    def new_state(self, device):
+        return torch.zeros((self.heads, self.vdim_p, self.dim_p), dtype=torch.float32, device=device)
+
+
+def short_conv(spec, proj, off, w, history, pos, q_scale, unit_eps, pos_dev=None):
+    """(act [M, channels], factors [M, 2 k_heads]) of the channels of proj [M, ld] from column `off` on; w fp32 [taps, channels],
+    history [taps, channels] is brought forward."""
+    lib = _lib.load_dense_library()
+    _need_cuda(w, history)
+    _need_f32(w)
+    _same("short_conv", history, proj)
+    M, C = proj.shape[0], spec.channels
+    if w.shape[1] != C or history.shape != w.shape or proj.shape[1] < off + C:
+        raise ValueError(f"short_conv: projections, filters and history must have {C} channels")
+    act = torch.empty((M, C), dtype=proj.dtype, device=proj.device)
+    factors = torch.empty((M, 2 * spec.k_heads), dtype=torch.float32, device=proj.device)
+    c = _lib.ShortConvArgs(proj=proj.data_ptr(), w=_ptr(w), history=_ptr(history), factors=_ptr(factors), pos_dev=_opt(pos_dev), ld=proj.stride(0),
+                           k_heads=spec.k_heads, heads=spec.heads, dim=spec.dim_p, vdim=spec.vdim_p, taps=w.shape[0], off=off, M=M, pos=pos, q_scale=q_scale,
+                           unit_eps=unit_eps)
+    _lib.check_dense(lib.dlm_short_conv(dtype_code(proj), ctypes.byref(c), _ptr(act), _stream()))
+    return act, factors
+
+
+# Up to this many tokens a portion goes through a recurrence token by token.
+STEPS_MAX_TOKENS = 16
+
+
+def recurrence(spec, qkv, offsets, state, pos, log2_decay=None, z=None, a_log=None, dt_bias=None, factors=None, beta=None, pos_dev=None, chunks=None):
+    """Read-outs fp32 [M, heads * vdim_p] of the tokens of qkv [M, ld] (q, k, v at the column `offsets`); `state` is brought forward.
+    log2_decay [heads]: a decay per head; z [M, heads * dim_p] with a_log, dt_bias, factors and beta [M, >= heads]: a decay per channel
+    and the delta rule.  chunks: which form to run (default: by the number of tokens)."""
+    lib = _lib.load_dense_library()
+    _need_cuda(state)
+    _need_f32(state, log2_decay, z, a_log, dt_bias, factors)
+    M, H = qkv.shape[0], spec.heads
+    if tuple(state.shape) != (H, spec.vdim_p, spec.dim_p) or qkv.stride(1) != 1:
+        raise ValueError("recurrence: the state has another shape")
+    if z is None:
+        if log2_decay.numel() != H:
+            raise ValueError(f"recurrence: {H} decays")
+    elif tuple(z.shape) != (M, H * spec.dim_p) or a_log.numel() != H or dt_bias.numel() != H * spec.dim_p or tuple(factors.shape) != (M, 2 * spec.k_heads) \
+            or beta.shape[0] != M or beta.shape[1] < H or beta.dtype != qkv.dtype:
+        raise ValueError("recurrence: shapes of the decay, the factors or beta do not match")
+    a = _lib.RecurrenceArgs(qkv=qkv.data_ptr(), log2_decay=_opt(log2_decay), z=_opt(z), a_log=_opt(a_log), dt_bias=_opt(dt_bias), factors=_opt(factors),
+                            beta=_opt(beta), state=_ptr(state), pos_dev=_opt(pos_dev), ld=qkv.stride(0), ld_beta=0 if beta is None else beta.stride(0),
+                            k_heads=spec.k_heads, heads=H, dim=spec.dim_p, vdim=spec.vdim_p, q_off=offsets[0], k_off=offsets[1], v_off=offsets[2], M=M, pos=pos)
+    o = torch.empty((M, spec.v_width), dtype=torch.float32, device=qkv.device)
+    nbytes = lib.dlm_recurrence_chunk_bytes(ctypes.byref(a))
+    if chunks is None:
+        chunks = M > STEPS_MAX_TOKENS and nbytes > 0
+    if chunks:
+        work = torch.empty((nbytes,), dtype=torch.uint8, device=qkv.device)
+        _lib.check_dense(lib.dlm_recurrence_chunks(dtype_code(qkv), ctypes.byref(a), _ptr(work), _ptr(o), _stream()))
+    else:
+        _lib.check_dense(lib.dlm_recurrence_steps(dtype_code(qkv), ctypes.byref(a), _ptr(o), _stream()))
+    return o
+
+
+def gated_norm(o, w, eps, groups, true_cols, gate, out):
+    """out[:, :groups * cols] = o / rms * w * sigmoid(gate) with the mean over the true_cols of a group's columns; w fp32 [cols]."""
+    lib = _lib.load_dense_library()
+    _need_cuda(o, w)
+    _need_f32(o, w)
+    _same("gated_norm", out, gate)
+    M, cols = o.shape[0], o.shape[1] // groups
+    if w.numel() != cols or out.shape[0] != M or gate.shape[0] != M or min(out.shape[1], gate.shape[1]) < groups * cols:
+        raise ValueError("gated_norm: shapes do not match")
+    _lib.check_dense(lib.dlm_gated_norm(dtype_code(gate), _ptr(o), _ptr(w), gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), M, groups, cols,
+                                        true_cols, eps, _stream()))

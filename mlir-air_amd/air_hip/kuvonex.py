@@ -18,7 +18,8 @@ from typing import List, Optional
 import numpy as np
 import torch
 
-from . import dense, generation, weights as wmod
+from . import dense
+from .dense_model import DenseModel, SequenceCache, place as _place
 
 # Up to this many tokens a portion attends over the latents: expanding keys and values of the whole cache costs
 # rank * (dim + vdim) per cached token and head whatever the portion's length, the latent form (2 rank + rot) instead
@@ -136,15 +137,6 @@ class KuvonexLayer:
     w_down: Optional[torch.Tensor] = None
 
 
-def _place(t, shape):
-    """t in the corner of a zero tensor of `shape`."""
-    if tuple(t.shape) == tuple(shape):
-        return t
-    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
-    out[tuple(slice(0, n) for n in t.shape)] = t
-    return out
-
-
 def prepare_layer(config, i, tensor, dtype=torch.bfloat16, device="cuda"):
     """Layer i from `tensor(name, shape)` (checkpoint orientation [out, in]) in the kernels' form."""
     l, p = config.layers[i], f"l{i}."
@@ -197,25 +189,20 @@ def rotation_table(base, dims, n, device):
     return torch.from_numpy(np.stack([np.cos(a), np.sin(a)], axis=-1).astype(np.float32)).to(device)
 
 
-class LatentCache:
+class LatentCache(SequenceCache):
     """Latent rows of one sequence: one matrix [capacity, rank + rot] per layer that has a latent of its own (layers that
-    share one have no entry), the number of tokens in it, and what a captured decode step keeps on the device."""
+    share one have no entry)."""
 
     def __init__(self, model, capacity):
-        self.capacity, self.pos = capacity, 0
+        super().__init__(model, capacity)
         dev = model.device
         self.rows = {i: torch.empty((capacity, l.spec.cache_width), dtype=model.dtype, device=dev) for i, l in enumerate(model.layers) if l.source == i}
-        self.token = torch.zeros((1,), dtype=torch.int32, device=dev)
-        self.position = torch.zeros((1,), dtype=torch.int32, device=dev)
-        self.history = torch.zeros((capacity + 1,), dtype=torch.int32, device=dev)
-        self.graph = None
         self.tables = {(l.rot_base, l.spec.rot): model.rotation(l.rot_base, l.spec.rot, capacity) for l in model.layers}
 
-    def reset(self):
-        self.pos = 0
 
+class KuvonexModel(DenseModel):
+    config_class = KuvonexConfig
 
-class KuvonexModel(generation.CausalLM):
     def __init__(self, config, tensor, dtype=torch.bfloat16, device="cuda"):
         """`tensor(name, shape)` gives the checkpoint's tensors (any device)."""
         dense.dtype_code(dtype)
@@ -234,18 +221,6 @@ class KuvonexModel(generation.CausalLM):
             if not (l.spec.decode_supported(dtype) or l.spec.prefill_supported(dtype)):
                 raise ValueError(f"layer {i}: no attention kernel for these head and latent sizes")
         self._tables = {}
-
-    @classmethod
-    def load(cls, path, config_json, dtype=torch.bfloat16, device="cuda"):
-        shards = wmod.SafetensorsDir(path)
-
-        def tensor(name, shape):
-            t = shards.tensor(name)
-            if tuple(t.shape) != tuple(shape):
-                raise ValueError(f"{name}: shape {tuple(t.shape)}, the configuration gives {tuple(shape)}")
-            return t
-
-        return cls(KuvonexConfig.from_json(config_json), tensor, dtype, device)
 
     def new_cache(self, max_tokens):
         return LatentCache(self, max_tokens)
@@ -304,97 +279,15 @@ class KuvonexModel(generation.CausalLM):
                 trace.append(res.clone())
         return res
 
-    def _ids(self, tokens):
-        if isinstance(tokens, torch.Tensor):   # already on the device: the caller answers for the range
-            return tokens.to(device=self.device, dtype=torch.int32).contiguous()
-        tokens = [int(t) for t in tokens]
-        if not tokens or min(tokens) < 0 or max(tokens) >= self.vocab:
-            raise ValueError(f"token ids must lie in 0 .. {self.vocab - 1}")
-        return torch.tensor(tokens, dtype=torch.int32, device=self.device)
+    def _pending(self, res):
+        return dense.Residual(res, None, None, self.config.eps, self.config.width)
 
-    def _advance(self, cache, n):
-        if cache.pos + n > cache.capacity:
-            raise ValueError(f"the sequence needs {cache.pos + n} tokens, its cache holds {cache.capacity}")
-        pos, cache.pos = cache.pos, cache.pos + n
-        return pos
+    def _head(self, r, keys=None):
+        return dense.gemv_final(r, self.final_norm, self.head, keys, self.vocab)
 
-    def _last_logits(self, res):
-        """(logits, greedy token) of the last row of a residual."""
-        r = dense.Residual(res[-1].contiguous(), None, None, self.config.eps, self.config.width)
-        return self._tail(r)
-
-    def _tail(self, r):
-        keys = dense.new_keys(self.head)
-        logits = dense.gemv_final(r, self.final_norm, self.head, keys, self.vocab)
-        best = torch.empty((1,), dtype=torch.int32, device=self.device)
-        dense.argmax(keys, best)
-        return logits[:self.vocab], best
-
-    # -- generation.CausalLM ---------------------------------------------------------------
-    def step(self, cache, tokens, want, trace=None):
+    def _head_rows(self, res, rows):
         c = self.config
-        ids = self._ids(tokens)
-        pos = self._advance(cache, len(ids))
-        if len(ids) == 1 and trace is None:
-            r = self._one_token(cache, ids, pos)
-            if not want:
-                return torch.empty((0, self.vocab), device=self.device)
-            logits = dense.gemv_final(r, self.final_norm, self.head)
-            return logits[:self.vocab].reshape(1, -1).expand(len(want), -1)
-        res = self._rows(cache, ids, pos, trace)
-        if not want:
-            return torch.empty((0, self.vocab), device=self.device)
-        rows = torch.tensor(list(want), dtype=torch.int32, device=self.device)
-        return dense.gemm(dense.norm_rows(res, self.final_norm, c.eps, c.width, self.dtype, rows), self.head, out_f32=True)[:, :self.vocab]
+        return dense.gemm(dense.norm_rows(res, self.final_norm, c.eps, c.width, self.dtype, rows), self.head, out_f32=True)
 
-    def prefill(self, cache, tokens):
-        ids = self._ids(tokens)
-        pos = self._advance(cache, len(ids))
-        if len(ids) == 1:
-            return self._tail(self._one_token(cache, ids, pos))
-        return self._last_logits(self._rows(cache, ids, pos))
-
-    def decode_token(self, cache, token):
-        pos = self._advance(cache, 1)
-        return self._tail(self._one_token(cache, self._ids([token]), pos))
-
-    def _greedy_step(self, cache):
-        """The token and position kept on the device -> the next token and position there."""
-        r = self._one_token(cache, cache.token, 0, cache.position)
-        keys = dense.new_keys(self.head)
-        dense.gemv_final(r, self.final_norm, self.head, keys, self.vocab)
-        dense.argmax(keys, cache.token, cache.position, cache.history)
-
-    def decode_greedy(self, cache, first, n_tokens):
-        """The step is captured as a HIP graph the first time a cache decodes (token and position live on the device)
-        and replayed per token; inside a caller's capture the launches are recorded one by one."""
-        start = self._advance(cache, n_tokens)
-        if not all(l.spec.decode_supported(self.dtype) for l in self.layers):
-            return self._decode_eagerly(cache, first, start, n_tokens)
-        capturing = torch.cuda.is_current_stream_capturing()
-        cache.token.copy_(first.to(torch.int32).reshape(1))
-        cache.position.fill_(start)
-        if capturing:
-            for _ in range(n_tokens):
-                self._greedy_step(cache)
-        elif n_tokens > 0:
-            if cache.graph is None:
-                self._greedy_step(cache)    # the first token runs as it is: nothing is set up for the first time in the capture
-                n_tokens -= 1
-                torch.cuda.synchronize()
-                cache.graph = torch.cuda.CUDAGraph()
-                with torch.cuda.graph(cache.graph):
-                    self._greedy_step(cache)
-            for _ in range(n_tokens):
-                cache.graph.replay()
-        return cache.history[start + 1:cache.pos + 1].clone()
-
-    def _decode_eagerly(self, cache, first, start, n_tokens):
-        out, tok = [], first.to(torch.int32).reshape(1)
-        for i in range(n_tokens):
-            _, tok = self._tail(self._one_token(cache, tok, start + i))
-            out.append(tok)
-        return torch.cat(out) if out else torch.empty((0,), dtype=torch.int32, device=self.device)
-
-    def check_health(self):
-        torch.cuda.synchronize()
+    def _captured_decode(self):
+        return all(l.spec.decode_supported(self.dtype) for l in self.layers)

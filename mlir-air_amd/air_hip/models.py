@@ -22,6 +22,7 @@ class Entry:
 REGISTRY = {
     "LlamaForCausalLM": Entry("decode", "LlamaModel", "w4a16"),
     "Kuvonex": Entry("kuvonex", "KuvonexModel", "dense_lm"),
+    "Sitirax": Entry("sitirax", "SitiraxModel", "dense_lm"),
 }
 
 

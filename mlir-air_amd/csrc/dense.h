@@ -154,6 +154,14 @@ __device__ __forceinline__ Vec8<float> pair8<float>(floatx4 a, floatx4 b) { retu
 
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float gelu_tanh_f32(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * z * z, z, z))); }
+__device__ __forceinline__ float softplus_f32(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+
+// sum over a group of `n` neighbouring lanes (a power of two), every lane of it receiving the sum
+__device__ __forceinline__ float group_sum(float v, int n) {
+    for (int m = 1; m < n; m <<= 1) v += __shfl_xor(v, m, 64);
+    return v;
+}
 
 // float -> unsigned key of the same order (-0 counts as +0)
 __device__ __forceinline__ uint32_t order_key(float v) {

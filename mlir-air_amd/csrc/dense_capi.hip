@@ -46,6 +46,100 @@ LatentRows rows_of(const dlm_latent_rows *r) {
     return {r->proj, (long)r->ld, r->kv_off, r->gate_off, r->lut, r->kv_norm, r->eps, r->cache, r->M, r->pos_dev, r->pos};
 }
 
+int check_head(int dtype, const dlm_head_shape *s, const dlm_head_rows *r) {
+    if (!s || !r || !r->proj || !r->cache || !r->q_norm || !r->k_norm) return DLM_ERR_NULL;
+    if (bad_type(dtype) || s->heads <= 0 || s->kv_heads <= 0 || s->heads % s->kv_heads || s->dim <= 0 || s->dim % 32 || s->vdim <= 0 || s->vdim % 32 ||
+        s->true_dim <= 0 || s->true_dim > s->dim || s->window <= 0 || s->ring <= 0 || s->ring % 64 || !(s->scale > 0.f) || r->M <= 0 || r->M > 65535 || r->pos < 0 ||
+        r->ld % 8 || r->off < 0 || r->off % 8 || !(r->eps >= 0.f) || r->M > s->ring)
+        return DLM_ERR_SHAPE;
+    // keys that are still seen must not share a row with new ones
+    if (!r->pos_dev && (int64_t)r->pos + r->M > s->ring && (int64_t)s->window - 1 + r->M > s->ring) return DLM_ERR_SHAPE;
+    if (odd(r->proj) || odd(r->cache) || odd(r->q_norm) || odd(r->k_norm)) return DLM_ERR_ALIGN;
+    return DLM_OK;
+}
+HeadShape head_of(const dlm_head_shape *s) {
+    return {s->heads, s->kv_heads, s->dim, s->vdim, s->true_dim, s->window, s->ring, s->scale, s->out_scale};
+}
+HeadRows head_rows_of(const dlm_head_rows *r) {
+    return {r->proj, (long)r->ld, r->off, r->q_norm, r->k_norm, r->eps, r->cache, r->M, r->pos_dev, r->pos};
+}
+
+int check_recurrence(int dtype, const dlm_recurrence_args *a) {
+    if (!a || !a->qkv || !a->state || (!a->log2_decay) == (!a->z)) return DLM_ERR_NULL;
+    if (a->z && (!a->a_log || !a->dt_bias || !a->factors || !a->beta)) return DLM_ERR_NULL;
+    if (bad_type(dtype) || a->heads <= 0 || a->k_heads <= 0 || a->heads % a->k_heads || a->heads > 65535 || a->dim <= 0 || a->dim % 64 || a->dim > kMaxStateDim ||
+        a->vdim <= 0 || a->vdim % 32 || a->M <= 0 || a->pos < 0 || a->ld % 8 || a->q_off < 0 || a->q_off % 8 || a->k_off < 0 || a->k_off % 8 || a->v_off < 0 ||
+        a->v_off % 8)
+        return DLM_ERR_SHAPE;
+    if (odd(a->qkv) || odd(a->state) || odd(a->z) || odd(a->dt_bias)) return DLM_ERR_ALIGN;
+    return DLM_OK;
+}
+LinearArgs linear_of(const dlm_recurrence_args *a) {
+    LinearArgs l;
+    l.k_heads = a->k_heads;
+    l.heads = a->heads;
+    l.dim = a->dim;
+    l.vdim = a->vdim;
+    l.qkv = a->qkv;
+    l.ld = a->ld;
+    l.q_off = a->q_off;
+    l.k_off = a->k_off;
+    l.v_off = a->v_off;
+    l.log2_decay = a->log2_decay;
+    l.z = a->z;
+    l.a_log = a->a_log;
+    l.dt_bias = a->dt_bias;
+    l.factors = a->factors;
+    l.beta = a->beta;
+    l.ld_beta = a->ld_beta;
+    l.state = a->state;
+    l.M = a->M;
+    l.pos_dev = a->pos_dev;
+    l.pos = a->pos;
+    return l;
+}
+
+// Fills the kernel's description of a one-token product's input.
+int take_intake(int dtype, const dlm_intake *in, int K, RowIntake &r) {
+    if (bad_type(dtype) || K <= 0 || K % 64 || K > kMaxLength * (dtype == kF32 ? 1 : 2)) return DLM_ERR_SHAPE;
+    switch (in->mode) {
+        case kIntakePlain:
+            if (!in->x) return DLM_ERR_NULL;
+            break;
+        case kIntakeResidual:
+            if (!in->res || !in->y || !in->norm_w) return DLM_ERR_NULL;
+            break;
+        case kIntakeEmbed:
+            if (!in->embed || !in->token || !in->res_out) return DLM_ERR_NULL;
+            break;
+        case kIntakeFinal:
+            if (!in->res || !in->final_w || (in->y && !in->norm_w)) return DLM_ERR_NULL;
+            break;
+        case kIntakeNormed:
+            if (!in->final_w || (in->embed ? !in->token : !in->res)) return DLM_ERR_NULL;
+            break;
+        default: return DLM_ERR_SHAPE;
+    }
+    if (in->mode != kIntakePlain && (in->width <= 0 || in->width > K || !(in->eps >= 0.f))) return DLM_ERR_SHAPE;
+    for (const void *q : {in->x, (const void *)in->res, (const void *)in->y, (const void *)in->norm_w, (const void *)in->final_w, (const void *)in->res_out,
+                          (const void *)in->h_out, in->embed})
+        if (odd(q)) return DLM_ERR_ALIGN;
+    r.mode = in->mode;
+    r.x = in->x;
+    r.res = in->res;
+    r.y = in->y;
+    r.norm_w = in->norm_w;
+    r.final_w = in->final_w;
+    r.eps = in->eps;
+    r.width = in->width;
+    r.res_out = in->res_out;
+    r.h_out = in->h_out;
+    r.embed = in->embed;
+    r.token = in->token;
+    r.scale = in->scale;
+    return DLM_OK;
+}
+
 }  // namespace
 
 extern "C" {
@@ -69,42 +163,23 @@ int dlm_gemv_keys(int K, int N) { return K > 0 && N > 0 ? 4 * dense_gemv_blocks(
 
 int dlm_gemv(int dtype, const void *w, const dlm_intake *in, void *out, float *out_f32, uint64_t *keys, int n_valid, int K, int N, void *stream) {
     if (!w || !in || (!out) == (!out_f32)) return DLM_ERR_NULL;
-    if (bad_type(dtype) || K <= 0 || K % 64 || K > kMaxLength * (dtype == kF32 ? 1 : 2) || N <= 0 || n_valid < 0 || n_valid > N) return DLM_ERR_SHAPE;
-    if (odd(w) || odd(out) || odd(out_f32)) return DLM_ERR_ALIGN;
+    if (N <= 0 || n_valid < 0 || n_valid > N) return DLM_ERR_SHAPE;
     RowIntake r;
-    r.mode = in->mode;
-    switch (in->mode) {
-        case kIntakePlain:
-            if (!in->x) return DLM_ERR_NULL;
-            break;
-        case kIntakeResidual:
-            if (!in->res || !in->y || !in->norm_w) return DLM_ERR_NULL;
-            break;
-        case kIntakeEmbed:
-            if (!in->embed || !in->token || !in->res_out) return DLM_ERR_NULL;
-            break;
-        case kIntakeFinal:
-            if (!in->res || !in->final_w || (in->y && !in->norm_w)) return DLM_ERR_NULL;
-            break;
-        default: return DLM_ERR_SHAPE;
-    }
-    if (in->mode != kIntakePlain && (in->width <= 0 || in->width > K || !(in->eps >= 0.f))) return DLM_ERR_SHAPE;
-    for (const void *q : {in->x, (const void *)in->res, (const void *)in->y, (const void *)in->norm_w, (const void *)in->final_w, (const void *)in->res_out,
-                          (const void *)in->h_out, in->embed})
-        if (odd(q)) return DLM_ERR_ALIGN;
-    r.x = in->x;
-    r.res = in->res;
-    r.y = in->y;
-    r.norm_w = in->norm_w;
-    r.final_w = in->final_w;
-    r.eps = in->eps;
-    r.width = in->width;
-    r.res_out = in->res_out;
-    r.h_out = in->h_out;
-    r.embed = in->embed;
-    r.token = in->token;
-    r.scale = in->scale;
+    const int c = take_intake(dtype, in, K, r);
+    if (c) return c;
+    if (odd(w) || odd(out) || odd(out_f32)) return DLM_ERR_ALIGN;
     return done(launch_dense_gemv(dtype, w, r, out, out_f32, reinterpret_cast<unsigned long long *>(keys), n_valid, K, N, hs(stream)));
+}
+
+int dlm_gemv_act(int dtype, const void *w, const dlm_intake *in, const dlm_row_output *ro, void *out, int K, int N, void *stream) {
+    if (!w || !in || !ro || !out) return DLM_ERR_NULL;
+    if (N <= 0 || ro->gate < kGateNone || ro->gate > kGateGelu) return DLM_ERR_SHAPE;
+    if (ro->gate && (N % 32 || (in->mode != kIntakePlain && in->mode != kIntakeNormed) || ro->silu_begin < ro->silu_end)) return DLM_ERR_SHAPE;
+    RowIntake r;
+    const int c = take_intake(dtype, in, K, r);
+    if (c) return c;
+    if (odd(w) || odd(out)) return DLM_ERR_ALIGN;
+    return done(launch_dense_gemv(dtype, w, r, out, nullptr, nullptr, 0, K, N, hs(stream), RowOutput{ro->silu_begin, ro->silu_end, ro->gate}));
 }
 
 int dlm_argmax(const uint64_t *keys, int n_keys, int32_t *token, int32_t *position, int32_t *history, void *stream) {
@@ -159,12 +234,12 @@ int dlm_gemm(int dtype, const dlm_gemm_args *g, void *stream) {
     if (g->tile_rows != 32 && g->tile_rows != 128 && g->tile_rows != 256) return DLM_ERR_SHAPE;
     if (g->tiles) {
         if (!g->order) return DLM_ERR_NULL;
-        if (g->n_tiles <= 0 || g->gather < 0 || g->epilogue == kOutF32 || g->w_stride < (int64_t)g->N * g->K) return DLM_ERR_SHAPE;
-        if (g->epilogue == kOutSwiglu && g->N % 32) return DLM_ERR_SHAPE;
-    } else if (g->epilogue == kOutSwiglu) {
-        return DLM_ERR_SHAPE;
+        if (g->n_tiles <= 0 || g->gather < 0 || g->epilogue == kOutF32 || g->epilogue == kOutGeglu || g->silu_begin < g->silu_end || g->w_stride < (int64_t)g->N * g->K) return DLM_ERR_SHAPE;
     }
-    if (g->epilogue < 0 || g->epilogue > 2 || g->ldo < (g->epilogue == kOutSwiglu ? g->N / 2 : g->N)) return DLM_ERR_SHAPE;
+    const bool paired = g->epilogue == kOutSwiglu || g->epilogue == kOutGeglu;
+    if (paired && g->N % 32) return DLM_ERR_SHAPE;
+    if (g->silu_begin < g->silu_end && (g->epilogue != kOutElem || g->silu_begin % 16 || g->silu_end % 16)) return DLM_ERR_SHAPE;
+    if (g->epilogue < 0 || g->epilogue > kOutGeglu || g->ldo < (paired ? g->N / 2 : g->N)) return DLM_ERR_SHAPE;
     if (odd(g->a) || odd(g->w) || odd(g->out)) return DLM_ERR_ALIGN;
     GemmArgs a;
     a.a = g->a;
@@ -181,6 +256,8 @@ int dlm_gemm(int dtype, const dlm_gemm_args *g, void *stream) {
     a.n_tiles = g->n_tiles;
     a.gather = g->gather;
     a.w_stride = g->w_stride;
+    a.silu_begin = g->silu_begin;
+    a.silu_end = g->silu_end;
     return done(launch_dense_gemm(dtype, a, g->tile_rows, hs(stream)));
 }
 
@@ -207,6 +284,97 @@ int dlm_norm_rows(int dtype, const float *res, const int32_t *rows, const float 
     if (bad_type(dtype) || n <= 0 || width <= 0 || width % 64 || true_width <= 0 || true_width > width || !(eps >= 0.f)) return DLM_ERR_SHAPE;
     if (odd(res) || odd(norm_w) || odd(out)) return DLM_ERR_ALIGN;
     return done(launch_norm_rows(dtype, res, rows, norm_w, eps, true_width, out, n, width, hs(stream)));
+}
+
+int dlm_add_norm_rows(int dtype, float *res, const float *y, const int32_t *tokens, const void *embed, float scale, const float *norm_w, float eps,
+                      int true_width, void *h, int M, int width, void *stream) {
+    if (!res || (tokens && !embed) || (h && !norm_w)) return DLM_ERR_NULL;
+    if (bad_type(dtype) || M <= 0 || width <= 0 || width % 64 || width > kMaxWidth || true_width <= 0 || true_width > width || !(eps >= 0.f) || (tokens && y))
+        return DLM_ERR_SHAPE;
+    if (odd(res) || odd(y) || odd(embed) || odd(norm_w) || odd(h)) return DLM_ERR_ALIGN;
+    return done(launch_add_norm_rows(dtype, res, y, tokens, embed, scale, norm_w, eps, true_width, h, M, width, hs(stream)));
+}
+
+int dlm_head_decode_supported(int dtype, const dlm_head_shape *s) {
+    return s && !bad_type(dtype) && s->kv_heads > 0 && decode_block_keys(dtype, head_view(head_of(s))) != 0;
+}
+int dlm_head_prefill_supported(int dtype, const dlm_head_shape *s) { return s && !bad_type(dtype) && head_prefill_supported(dtype, head_of(s)); }
+
+int dlm_head_prepare(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, void *q, void *stream) {
+    const int c = check_head(dtype, s, r);
+    if (c) return c;
+    if (!q) return DLM_ERR_NULL;
+    if (odd(q)) return DLM_ERR_ALIGN;
+    return done(launch_head_prepare(dtype, head_of(s), head_rows_of(r), q, hs(stream)));
+}
+
+int dlm_head_prefill(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, const void *q, void *out, int64_t ldo, void *stream) {
+    const int c = check_head(dtype, s, r);
+    if (c) return c;
+    if (!q || !out) return DLM_ERR_NULL;
+    if (r->pos_dev || !head_prefill_supported(dtype, head_of(s)) || ldo % 8 || ldo < (int64_t)s->heads * s->vdim) return DLM_ERR_SHAPE;
+    if (odd(q) || odd(out)) return DLM_ERR_ALIGN;
+    return done(launch_head_prefill(dtype, head_of(s), head_rows_of(r), q, out, ldo, hs(stream)));
+}
+
+int dlm_head_decode(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, const void *q, int nsplit, float *part_o, float *part_ml, void *stream) {
+    const int c = check_head(dtype, s, r);
+    if (c) return c;
+    if (!q || !part_o || !part_ml) return DLM_ERR_NULL;
+    const CacheView v = head_view(head_of(s));
+    if (nsplit <= 0 || nsplit > 256 || !decode_block_keys(dtype, v)) return DLM_ERR_SHAPE;
+    if (odd(q) || odd(part_o)) return DLM_ERR_ALIGN;
+    return done(launch_cache_decode(dtype, v, q, r->cache, r->M, r->pos_dev, r->pos, nsplit, part_o, part_ml, hs(stream)));
+}
+
+int dlm_head_merge(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, int nsplit, const float *part_o, const float *part_ml, void *out, int64_t ldo,
+                   void *stream) {
+    const int c = check_head(dtype, s, r);
+    if (c) return c;
+    if (!part_o || !part_ml || !out) return DLM_ERR_NULL;
+    if (nsplit <= 0 || nsplit > 256 || !decode_block_keys(dtype, head_view(head_of(s))) || ldo % 8 || ldo < (int64_t)s->heads * s->vdim) return DLM_ERR_SHAPE;
+    if (odd(part_o) || odd(out)) return DLM_ERR_ALIGN;
+    return done(launch_head_merge(dtype, head_of(s), head_rows_of(r), nsplit, part_o, part_ml, out, ldo, hs(stream)));
+}
+
+int dlm_short_conv(int dtype, const dlm_short_conv_args *c, void *act, void *stream) {
+    if (!c || !c->proj || !c->w || !c->history || !c->factors || !act) return DLM_ERR_NULL;
+    if (bad_type(dtype) || c->k_heads <= 0 || c->heads <= 0 || c->dim <= 0 || c->dim % 4 || c->vdim <= 0 || c->vdim % 4 || c->taps <= 0 || c->M <= 0 ||
+        c->M > 65535 * 4 || c->pos < 0 || c->ld % 8 || c->off < 0 || c->off % 8 || c->taps > 65535 || (c->pos_dev && c->M > 1) || !(c->unit_eps >= 0.f))
+        return DLM_ERR_SHAPE;
+    if (odd(c->proj) || odd(c->w) || odd(c->history) || odd(act)) return DLM_ERR_ALIGN;
+    const ConvArgs a = {c->k_heads, c->heads, c->dim, c->vdim, c->taps, (long)c->ld, c->off, c->w, c->factors, c->q_scale, c->unit_eps, c->M, c->pos_dev, c->pos};
+    return done(launch_short_conv(dtype, a, c->proj, c->history, act, hs(stream)));
+}
+
+int dlm_recurrence_steps(int dtype, const dlm_recurrence_args *a, float *o, void *stream) {
+    const int c = check_recurrence(dtype, a);
+    if (c) return c;
+    if (!o) return DLM_ERR_NULL;
+    return done(launch_recurrence_steps(dtype, linear_of(a), o, hs(stream)));
+}
+
+size_t dlm_recurrence_chunk_bytes(const dlm_recurrence_args *a) {
+    return a && a->heads > 0 && a->dim > 0 && a->vdim > 0 && a->M > 0 && linear_chunks_supported(linear_of(a)) ? linear_chunk_bytes(linear_of(a)) : 0;
+}
+
+int dlm_recurrence_chunks(int dtype, const dlm_recurrence_args *a, void *work, float *o, void *stream) {
+    const int c = check_recurrence(dtype, a);
+    if (c) return c;
+    if (!work || !o) return DLM_ERR_NULL;
+    if (!linear_chunks_supported(linear_of(a))) return DLM_ERR_SHAPE;
+    if (odd(work) || odd(o)) return DLM_ERR_ALIGN;
+    return done(launch_linear_chunks(dtype, linear_of(a), work, o, hs(stream)));
+}
+
+int dlm_gated_norm(int dtype, const float *o, const float *w, const void *gate, int64_t ld_gate, void *out, int64_t ld_out, int M, int groups, int cols,
+                   int true_cols, float eps, void *stream) {
+    if (!o || !w || !gate || !out) return DLM_ERR_NULL;
+    if (bad_type(dtype) || M <= 0 || M > 65535 || groups <= 0 || cols <= 0 || cols % 4 || true_cols <= 0 || true_cols > cols || !(eps >= 0.f) || ld_gate % 4 || ld_out % 4 ||
+        ld_out < (int64_t)groups * cols)
+        return DLM_ERR_SHAPE;
+    if (odd(o) || odd(w)) return DLM_ERR_ALIGN;
+    return done(launch_gated_norm(dtype, GatedNorm{o, groups, cols, true_cols, w, eps, (long)ld_gate, (long)ld_out}, gate, out, M, hs(stream)));
 }
 
 int dlm_latent_decode_supported(int dtype, const dlm_latent_shape *s) { return s && !bad_type(dtype) && latent_decode_supported(dtype, shape_of(s)); }

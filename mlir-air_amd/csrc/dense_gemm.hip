@@ -32,6 +32,7 @@ struct GemmKernelArgs {
     int gather;
     long w_stride;
     int tiles_m, tiles_n;
+    int silu_begin, silu_end;
 };
 
 // BM x BN tile, WM x WN waves (m x n); GROUPED: expert row tiles
@@ -152,14 +153,14 @@ __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKern
         size_t row = m;
         if constexpr (GROUPED)
             if (p.gather == 0) row = p.order[m];
-        if constexpr (EPI == kOutSwiglu) {
+        if constexpr (EPI == kOutSwiglu || EPI == kOutGeglu) {
 #pragma unroll
             for (int j = 0; j < NT; j += 2) {
                 const int n = n0 + wn * (BN / WN) + 16 * j;
                 if (n >= p.N) continue;
                 float v[4];
 #pragma unroll
-                for (int r = 0; r < 4; ++r) v[r] = silu_f32(acc[j][i][r]) * acc[j + 1][i][r];
+                for (int r = 0; r < 4; ++r) v[r] = (EPI == kOutGeglu ? gelu_tanh_f32(acc[j][i][r]) : silu_f32(acc[j][i][r])) * acc[j + 1][i][r];
                 store4(static_cast<T *>(p.out) + row * p.ldo + n / 2 + 4 * g, v[0], v[1], v[2], v[3]);
             }
         } else {
@@ -167,6 +168,12 @@ __global__ void __launch_bounds__(64 * WM * WN) dense_gemm_kernel(const GemmKern
             for (int j = 0; j < NT; ++j) {
                 const int n = n0 + wn * (BN / WN) + 16 * j + 4 * g;
                 if (n >= p.N) continue;
+                if constexpr (EPI == kOutElem && !GROUPED) {
+                    if (n >= p.silu_begin && n < p.silu_end) {
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) acc[j][i][r] = silu_f32(acc[j][i][r]);
+                    }
+                }
                 if constexpr (EPI == kOutF32)
                     store4(static_cast<float *>(p.out) + row * p.ldo + n, acc[j][i][0], acc[j][i][1], acc[j][i][2], acc[j][i][3]);
                 else
@@ -191,6 +198,8 @@ hipError_t launch_tile(const GemmArgs &g, hipStream_t stream) {
     p.order = g.order;
     p.gather = g.gather;
     p.w_stride = g.w_stride;
+    p.silu_begin = g.silu_begin;
+    p.silu_end = g.silu_end;
     p.tiles_m = g.tiles ? g.n_tiles : (g.M + BM - 1) / BM;
     p.tiles_n = (g.N + BN - 1) / BN;
     const int total = p.tiles_m * p.tiles_n, grid = (total + 7) / 8 * 8;
@@ -206,8 +215,12 @@ hipError_t launch_tile(const GemmArgs &g, hipStream_t stream) {
     if (g.tiles)
         return g.epilogue == kOutSwiglu ? run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutSwiglu, true>)
                                         : run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutElem, true>);
-    return g.epilogue == kOutF32 ? run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutF32, false>)
-                                 : run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutElem, false>);
+    switch (g.epilogue) {
+        case kOutF32: return run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutF32, false>);
+        case kOutSwiglu: return run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutSwiglu, false>);
+        case kOutGeglu: return run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutGeglu, false>);
+        default: return run(&dense_gemm_kernel<T, BM, BN, WM, WN, STAGES, kOutElem, false>);
+    }
 }
 
 }  // namespace

@@ -7,7 +7,8 @@
 //
 // The intake computes x where another kernel would otherwise be launched for it: the embedding row, or the residual
 // stream with the normed output of the previous sublayer added (every workgroup redoes this small sum from L2; one of
-// them stores it), or the final norm of that.  The first weights are requested before it.
+// them stores it), or the final norm of that, or the norm of the stream with the previous sublayer's output added.  The first
+// weights are requested before it.  The row sums can be combined in pairs: activation of a gate row times an up row.
 #include "dense.h"
 #include "dense_kernels.h"
 
@@ -35,6 +36,7 @@ struct GemvParams {
     const T *embed;
     const int32_t *token;
     float scale;
+    RowOutput ro;
 };
 
 // sum over the workgroup, for every thread
@@ -69,6 +71,38 @@ __device__ __forceinline__ void take_in(const GemvParams<T> &p, T *xs, float *re
                 store4(p.res_out + i, e[0], e[1], e[2], e[3]);
                 if (p.h_out) store4(p.h_out + i, e[0], e[1], e[2], e[3]);
             }
+        }
+    } else if constexpr (MODE == kIntakeNormed) {
+        const T *row = p.embed ? p.embed + (size_t)p.token[0] * p.K : nullptr;
+        auto value = [&](int i, float (&v)[4]) {
+            if (row) {
+                load4(row + i, v);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) v[j] *= p.scale;
+                return;
+            }
+            load4(p.res + i, v);
+            if (p.y) {
+                float u[4];
+                load4(p.y + i, u);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) v[j] += u[j];
+            }
+        };
+        float ss = 0.f;
+        for (int i = 4 * tid; i < p.K; i += 4 * kGemvThreads) {
+            float v[4];
+            value(i, v);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) ss = fmaf(v[j], v[j], ss);
+            if (blockIdx.x == 0 && p.res_out) store4(p.res_out + i, v[0], v[1], v[2], v[3]);
+        }
+        const float rstd = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
+        for (int i = 4 * tid; i < p.K; i += 4 * kGemvThreads) {
+            float v[4], w[4];
+            value(i, v);
+            load4(p.final_w + i, w);
+            store4(xs + i, v[0] * rstd * w[0], v[1] * rstd * w[1], v[2] * rstd * w[2], v[3] * rstd * w[3]);
         }
     } else {
         float rstd = 0.f;
@@ -121,12 +155,14 @@ __device__ __forceinline__ void take_in(const GemvParams<T> &p, T *xs, float *re
     }
 }
 
-template <class T, int R, int U>
+// (PAIR: rows 2 o and 2 o + 1 of the walk are the gate and the up row of output o)
+template <class T, int R, int U, bool PAIR>
 __device__ __forceinline__ void request(Vec8<T> (&w)[R][U], const T *base, int K, int N, int row0, int c0) {
     const int lane = threadIdx.x & 63;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-        const int row = row0 + r < N ? row0 + r : N - 1;   // past the end: read in range, never stored
+        int row = row0 + r < N ? row0 + r : N - 1;   // past the end: read in range, never stored
+        if constexpr (PAIR) row = (row >> 5) * 32 + ((row & 31) >> 1) + 16 * (row & 1);
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             const int k = (c0 + u) * kPiece + 8 * lane;
@@ -135,7 +171,7 @@ __device__ __forceinline__ void request(Vec8<T> (&w)[R][U], const T *base, int K
     }
 }
 
-template <class T, int R, int U, int MODE>
+template <class T, int R, int U, int MODE, bool PAIR>
 __global__ void __launch_bounds__(kGemvThreads) dense_gemv_kernel(const GemvParams<T> p) {
     extern __shared__ __attribute__((aligned(16))) char gemv_lds[];
     __shared__ float red[kGemvWaves];
@@ -145,7 +181,7 @@ __global__ void __launch_bounds__(kGemvThreads) dense_gemv_kernel(const GemvPara
     const int pieces = (p.K + kPiece - 1) / kPiece;
     int g = blockIdx.x * kGemvWaves + wave;
     Vec8<T> w[R][U];
-    if (g < p.groups) request<T, R, U>(w, p.w, p.K, p.N, g * R, 0);
+    if (g < p.groups) request<T, R, U, PAIR>(w, p.w, p.K, p.N, g * R, 0);
     take_in<T, MODE>(p, xs, red);
     __syncthreads();
     unsigned long long best = 0;
@@ -161,10 +197,20 @@ __global__ void __launch_bounds__(kGemvThreads) dense_gemv_kernel(const GemvPara
 #pragma unroll
                 for (int r = 0; r < R; ++r) acc[r] = dot8(w[r][u], xv, acc[r]);
             }
-            if (c0 + U < pieces) request<T, R, U>(w, p.w, p.K, p.N, g * R, c0 + U);
+            if (c0 + U < pieces) request<T, R, U, PAIR>(w, p.w, p.K, p.N, g * R, c0 + U);
         }
-        if (g + stride < p.groups) request<T, R, U>(w, p.w, p.K, p.N, (g + stride) * R, 0);
+        if (g + stride < p.groups) request<T, R, U, PAIR>(w, p.w, p.K, p.N, (g + stride) * R, 0);
         float mine = 0.f;
+        if constexpr (PAIR) {
+#pragma unroll
+            for (int r = 0; r < R; r += 2) {
+                const float a = wave_reduce<false>(acc[r]), b = wave_reduce<false>(acc[r + 1]);
+                mine = lane == r / 2 ? (p.ro.gate == kGateGelu ? gelu_tanh_f32(a) : silu_f32(a)) * b : mine;
+            }
+            const int o = g * (R / 2) + lane;
+            if (lane < R / 2 && 2 * o < p.N) p.out[o] = from_float<T>(mine);
+            continue;
+        }
 #pragma unroll
         for (int r = 0; r < R; ++r) {
             const float s = wave_reduce<false>(acc[r]);
@@ -172,6 +218,7 @@ __global__ void __launch_bounds__(kGemvThreads) dense_gemv_kernel(const GemvPara
         }
         const int row = g * R + lane;
         if (lane < R && row < p.N) {
+            if (row >= p.ro.silu_begin && row < p.ro.silu_end) mine = silu_f32(mine);
             if (p.out_f32) p.out_f32[row] = mine;
             else p.out[row] = from_float<T>(mine);
             if (p.keys && row < p.n_valid) {
@@ -217,11 +264,17 @@ hipError_t launch_mode(const GemvParams<T> &p, int mode, int grid, size_t lds, h
         hipLaunchKernelGGL(kernel, dim3(grid), dim3(kGemvThreads), lds, stream, p);
         return hipGetLastError();
     };
+    if (p.ro.gate) {
+        if constexpr (R >= 2)
+            return mode == kIntakeNormed ? run(&dense_gemv_kernel<T, R, U, kIntakeNormed, true>) : run(&dense_gemv_kernel<T, R, U, kIntakePlain, true>);
+        return hipErrorInvalidValue;
+    }
     switch (mode) {
-        case kIntakePlain: return run(&dense_gemv_kernel<T, R, U, kIntakePlain>);
-        case kIntakeResidual: return run(&dense_gemv_kernel<T, R, U, kIntakeResidual>);
-        case kIntakeEmbed: return run(&dense_gemv_kernel<T, R, U, kIntakeEmbed>);
-        default: return run(&dense_gemv_kernel<T, R, U, kIntakeFinal>);
+        case kIntakePlain: return run(&dense_gemv_kernel<T, R, U, kIntakePlain, false>);
+        case kIntakeResidual: return run(&dense_gemv_kernel<T, R, U, kIntakeResidual, false>);
+        case kIntakeEmbed: return run(&dense_gemv_kernel<T, R, U, kIntakeEmbed, false>);
+        case kIntakeNormed: return run(&dense_gemv_kernel<T, R, U, kIntakeNormed, false>);
+        default: return run(&dense_gemv_kernel<T, R, U, kIntakeFinal, false>);
     }
 }
 
@@ -229,8 +282,9 @@ int rows_per_wave(int K, int N) { return K > 2048 || N < 512 ? 1 : K > 1024 ? 2 
 
 template <class T>
 hipError_t launch_typed(const void *w, const RowIntake &in, void *out, float *out_f32, unsigned long long *keys, int n_valid, int K, int N,
-                        hipStream_t stream) {
+                        const RowOutput &ro, hipStream_t stream) {
     GemvParams<T> p;
+    p.ro = ro;
     p.w = static_cast<const T *>(w);
     p.out = static_cast<T *>(out);
     p.out_f32 = out_f32;
@@ -250,9 +304,9 @@ hipError_t launch_typed(const void *w, const RowIntake &in, void *out, float *ou
     p.embed = static_cast<const T *>(in.embed);
     p.token = in.token;
     p.scale = in.scale;
-    const int R = rows_per_wave(K, N);
+    const int R = ro.gate && K > 1024 ? 2 : ro.gate ? 4 : rows_per_wave(K, N);
     p.groups = (N + R - 1) / R;
-    const int grid = dense_gemv_blocks(K, N);
+    const int need = (p.groups + kGemvWaves - 1) / kGemvWaves, grid = need < kMaxBlocks ? need : kMaxBlocks;
     const size_t lds = (size_t)((K + kPiece - 1) / kPiece) * kPiece * sizeof(T);
     switch (R) {
         case 1: return launch_mode<T, 1, 8>(p, in.mode, grid, lds, stream);
@@ -270,9 +324,9 @@ int dense_gemv_blocks(int K, int N) {
 }
 
 hipError_t launch_dense_gemv(int dtype, const void *w, const RowIntake &in, void *out, float *out_f32, unsigned long long *keys, int n_valid,
-                             int K, int N, hipStream_t stream) {
-    return dtype == kF32 ? launch_typed<float>(w, in, out, out_f32, keys, n_valid, K, N, stream)
-                         : launch_typed<bf16>(w, in, out, out_f32, keys, n_valid, K, N, stream);
+                             int K, int N, hipStream_t stream, const RowOutput &ro) {
+    return dtype == kF32 ? launch_typed<float>(w, in, out, out_f32, keys, n_valid, K, N, ro, stream)
+                         : launch_typed<bf16>(w, in, out, out_f32, keys, n_valid, K, N, ro, stream);
 }
 
 hipError_t launch_argmax_keys(const unsigned long long *keys, int n, int32_t *token, int32_t *position, int32_t *history, hipStream_t stream) {

@@ -17,6 +17,7 @@ enum : int {
     kIntakeResidual = 1,   // res + y / rms(y) * norm_w, also left in res_out (and h_out)
     kIntakeEmbed = 2,      // embed[*token] * scale, also left in res_out (and h_out)
     kIntakeFinal = 3,      // the norm final_w of (res + y / rms(y) * norm_w), or of res without y
+    kIntakeNormed = 4,     // the norm final_w of v = embed[*token] * scale, res + y or res; v also left in res_out
 };
 struct RowIntake {
     int mode = kIntakePlain;
@@ -30,10 +31,16 @@ struct RowIntake {
     const int32_t *token = nullptr;
     float scale = 1.f;
 };
+// What becomes of the row sums: stored as they are, with silu on rows silu_begin .. silu_end - 1, or (gate != 0) combined in pairs:
+// W holds 16 gate rows, 16 up rows, ... and out[N / 2] = gate's activation times up.
+enum : int { kGateNone = 0, kGateSilu = 1, kGateGelu = 2 };
+struct RowOutput {
+    int silu_begin = 0, silu_end = 0, gate = kGateNone;
+};
 // y[N] = W[N, K] x[K]; out in the element type, or fp32 in out_f32.  keys (4 per workgroup): argmax keys of the
 // first n_valid rows.
 hipError_t launch_dense_gemv(int dtype, const void *w, const RowIntake &in, void *out, float *out_f32, unsigned long long *keys,
-                             int n_valid, int K, int N, hipStream_t stream);
+                             int n_valid, int K, int N, hipStream_t stream, const RowOutput &ro = RowOutput());
 int dense_gemv_blocks(int K, int N);   // workgroups of that launch; it writes four keys per workgroup
 // token[0] = argmax from the keys; position[0] += 1; history[position] = token (each optional)
 hipError_t launch_argmax_keys(const unsigned long long *keys, int n, int32_t *token, int32_t *position, int32_t *history,
@@ -60,7 +67,8 @@ int moe_max_tiles(int entries, int experts, int bm);
 hipError_t launch_moe_plan(const int32_t *ids, int entries, int experts, int bm, int32_t *order, int32_t *tiles, hipStream_t stream);
 
 // Products over many rows: out[M, N] = A[M, K] W[N, K]^T.
-enum : int { kOutElem = 0, kOutF32 = 1, kOutSwiglu = 2 };   // swiglu: W holds 16 gate rows, 16 up rows, ...; out is [M, N / 2]
+// swiglu, geglu: W holds 16 gate rows, 16 up rows, ...; out is [M, N / 2], silu or the tanh form of gelu of the gate times up
+enum : int { kOutElem = 0, kOutF32 = 1, kOutSwiglu = 2, kOutGeglu = 3 };
 struct GemmArgs {
     const void *a = nullptr, *w = nullptr;
     void *out = nullptr;
@@ -72,10 +80,14 @@ struct GemmArgs {
     int n_tiles = 0;       // the most tiles (moe_max_tiles)
     int gather = 0;        // > 0: A row of an entry = entry / gather, out row = sorted place; 0: A row = sorted place, out row = entry
     long w_stride = 0;     // elements from one expert's W to the next
+    int silu_begin = 0, silu_end = 0;   // columns that silu is applied to (kOutElem, multiples of 16)
 };
 int dense_gemm_tile_rows(int dtype, int rows, int N, int matrices);   // rows of a tile (what launch_moe_plan gets as bm)
 hipError_t launch_dense_gemm(int dtype, const GemmArgs &g, int tile_rows, hipStream_t stream);
 
+// v = embed[tokens] * scale, or res + y, or res; res = v; h (optional) = the norm norm_w of v in the element type
+hipError_t launch_add_norm_rows(int dtype, float *res, const float *y, const int32_t *tokens, const void *embed, float scale, const float *norm_w,
+                                float eps, int true_width, void *h, int M, int width, hipStream_t stream);
 hipError_t launch_embed_rows(int dtype, const int32_t *tokens, const void *embed, float scale, float *res, void *h, int M, int width,
                              hipStream_t stream);
 // res += y / rms(y) * norm_w per row; h = res in the element type.  With weights (experts): y is [M * top, width] in the
@@ -85,6 +97,104 @@ hipError_t launch_residual_norm_rows(int dtype, float *res, const void *y, const
 // out[i] = norm of res[rows[i]] (rows nullptr: i)
 hipError_t launch_norm_rows(int dtype, const float *res, const int32_t *rows, const float *norm_w, float eps, int true_width, void *out, int n,
                             int width, hipStream_t stream);
+
+// Attention of a few rows over a cache, split along the keys: what a cache row is.  Rows of queries are [token][head] within a
+// key / value head, [key / value head] outermost; so are the partial results.
+struct CacheView {
+    int heads = 0, kv_heads = 1;        // query heads of one key / value head, key / value heads
+    int q_len = 0, row_len = 0;         // elements that are scored, elements of a cache row
+    int v_off = 0, v_cols = 0;          // the part of a row that is summed
+    int window = 1 << 30;               // a position sees itself and the window - 1 positions before it
+    int ring = 0;                       // rows of the cache that positions go round in (whole blocks of keys), 0: it is as long as the sequence
+    long head_stride = 0;               // elements between the matrices of two key / value heads
+    float scale = 1.f;
+};
+// Keys of one split of `n` keys, in whole blocks, and the block that the first visible key lies in: the same for the splits and
+// for what merges them.
+__host__ __device__ __forceinline__ int keys_per_split(int n, int nsplit, int kb) {
+    const int blocks = (n + kb - 1) / kb;
+    return (blocks + nsplit - 1) / nsplit * kb;
+}
+__host__ __device__ __forceinline__ int first_block_key(int pos0, int window, int kb) { return pos0 < window ? 0 : (pos0 - window + 1) / kb * kb; }
+int decode_block_keys(int dtype, const CacheView &v);   // keys of a block, 0: no kernel for these sizes
+hipError_t launch_cache_decode(int dtype, const CacheView &v, const void *q, const void *cache, int M, const int32_t *pos_dev, int pos, int nsplit,
+                               float *part_o, float *part_ml, hipStream_t stream);
+
+// Attention of H query heads over G key / value heads of their own projections (head h: key / value head h / (H / G)), with a norm
+// on queries and keys and a window.  A cache row of a key / value head is [key | value]; the heads' matrices follow each other.
+struct HeadShape {
+    int heads, kv_heads, dim, vdim;     // padded sizes (multiples of 32)
+    int true_dim;                       // elements in the mean of the norms
+    int window, ring;                   // ring: rows of a head's matrix
+    float scale, out_scale;             // of the scores, of the result
+};
+struct HeadRows {
+    const void *proj = nullptr;         // [M, ld]: q of all heads, k and v of all key / value heads from column `off`
+    long ld = 0;
+    int off = 0;
+    const float *q_norm = nullptr, *k_norm = nullptr;
+    float eps = 0.f;
+    void *cache = nullptr;
+    int M = 0;
+    const int32_t *pos_dev = nullptr;
+    int pos = 0;
+};
+// normed queries q [kv_heads][M][heads / kv_heads][dim], rows appended to the cache
+hipError_t launch_head_prepare(int dtype, const HeadShape &s, const HeadRows &r, void *q, hipStream_t stream);
+CacheView head_view(const HeadShape &s);
+hipError_t launch_head_merge(int dtype, const HeadShape &s, const HeadRows &r, int nsplit, const float *part_o, const float *part_ml, void *out, long ldo,
+                             hipStream_t stream);
+hipError_t launch_head_prefill(int dtype, const HeadShape &s, const HeadRows &r, const void *q, void *out, long ldo, hipStream_t stream);
+bool head_prefill_supported(int dtype, const HeadShape &s);
+
+// Linear recurrences.  dim is padded to a multiple of 64, vdim of 32.
+struct ConvArgs {
+    int k_heads, heads, dim, vdim;      // channels: q of k_heads, k of k_heads, v of heads
+    int taps;
+    long ld;
+    int off;                            // column of q in the projections
+    const float *w;                     // [taps][channels]
+    float *factors;                     // [M][q of k_heads | k of k_heads]: q_scale / |q|, 1 / |k|
+    float q_scale, unit_eps;
+    int M;
+    const int32_t *pos_dev;             // (NULL with more than one token)
+    int pos;
+};
+// act [M, channels]; history [taps, channels]
+hipError_t launch_short_conv(int dtype, const ConvArgs &c, const void *proj, void *history, void *act, hipStream_t stream);
+
+struct LinearArgs {
+    int k_heads, heads, dim, vdim;
+    const void *qkv;                    // [M, ld]: q at q_off, k at k_off (k_heads x dim), v at v_off (heads x vdim)
+    long ld;
+    int q_off, k_off, v_off;
+    const float *log2_decay;            // [heads]: one decay per head, or ...
+    const float *z;                     // ... [M, heads x dim]: exp(-exp(a_log) softplus(z + dt_bias)) per channel, and the delta rule
+    const float *a_log, *dt_bias;
+    const float *factors;               // (delta rule) of ConvArgs
+    const void *beta;                   // (delta rule) [M, ld_beta]: sigmoid of it
+    long ld_beta;
+    float *state;                       // [heads][vdim][dim]
+    int M;
+    const int32_t *pos_dev;
+    int pos;
+};
+constexpr int kMaxStateDim = 512;
+// o [M, heads x vdim]
+hipError_t launch_recurrence_steps(int dtype, const LinearArgs &a, float *o, hipStream_t stream);
+// long portions by chunks; work: linear_chunk_bytes of device memory
+bool linear_chunks_supported(const LinearArgs &a);
+size_t linear_chunk_bytes(const LinearArgs &a);
+hipError_t launch_linear_chunks(int dtype, const LinearArgs &a, void *work, float *o, hipStream_t stream);
+
+struct GatedNorm {
+    const float *o;                     // [M, groups x cols]
+    int groups, cols, true_cols;        // a norm runs over the cols of one group
+    const float *w;                     // [cols]
+    float eps;
+    long ld_gate, ld_out;
+};
+hipError_t launch_gated_norm(int dtype, const GatedNorm &g, const void *gate, void *out, int M, hipStream_t stream);
 
 // Latent attention.  Sizes are the padded ones; a cache row is [latent kv_rank | rotated key part rot].
 struct LatentShape {

@@ -6,7 +6,10 @@
 //   latent_absorb    appends the cache rows and moves the key projection to the query side: qa = W_uk^T q_unrotated per head,
 //                    followed by the rotated part, so that a score is one product of length rank + rot with a cache row
 //   latent_decode    attention of all rows and heads over the cached rows: HBM-bound on the cache, which is read once per
-//                    16 (row, head) pairs; both products on MFMA, keys split over workgroups
+//                    16 (row, head) pairs; both products on MFMA, keys split over workgroups.  The kernel is the one of every
+//                    cache whose rows hold a part that is scored and a part that is summed: for latents they overlap, for
+//                    grouped keys and values (head_attention.hip) they lie side by side, in one matrix per key / value head,
+//                    and the keys may be limited to a window and kept in a ring of rows
 //   latent_combine   merges the splits with the sink, applies the value projection of the head to the merged latent and the
 //                    output gate
 //
@@ -135,12 +138,6 @@ __global__ void __launch_bounds__(kLatThreads) latent_absorb_kernel(const Latent
     }
 }
 
-// Keys of one split of the cached rows, in whole blocks: the same split is found by latent_decode and latent_combine.
-__host__ __device__ __forceinline__ int keys_per_split(int total, int nsplit, int kb) {
-    const int blocks = (total + kb - 1) / kb;
-    return (blocks + nsplit - 1) / nsplit * kb;
-}
-
 // Rows of `chunks` times 8 elements that follow each other in memory -> LDS rows of another pitch, by the whole workgroup, in
 // batches of BATCH chunks per thread: every thread requests a batch before it stores the first of it.
 template <class T, int BATCH>
@@ -172,54 +169,65 @@ struct RowCopy {
 };
 
 // blockIdx.x = split, blockIdx.y = 16 rows (row = token * heads + head).  CT: 16-column tiles of the latent per wave.
-template <class T, int KB, int CT>
-__global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const LatentArgs<T> p, const T *qa, int nsplit, float *part_o, float *part_ml) {
+// blockIdx.z = key / value head.  BATCH: chunks per thread that a copy of keys has in flight.
+template <class T, int KB, int CT, int BATCH>
+__global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const CacheView v, const T *qa, const T *cache, int M, const int32_t *pos_dev, int pos, int nsplit,
+                                                                    float *part_o, float *part_ml) {
     extern __shared__ __attribute__((aligned(16))) char latent_lds[];
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int ql = lane & 15, g = lane >> 4;
-    const int lq = p.s.rank + p.s.rot, pitch = lq + 16 / (int)sizeof(T), rows = p.M * p.s.heads, row0 = blockIdx.y * 16;
+    const int lq = v.q_len, row_len = v.row_len, qpitch = lq + 16 / (int)sizeof(T), pitch = row_len + 16 / (int)sizeof(T);
+    const int rows = M * v.heads, row0 = blockIdx.y * 16;
+    qa += (size_t)blockIdx.z * rows * lq;
+    cache += (size_t)blockIdx.z * v.head_stride;
+    part_o += (size_t)blockIdx.z * rows * nsplit * v.v_cols;
+    part_ml += (size_t)blockIdx.z * rows * nsplit * 2;
     constexpr int SP = KB + 4, PP = KB + 8;       // pitches of the scores and of the probabilities
     T *tile = reinterpret_cast<T *>(latent_lds);  // [KB][pitch]
-    T *qt = tile + KB * pitch;                    // [16][pitch]
-    T *pt = qt + 16 * pitch;                      // [16][PP]
+    T *qt = tile + KB * pitch;                    // [16][qpitch]
+    T *pt = qt + 16 * qpitch;                     // [16][PP]
     float *st = reinterpret_cast<float *>(pt + 16 * PP);   // [parts][16][SP]
     float *al = st + 4 / (KB / 16) * 16 * SP;     // [16] rescaling factors of the block
 
-    const int pos0 = first_position(p), total = pos0 + p.M;
-    const int per = keys_per_split(total, nsplit, KB);
-    const int k0 = blockIdx.x * per;
+    const int pos0 = pos_dev ? pos_dev[0] : pos, total = pos0 + M;
+    const int first_key = first_block_key(pos0, v.window, KB);
+    const int per = keys_per_split(total - first_key, nsplit, KB);
+    const int k0 = first_key + blockIdx.x * per;
     const int last_row = row0 + 15 < rows ? row0 + 15 : rows - 1;
-    const int seen = pos0 + last_row / p.s.heads + 1;          // keys that any of these rows sees
+    const int seen = pos0 + last_row / v.heads + 1;            // keys that any of these rows sees
     const int k1 = k0 + per < seen ? k0 + per : seen;
 
-    const int chunks = lq / 8;
+    const int chunks = row_len / 8, qchunks = lq / 8;
     // A block of keys that is one batch travels to registers while the block before it is multiplied.
-    constexpr int BATCH = sizeof(T) == 2 ? 10 : 8;
     RowCopy<T, BATCH> copy;
     const int count = KB * chunks;
     const bool one_batch = count <= BATCH * kLatThreads;
-    auto request = [&](int kb, int first) { copy.request(p.cache + (size_t)kb * lq, first, (total - kb < KB ? total - kb : KB) * chunks); };
+    // (a ring holds whole blocks: its rows of one block follow each other)
+    auto request = [&](int kb, int first) {
+        copy.request(cache + (size_t)(v.ring ? kb % v.ring : kb) * row_len, first, (total - kb < KB ? total - kb : KB) * chunks);
+    };
     if (k0 < k1) {
         if (one_batch) request(k0, 0);
         constexpr int QB = sizeof(T) == 2 ? 5 : 3;
         RowCopy<T, QB> queries;
-        const int n = 16 * chunks, valid = (rows - row0 < 16 ? rows - row0 : 16) * chunks;
+        const int n = 16 * qchunks, valid = (rows - row0 < 16 ? rows - row0 : 16) * qchunks;
         for (int first = 0; first < n; first += QB * kLatThreads) {
             queries.request(qa + (size_t)row0 * lq, first, valid);
-            queries.store(qt, pitch, chunks, first, n);
+            queries.store(qt, qpitch, qchunks, first, n);
         }
     }
     // softmax threads: row tid / 16, keys (tid % 16) + 16 j of a block
     const int srow = tid >> 4, skey = tid & 15;
     const int row_of_mine = row0 + srow < rows ? row0 + srow : rows - 1;
-    const int my_limit = pos0 + row_of_mine / p.s.heads;       // last visible key
+    const int my_limit = pos0 + row_of_mine / v.heads;         // last visible key ...
+    const int my_first = my_limit - v.window;                  // ... and the last one in front of its window
     float m = kAttnNegBig, l = 0.f;
     floatx4 o[CT];
 #pragma unroll
     for (int c = 0; c < CT; ++c) o[c] = floatx4{0.f, 0.f, 0.f, 0.f};
-    const int tiles = p.s.rank / 16;
-    const float scale2 = p.s.scale * 1.4426950408889634f;
+    const int tiles = v.v_cols / 16;
+    const float scale2 = v.scale * 1.4426950408889634f;
 
     for (int kb = k0; kb < k1; kb += KB) {
         if (one_batch) {
@@ -236,7 +244,7 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
             constexpr int PARTS = 4 / (KB / 16);
             const int kt = wave % (KB / 16), part = wave / (KB / 16);
             floatx4 s0 = floatx4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
-            const T *a = tile + (16 * kt + ql) * pitch + 8 * g, *b = qt + ql * pitch + 8 * g;
+            const T *a = tile + (16 * kt + ql) * pitch + 8 * g, *b = qt + ql * qpitch + 8 * g;
             const int steps = lq / 32, ks1 = steps * (part + 1) / PARTS;
             int ks = steps * part / PARTS;
             for (; ks + 2 <= ks1; ks += 2) {
@@ -249,7 +257,7 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
         }
         __syncthreads();
         {
-            float v[KB / 16];
+            float sc[KB / 16];
             float top = kAttnNegBig;
 #pragma unroll
             for (int j = 0; j < KB / 16; ++j) {
@@ -257,15 +265,15 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
                 float raw = st[srow * SP + key];
 #pragma unroll
                 for (int q = 1; q < 4 / (KB / 16); ++q) raw += st[q * 16 * SP + srow * SP + key];
-                v[j] = kb + key <= my_limit ? raw * scale2 : kAttnNegBig;
-                top = fmaxf(top, v[j]);
+                sc[j] = kb + key <= my_limit && kb + key > my_first ? raw * scale2 : kAttnNegBig;
+                top = fmaxf(top, sc[j]);
             }
             top = row_reduce16<true>(top);
             const float mn = fmaxf(m, top), alpha = __builtin_amdgcn_exp2f(m - mn);
             float sum = 0.f;
 #pragma unroll
             for (int j = 0; j < KB / 16; ++j) {
-                const float e = v[j] > 0.5f * kAttnNegBig ? __builtin_amdgcn_exp2f(v[j] - mn) : 0.f;
+                const float e = sc[j] > 0.5f * kAttnNegBig ? __builtin_amdgcn_exp2f(sc[j] - mn) : 0.f;
                 sum += e;
                 pt[srow * PP + skey + 16 * j] = from_float<T>(e);
             }
@@ -289,14 +297,14 @@ __global__ void __launch_bounds__(kLatThreads) latent_decode_kernel(const Latent
             if (ct < tiles) {
                 o[c] *= alpha;
 #pragma unroll
-                for (int t = 0; t < KB / 32; ++t) o[c] = mma32(column8(tile + 32 * t * pitch, pitch, 16 * ct), pv[t], o[c]);
+                for (int t = 0; t < KB / 32; ++t) o[c] = mma32(column8(tile + 32 * t * pitch, pitch, v.v_off + 16 * ct), pv[t], o[c]);
             }
         }
         __syncthreads();
     }
     if (k0 >= total) return;       // (the merge does not look at splits that start behind the last key)
     if (row0 + ql < rows) {
-        float *dst = part_o + ((size_t)(row0 + ql) * nsplit + blockIdx.x) * p.s.rank + 4 * g;
+        float *dst = part_o + ((size_t)(row0 + ql) * nsplit + blockIdx.x) * v.v_cols + 4 * g;
 #pragma unroll
         for (int c = 0; c < CT; ++c) {
             const int ct = wave + 4 * c;
@@ -419,10 +427,20 @@ LatentArgs<T> args_of(const LatentShape &s, const LatentRows &r) {
     return a;
 }
 
+CacheView view_of(const LatentShape &s) {
+    CacheView v;
+    v.heads = s.heads;
+    v.q_len = v.row_len = s.rank + s.rot;
+    v.v_off = 0;
+    v.v_cols = s.rank;
+    v.scale = s.scale;
+    return v;
+}
+
 template <class T>
-size_t decode_lds(const LatentShape &s, int kb) {
-    const size_t pitch = s.rank + s.rot + 16 / sizeof(T);
-    return ((kb + 16) * pitch + 16 * (kb + 8)) * sizeof(T) + (64 / kb * 16 * (kb + 4) + 16) * sizeof(float);
+size_t decode_lds(const CacheView &v, int kb) {
+    const size_t pad = 16 / sizeof(T);
+    return (kb * (v.row_len + pad) + 16 * (v.q_len + pad) + 16 * (kb + 8)) * sizeof(T) + (64 / kb * 16 * (kb + 4) + 16) * sizeof(float);
 }
 constexpr size_t kLdsLimit = 160 * 1024;
 
@@ -431,33 +449,36 @@ constexpr int decode_block() { return 32; }
 
 // keys per block: fewer where a block of the usual size does not fit in LDS (0: not at all)
 template <class T>
-int decode_kb(const LatentShape &s) {
-    if (s.rank > 1024) return 0;
+int decode_kb(const CacheView &v) {
+    if (v.v_cols > 1024) return 0;
     int kb = decode_block<T>();
-    while (kb >= 32 && decode_lds<T>(s, kb) > kLdsLimit) kb /= 2;
+    while (kb >= 32 && decode_lds<T>(v, kb) > kLdsLimit) kb /= 2;
     return kb >= 32 ? kb : 0;
 }
 
 template <class T>
-hipError_t decode(const LatentShape &s, const LatentRows &r, const void *qa, int nsplit, float *part_o, float *part_ml, hipStream_t stream) {
-    const LatentArgs<T> a = args_of<T>(s, r);
-    const int kb = decode_kb<T>(s);
-    const size_t lds = decode_lds<T>(s, kb);
-    const dim3 grid(nsplit, (r.M * s.heads + 15) / 16);
+hipError_t decode(const CacheView &v, const void *qa, const void *cache, int M, const int32_t *pos_dev, int pos, int nsplit, float *part_o,
+                  float *part_ml, hipStream_t stream) {
+    const int kb = decode_kb<T>(v);
+    const size_t lds = decode_lds<T>(v, kb);
+    const dim3 grid(nsplit, (M * v.heads + 15) / 16, v.kv_heads);
     auto run = [&](auto kernel) {
         if (lds > 48 * 1024) {
             const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
             if (e != hipSuccess) return e;
         }
-        hipLaunchKernelGGL(kernel, grid, dim3(kLatThreads), lds, stream, a, static_cast<const T *>(qa), nsplit, part_o, part_ml);
+        hipLaunchKernelGGL(kernel, grid, dim3(kLatThreads), lds, stream, v, static_cast<const T *>(qa), static_cast<const T *>(cache), M, pos_dev, pos, nsplit,
+                           part_o, part_ml);
         return hipGetLastError();
     };
-    const int ct = (s.rank / 16 + 3) / 4;
+    const int ct = (v.v_cols / 16 + 3) / 4;
+    constexpr int B = sizeof(T) == 2 ? 10 : 8, S = sizeof(T) == 2 ? 4 : 8;   // short rows: a block is at most 4 (or 8) chunks per thread
     if (kb == 32) {
-        if (ct <= 2) return run(&latent_decode_kernel<T, 32, 2>);
-        if (ct <= 4) return run(&latent_decode_kernel<T, 32, 4>);
-        if (ct <= 8) return run(&latent_decode_kernel<T, 32, 8>);
-        return run(&latent_decode_kernel<T, 32, 16>);
+        if (ct <= 2 && kb * v.row_len <= 8 * S * kLatThreads) return run(&latent_decode_kernel<T, 32, 2, S>);
+        if (ct <= 2) return run(&latent_decode_kernel<T, 32, 2, B>);
+        if (ct <= 4) return run(&latent_decode_kernel<T, 32, 4, B>);
+        if (ct <= 8) return run(&latent_decode_kernel<T, 32, 8, B>);
+        return run(&latent_decode_kernel<T, 32, 16, B>);
     }
     return hipErrorInvalidValue;
 }
@@ -476,15 +497,23 @@ hipError_t combine(const LatentShape &s, const LatentRows &r, int nsplit, const 
                    void *out, long ldo, hipStream_t stream) {
     const int blocks = (s.vdim + kValueRows - 1) / kValueRows;
     hipLaunchKernelGGL(latent_combine_kernel<T>, dim3(s.heads * blocks, r.M), dim3(kMergeThreads), ((size_t)(s.rank + 511) / 512 * 512 + 3 * 512) * sizeof(float),
-                       stream, args_of<T>(s, r), nsplit, decode_kb<T>(s), part_o, part_ml, sink, static_cast<const T *>(w_uv), static_cast<T *>(out), ldo,
+                       stream, args_of<T>(s, r), nsplit, decode_kb<T>(view_of(s)), part_o, part_ml, sink, static_cast<const T *>(w_uv), static_cast<T *>(out), ldo,
                        blocks);
     return hipGetLastError();
 }
 
 }  // namespace
 
+int decode_block_keys(int dtype, const CacheView &v) { return dtype == kF32 ? decode_kb<float>(v) : decode_kb<bf16>(v); }
+
+hipError_t launch_cache_decode(int dtype, const CacheView &v, const void *q, const void *cache, int M, const int32_t *pos_dev, int pos, int nsplit,
+                               float *part_o, float *part_ml, hipStream_t stream) {
+    return dtype == kF32 ? decode<float>(v, q, cache, M, pos_dev, pos, nsplit, part_o, part_ml, stream)
+                         : decode<bf16>(v, q, cache, M, pos_dev, pos, nsplit, part_o, part_ml, stream);
+}
+
 bool latent_decode_supported(int dtype, const LatentShape &s) {
-    return s.dim <= 1024 && (dtype == kF32 ? decode_kb<float>(s) : decode_kb<bf16>(s)) != 0;
+    return s.dim <= 1024 && decode_block_keys(dtype, view_of(s)) != 0;
 }
 
 hipError_t launch_latent_prepare(int dtype, const LatentShape &s, const LatentRows &r, hipStream_t stream) {
@@ -499,7 +528,7 @@ hipError_t launch_latent_absorb(int dtype, const LatentShape &s, const LatentRow
 
 hipError_t launch_latent_decode(int dtype, const LatentShape &s, const LatentRows &r, const void *qa, int nsplit, float *part_o, float *part_ml,
                                 hipStream_t stream) {
-    return dtype == kF32 ? decode<float>(s, r, qa, nsplit, part_o, part_ml, stream) : decode<bf16>(s, r, qa, nsplit, part_o, part_ml, stream);
+    return launch_cache_decode(dtype, view_of(s), qa, r.cache, r.M, r.pos_dev, r.pos, nsplit, part_o, part_ml, stream);
 }
 
 hipError_t launch_latent_combine(int dtype, const LatentShape &s, const LatentRows &r, int nsplit, const float *part_o, const float *part_ml,

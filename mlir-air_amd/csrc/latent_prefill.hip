@@ -1,7 +1,9 @@
 // Causal attention of a long portion on expanded keys and values, for gfx950: queries [dim | rot] per head (rotated by
 // latent_prepare), keys = the head's dim columns of the expanded matrix followed by the rotated part of the cache row that
 // all heads share, values = the head's vdim columns, a learned sink per head in the denominator, and the output gate
-// applied before the only store.
+// applied before the only store.  WINDOW is the same kernel on grouped keys and values of their own projections
+// (head_attention.hip): rows [key | value] of one matrix per key / value head, positions going round in a ring of rows, a limit to
+// how far back a query sees, neither sink nor gate.
 //
 // Both products are computed transposed, so that a lane owns one query from the scores to the output:
 //   S^T[key, q] = K . Q^T      A = K rows from LDS, B = Q^T held in registers
@@ -37,7 +39,10 @@ struct PrefillArgs {
     int v_off, gate_off;     // columns of the values in kv, of the gate in q's matrix
     int M, total;            // queries, keys (the queries are the last M positions)
     float scale_log2;
-    const float *sink;
+    const float *sink;       // (NULL: none)
+    long head_q, group_q, head_k, head_v;   // elements between two heads' queries, key / value heads' queries, keys, values
+    int group, window, ring;                // query heads per key / value head
+    float out_scale;
 };
 
 template <class T>
@@ -50,7 +55,7 @@ __device__ __forceinline__ Vec8<float> ones8<float>() { return {floatx4{1.f, 1.f
 // NQ: K-steps of 32 of a score; NV: 16-column tiles of the output; EXACT: the sizes are exactly these, otherwise at most
 // these.  blockIdx.z picks a range of 16 NV value columns.
 // (EXACT addresses K and V rows with 32-bit offsets: the expanded matrix is smaller than 4 GiB.)
-template <class T, int NQ, int NV, int QB, int KB, int SETS, bool EXACT>
+template <class T, int NQ, int NV, int QB, int KB, int SETS, bool EXACT, bool WINDOW>
 __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kernel(const PrefillArgs<T> p) {
     constexpr int NKK = KB / 16, NT = KB / 32, QW = 64 * QB;
     extern __shared__ __attribute__((aligned(16))) char pf_lds[];
@@ -72,6 +77,10 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
     const int item_end = (item + 1) * QW < p.M ? (item + 1) * QW : p.M;
     const int blocks = (pos0 + item_end + KB - 1) / KB;
     const int wave_last = pos0 + q0 + 16 * QB - 1;                // last position of this wave's queries
+    const int kvh = WINDOW ? head / p.group : head;
+    // blocks that are wholly in front of the window of every query of the item are left out, and of those of a wave by the wave
+    const int item_first = WINDOW ? pos0 + item * QW - p.window + 1 : 0, first = item_first > 0 ? item_first / KB : 0;
+    const int wave_first = WINDOW ? pos0 + q0 - p.window + 1 : 0;
 
     Vec8<T> qf[QB][NQ];
     floatx4 o[QB][NV], l[QB];
@@ -81,7 +90,7 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
     for (int b = 0; b < QB; ++b) {
         const int qi = q0 + 16 * b + ql;
         qpos[b] = pos0 + qi;
-        const T *row = p.q + (size_t)(qi < p.M ? qi : p.M - 1) * p.ldq + (size_t)head * qd + 8 * g;
+        const T *row = p.q + (size_t)(qi < p.M ? qi : p.M - 1) * p.ldq + (WINDOW ? kvh * p.group_q + (head - kvh * p.group) * p.head_q : (size_t)head * qd) + 8 * g;
 #pragma unroll
         for (int ks = 0; ks < NQ; ++ks)
             if (EXACT || ks < nq) qf[b][ks] = load8(row + 32 * ks);
@@ -92,19 +101,21 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
     }
 
     // a chunk is 8 elements of a row; the first dim of a K row come from the expanded matrix, the rest from the cache
-    const T *k_base = p.kv + (size_t)head * p.dim, *v_base = p.kv + p.v_off + (size_t)head * p.vdim + vcol0, *r_base = p.cache + p.rot_off;
+    const T *k_base = p.kv + kvh * p.head_k, *v_base = p.kv + p.v_off + kvh * p.head_v + vcol0, *r_base = p.cache + p.rot_off;
+    auto row_of = [&](int kb, int i) {   // row of key kb + i of a block (a ring holds whole blocks)
+        const int key = kb + i < p.total ? i : p.total - 1 - kb;
+        return (WINDOW ? kb % p.ring : kb) + key;
+    };
     auto at = [&](const T *base, int row, long ld, int e) -> Vec8<T> {
         if constexpr (EXACT) return load8(reinterpret_cast<const T *>(reinterpret_cast<const char *>(base) + (uint32_t)(row * (uint32_t)ld + e) * (uint32_t)sizeof(T)));
         return load8(base + (size_t)row * ld + e);
     };
     auto k_chunk = [&](int kb, int c, int cpr) -> Vec8<T> {
-        const int key = kb + c / cpr, e = 8 * (c % cpr);
-        const int row = key < p.total ? key : p.total - 1;
-        return e < p.dim ? at(k_base, row, p.ldkv, e) : at(r_base, row, p.ldc, e - p.dim);
+        const int row = row_of(kb, c / cpr), e = 8 * (c % cpr);
+        return WINDOW || e < p.dim ? at(k_base, row, p.ldkv, e) : at(r_base, row, p.ldc, e - p.dim);
     };
     auto v_chunk = [&](int kb, int c, int cpr) -> Vec8<T> {
-        const int key = kb + c / cpr, e = 8 * (c % cpr);
-        return at(v_base, key < p.total ? key : p.total - 1, p.ldkv, e);
+        return at(v_base, row_of(kb, c / cpr), p.ldkv, 8 * (c % cpr));
     };
     constexpr int CK = 4 * NQ, CV = 2 * NV;                       // chunks per row (EXACT)
     constexpr int NCK = EXACT ? KB * CK / kSetThreads : 1, NCV = EXACT ? KB * CV / kSetThreads : 1;
@@ -137,13 +148,13 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
         }
     };
 
-    if (set < blocks) fetch(set);
-    for (int it0 = 0; it0 < blocks; it0 += SETS) {
+    if (first + set < blocks) fetch(first + set);
+    for (int it0 = first; it0 < blocks; it0 += SETS) {
         const int it = it0 + set, kb = it * KB;
         if (it < blocks) stage(it);
         __syncthreads();
         if (it + SETS < blocks) fetch(it + SETS);
-        if (it < blocks && kb <= wave_last) {
+        if (it < blocks && kb <= wave_last && kb + KB > wave_first) {
             floatx4 s[NKK][QB];
 #pragma unroll
             for (int kk = 0; kk < NKK; ++kk) {
@@ -169,6 +180,13 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
 #pragma unroll
                         for (int r = 0; r < 4; ++r)
                             if (kb + 16 * kk + 4 * g + r > qpos[b]) s[kk][b][r] = kMasked;
+                }
+                if (WINDOW && kb <= wave_last - p.window) {
+#pragma unroll
+                    for (int kk = 0; kk < NKK; ++kk)
+#pragma unroll
+                        for (int r = 0; r < 4; ++r)
+                            if (kb + 16 * kk + 4 * g + r <= qpos[b] - p.window) s[kk][b][r] = kMasked;
                 }
                 float v = kMasked;
 #pragma unroll
@@ -247,12 +265,12 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
         }
     }
 
-    const float snk = p.sink[head] * 1.4426950408889634f;
+    const float snk = p.sink ? p.sink[head] * 1.4426950408889634f : 0.f;
 #pragma unroll
     for (int b = 0; b < QB; ++b) {
         const int qi = q0 + 16 * b + ql;
         if (qi >= p.M) continue;
-        const float inv = 1.0f / (l[b][0] + exp2f(snk - m[b] * p.scale_log2));
+        const float inv = (WINDOW ? p.out_scale : 1.0f) / (l[b][0] + (p.sink ? exp2f(snk - m[b] * p.scale_log2) : 0.f));
         const int col = head * p.vdim + vcol0 + 4 * g;
         const T *gate = p.q + (size_t)qi * p.ldq + p.gate_off + col;
         T *dst = p.out + (size_t)qi * p.ldo + col;
@@ -260,9 +278,9 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
         for (int d = 0; d < NV; ++d)
             if (EXACT || d < nv) {
                 float z[4];
-                load4(gate + 16 * d, z);
+                if (!WINDOW) load4(gate + 16 * d, z);
 #pragma unroll
-                for (int r = 0; r < 4; ++r) z[r] = o[b][d][r] * inv * sigmoid_f32(z[r]);
+                for (int r = 0; r < 4; ++r) z[r] = o[b][d][r] * inv * (WINDOW ? 1.0f : sigmoid_f32(z[r]));
                 store4(dst + 16 * d, z[0], z[1], z[2], z[3]);
             }
     }
@@ -270,14 +288,14 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
 
 constexpr size_t kLdsLimit = 160 * 1024;
 
-template <class T, int NQ, int NV, int QB, int KB, int SETS, bool EXACT>
+template <class T, int NQ, int NV, int QB, int KB, int SETS, bool EXACT, bool WINDOW = false>
 hipError_t launch(const PrefillArgs<T> &p, hipStream_t stream) {
     const int vd = p.vdim < 16 * NV ? p.vdim : 16 * NV;
     size_t lds = (size_t)SETS * KB * ((p.dim + p.rot + 16 / sizeof(T)) + (vd + 32 / sizeof(T))) * sizeof(T);
     const size_t exchange = SETS == 2 ? 4 * QB * (4 * NV + 2) * 64 * sizeof(float) : 0;
     if (lds < exchange) lds = exchange;
     if (lds > kLdsLimit) return hipErrorInvalidValue;
-    auto kernel = &latent_prefill_kernel<T, NQ, NV, QB, KB, SETS, EXACT>;
+    auto kernel = &latent_prefill_kernel<T, NQ, NV, QB, KB, SETS, EXACT, WINDOW>;
     if (lds > 48 * 1024) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
@@ -289,7 +307,7 @@ hipError_t launch(const PrefillArgs<T> &p, hipStream_t stream) {
 
 template <class T>
 PrefillArgs<T> args_of(const LatentShape &s, const LatentRows &r, const void *kv, long ldkv, const float *sink, void *out, long ldo) {
-    PrefillArgs<T> p;
+    PrefillArgs<T> p{};
     p.q = static_cast<const T *>(r.proj);
     p.kv = static_cast<const T *>(kv);
     p.cache = static_cast<const T *>(r.cache);
@@ -309,6 +327,34 @@ PrefillArgs<T> args_of(const LatentShape &s, const LatentRows &r, const void *kv
     p.total = r.pos + r.M;
     p.scale_log2 = s.scale * 1.4426950408889634f;
     p.sink = sink;
+    p.head_k = s.dim;
+    p.head_v = s.vdim;
+    return p;
+}
+
+template <class T>
+PrefillArgs<T> args_of(const HeadShape &s, const HeadRows &r, const void *q, void *out, long ldo) {
+    PrefillArgs<T> p{};
+    p.q = static_cast<const T *>(q);
+    p.kv = p.cache = static_cast<const T *>(r.cache);
+    p.out = static_cast<T *>(out);
+    p.group = s.heads / s.kv_heads;
+    p.ldq = (long)p.group * s.dim;
+    p.head_q = s.dim;
+    p.group_q = (long)r.M * p.ldq;
+    p.ldkv = s.dim + s.vdim;
+    p.ldo = ldo;
+    p.heads = s.heads;
+    p.dim = s.dim;
+    p.vdim = s.vdim;
+    p.v_off = s.dim;
+    p.head_k = p.head_v = (long)s.ring * p.ldkv;
+    p.window = s.window;
+    p.ring = s.ring;
+    p.M = r.M;
+    p.total = r.pos + r.M;
+    p.scale_log2 = s.scale * 1.4426950408889634f;
+    p.out_scale = s.out_scale;
     return p;
 }
 
@@ -336,6 +382,29 @@ hipError_t launch_latent_prefill(int dtype, const LatentShape &s, const LatentRo
     if (nq <= 4 && nv <= 4) return launch<bf16, 4, 4, 1, 64, 1, false>(p, stream);
     if (nq <= 8 && nv <= 8) return launch<bf16, 8, 8, 1, 64, 1, false>(p, stream);
     return launch<bf16, 16, 16, 1, 32, 1, false>(p, stream);
+}
+
+bool head_prefill_supported(int dtype, const HeadShape &s) {
+    (void)dtype;
+    return s.dim <= 512;
+}
+
+hipError_t launch_head_prefill(int dtype, const HeadShape &s, const HeadRows &r, const void *q, void *out, long ldo, hipStream_t stream) {
+    const int nq = s.dim / 32, nv = s.vdim / 16;
+    if (dtype == kF32) {
+        const PrefillArgs<float> p = args_of<float>(s, r, q, out, ldo);
+        if (nq <= 4 && nv <= 4) return launch<float, 4, 4, 1, 32, 1, false, true>(p, stream);
+        if (nq <= 8 && nv <= 8) return launch<float, 8, 8, 1, 32, 1, false, true>(p, stream);
+        return launch<float, 16, 16, 1, 32, 1, false, true>(p, stream);
+    }
+    const PrefillArgs<bf16> p = args_of<bf16>(s, r, q, out, ldo);
+    if ((double)s.ring * (s.dim + s.vdim) * sizeof(bf16) < 4e9) {
+        if (nq == 4 && nv == 8) return launch<bf16, 4, 8, 2, 64, 2, true, true>(p, stream);
+        if (nq == 2 && nv == 4) return launch<bf16, 2, 4, 2, 64, 2, true, true>(p, stream);
+    }
+    if (nq <= 4 && nv <= 4) return launch<bf16, 4, 4, 1, 64, 1, false, true>(p, stream);
+    if (nq <= 8 && nv <= 8) return launch<bf16, 8, 8, 1, 64, 1, false, true>(p, stream);
+    return launch<bf16, 16, 16, 1, 32, 1, false, true>(p, stream);
 }
 
 }  // namespace w4a16

@@ -92,7 +92,58 @@ __global__ void __launch_bounds__(kRowThreads) norm_rows_kernel(const float *res
     }
 }
 
+// the residual brought up to date and its norm: what the sublayers of a model with norms on their inputs read
+template <class T>
+__global__ void __launch_bounds__(kRowThreads) add_norm_rows_kernel(float *res, const float *y, const int32_t *tokens, const T *embed, float scale,
+                                                                    const float *norm_w, float eps, int true_width, T *h, int width) {
+    extern __shared__ float sum_lds[];
+    __shared__ float red[4];
+    const size_t m = blockIdx.x;
+    const T *row = tokens ? embed + (size_t)tokens[m] * width : nullptr;
+    float ss = 0.f;
+    for (int i = 4 * threadIdx.x; i < width; i += 4 * kRowThreads) {
+        float v[4];
+        if (row) {
+            load4(row + i, v);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] *= scale;
+        } else {
+            load4(res + m * width + i, v);
+            if (y) {
+                float u[4];
+                load4(y + m * width + i, u);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) v[j] += u[j];
+            }
+        }
+        if (row || y) store4(res + m * width + i, v[0], v[1], v[2], v[3]);
+        store4(sum_lds + i, v[0], v[1], v[2], v[3]);   // read back by the same thread
+#pragma unroll
+        for (int j = 0; j < 4; ++j) ss = fmaf(v[j], v[j], ss);
+    }
+    if (!h) return;
+    const float rstd = 1.0f / sqrtf(row_total(ss, red) / (float)true_width + eps);
+    for (int i = 4 * threadIdx.x; i < width; i += 4 * kRowThreads) {
+        float v[4], w[4];
+        load4(sum_lds + i, v);
+        load4(norm_w + i, w);
+        store4(h + m * width + i, v[0] * rstd * w[0], v[1] * rstd * w[1], v[2] * rstd * w[2], v[3] * rstd * w[3]);
+    }
+}
+
 }  // namespace
+
+hipError_t launch_add_norm_rows(int dtype, float *res, const float *y, const int32_t *tokens, const void *embed, float scale, const float *norm_w,
+                                float eps, int true_width, void *h, int M, int width, hipStream_t stream) {
+    const size_t lds = (size_t)width * sizeof(float);   // (the C ABI keeps width within 64 KiB)
+    if (dtype == kF32)
+        hipLaunchKernelGGL(add_norm_rows_kernel<float>, dim3(M), dim3(kRowThreads), lds, stream, res, y, tokens, static_cast<const float *>(embed), scale,
+                           norm_w, eps, true_width, static_cast<float *>(h), width);
+    else
+        hipLaunchKernelGGL(add_norm_rows_kernel<bf16>, dim3(M), dim3(kRowThreads), lds, stream, res, y, tokens, static_cast<const bf16 *>(embed), scale, norm_w,
+                           eps, true_width, static_cast<bf16 *>(h), width);
+    return hipGetLastError();
+}
 
 hipError_t launch_embed_rows(int dtype, const int32_t *tokens, const void *embed, float scale, float *res, void *h, int M, int width,
                              hipStream_t stream) {

@@ -256,7 +256,8 @@ def test_dense_abi_rejects_bad_arguments_before_touching_the_gpu():
         assert s(r(**k)) == SHAPE, k
     assert s(r(logits=None)) == NULL
     a = lambda **k: lib.dlm_gemm(0, ctypes.byref(_lib.GemmArgs(**{**dict(a=p, w=p, out=p, lda=64, ldo=32, M=3, N=32, K=64, tile_rows=32), **k})), None)
-    for k in (dict(K=96 - 8), dict(N=24), dict(lda=56), dict(ldo=16), dict(M=0), dict(tile_rows=64), dict(epilogue=2), dict(epilogue=3)):
+    for k in (dict(K=96 - 8), dict(N=24), dict(lda=56), dict(ldo=16), dict(M=0), dict(tile_rows=64), dict(epilogue=4), dict(epilogue=2, N=16), dict(epilogue=3, N=48),
+              dict(silu_begin=0, silu_end=8), dict(silu_begin=0, silu_end=16, epilogue=1)):
         assert a(**k) == SHAPE, k
     assert a(tiles=p) == NULL and a(tiles=p, order=p, n_tiles=1, w_stride=5) == SHAPE
     shape = dict(heads=2, dim=32, rot=32, vdim=32, rank=64, rot_pairs=4, true_rank=64, scale=1.0)
