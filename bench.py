@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the MI355X W4A16 path.  One JSON line on stdout.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload gemv|probe|gemv_awq|dequant|gemm16|gemm64|gemm64_down|gemm16_awq|prefill|prefill_awq|ffn|ffn_awq|block|block_awq|layer|layer_awq|q4nx_gemv|q4nx_gemm16|q4nx_prefill|lm_head|decode_1b|decode_8b|prefill_block|prefill_block_awq|prefill_1b|prefill_1b_awq|prefill_8b|kuvonex]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload gemv|probe|gemv_awq|dequant|gemm16|gemm64|gemm64_down|gemm16_awq|prefill|prefill_awq|ffn|ffn_awq|block|block_awq|layer|layer_awq|q4nx_gemv|q4nx_gemm16|q4nx_prefill|lm_head|decode_1b|decode_8b|prefill_block|prefill_block_awq|prefill_1b|prefill_1b_awq|prefill_8b|kuvonex|sitirax]
 
 Default workload is the decode GEMV (x bf16 [1,4096], W int4 [4096 x 11008], group 128).
 A step is one launch of the hot path on synthetic inputs that are already resident in HBM.
@@ -753,6 +753,23 @@ def llama_costs(c, M, pos):
     return flops, c["n_layers"] * layer + 2 * c["vocab_size"] * E
 
 
+def measure_models(rows, steps, warmup, prompt_len):
+    """name -> (make, (flops of the prompt, bytes of a token)) -> name -> prompt pass and greedy decode, one model at a time."""
+    import torch
+
+    out = {}
+    for name, (make, (flops, nbytes)) in rows.items():
+        model = make()
+        pre, dec, ok = time_model(model, prompt_len, steps, warmup, 3)
+        del model
+        torch.cuda.empty_cache()
+        out[name] = {"prefill_ms": pre * 1e3, "prefill_tokens_per_s": prompt_len / pre, "prefill_TFLOP/s": flops / pre / 1e12,
+                     "prefill_frac_mfma_peak": flops / pre / 1e12 / MFMA_BF16_PEAK_TFLOPS, "decode_us_per_token": dec * 1e6,
+                     "decode_tokens_per_s": 1 / dec, "decode_GB/s": nbytes / dec / 1e9, "decode_frac_hbm_peak": nbytes / dec / 1e9 / HBM_PEAK_GBS,
+                     "finite": ok}
+    return out
+
+
 def run_kuvonex(steps, warmup, only=None, prompt_len=2048, llama=True):
     """Prompt pass and greedy decode of the Kuvonex sizes and of the int4 Llama layers beside them."""
     import torch
@@ -764,16 +781,74 @@ def run_kuvonex(steps, warmup, only=None, prompt_len=2048, llama=True):
         if llama:
             c = KUVONEX_SIZES[size]["llama"]
             rows["llama_int4"] = (lambda: random_llama(c), llama_costs(c, prompt_len, prompt_len + steps // 2))
-        out[size] = {}
-        for name, (make, (flops, nbytes)) in rows.items():
-            model = make()
-            pre, dec, ok = time_model(model, prompt_len, steps, warmup, 3)
-            del model
-            torch.cuda.empty_cache()
-            out[size][name] = {"prefill_ms": pre * 1e3, "prefill_tokens_per_s": prompt_len / pre, "prefill_TFLOP/s": flops / pre / 1e12,
-                               "prefill_frac_mfma_peak": flops / pre / 1e12 / MFMA_BF16_PEAK_TFLOPS, "decode_us_per_token": dec * 1e6,
-                               "decode_tokens_per_s": 1 / dec, "decode_GB/s": nbytes / dec / 1e9, "decode_frac_hbm_peak": nbytes / dec / 1e9 / HBM_PEAK_GBS,
-                               "finite": ok}
+        out[size] = measure_models(rows, steps, warmup, prompt_len)
+    return out
+
+
+# Sitirax layers (even ones: windowed grouped attention beside lightning attention, odd ones: the gated delta rule; a gated
+# feed-forward in each) beside Kuvonex layers of the same width, layer count, vocabulary and feed-forward length per token.
+SITIRAX_SIZES = {
+    "w2048": dict(width=2048, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, rank=128, conv=4, ff=8192, vocab=32768),
+    "w4096": dict(width=4096, layers=4, heads=32, kv_heads=8, dim=128, vdim=128, window=1024, rank=128, conv=4, ff=14336, vocab=32768),
+}
+
+
+def random_sitirax(size, dtype=None):
+    """A random-weight model of SITIRAX_SIZES[size]."""
+    import torch
+
+    from air_hip import sitirax
+
+    z = SITIRAX_SIZES[size]
+    heads = dict(heads=z["heads"], dim=z["dim"], vdim=z["vdim"])
+    left = dict(heads, kv_heads=z["kv_heads"], scale=z["dim"] ** -0.5, mask=dict(size=z["window"]))
+    right = dict(heads, decay=[1.0 - 2.0 ** (-1 - 8 * h / z["heads"]) for h in range(z["heads"])])
+    mixers = [dict(type="parallel", mixer=dict(left=left, right=right, left_scale=1.0, right_scale=1.0)),
+              dict(type="channel_delta", mixer=dict(heads, kv_heads=z["heads"], conv=z["conv"]))]
+    layers = [dict(mixers[i % 2], mlp=dict(kind="dense", ff=z["ff"])) for i in range(z["layers"])]
+    cfg = sitirax.SitiraxConfig.from_json(dict(vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-6), logit_scale=1.0, layers=layers))
+    g = torch.Generator(device="cuda")
+    g.manual_seed(7)
+
+    def tensor(name, shape):
+        shape = [z["rank"] if n is None else n for n in shape]
+        t = torch.randn(shape, device="cuda", generator=g)
+        if "norm" in name:
+            return 1.0 + 0.1 * t
+        if name.endswith("A_log") or name.endswith("dt_bias"):
+            return t - 2.0
+        return t.mul_(1.0 if name == "embed" else shape[-1] ** -0.5).to(torch.bfloat16)
+
+    return sitirax.SitiraxModel(cfg, tensor, dtype or torch.bfloat16)
+
+
+def sitirax_costs(size, M, pos):
+    """(FLOPs of a prompt of M tokens, bytes of a decoded token at position pos) the algorithm needs."""
+    z = SITIRAX_SIZES[size]
+    W, H, G, D, V, R = z["width"], z["heads"], z["kv_heads"], z["dim"], z["vdim"], z["rank"]
+    pairs, ff = (z["layers"] + 1) // 2, 3 * W * z["ff"]
+    deltas = z["layers"] - pairs
+    parallel = W * (H * D + G * (D + V) + H * V) + W * H * (2 * D + 3 * V)
+    delta = W * (2 * H * D + 2 * H * V + H + 2 * R) + R * H * (D + V)
+    weights = pairs * (parallel + ff) + deltas * (delta + ff)
+    seen = sum(min(i + 1, z["window"]) for i in range(M))
+    flops = 2 * M * weights + pairs * 2 * seen * H * (D + V) + 2 * W * z["vocab"]
+    flops += M * H * 2 * D * V * (2 * pairs + 3 * deltas)                # the recurrences token by token
+    state = 2 * 4 * H * D * V                                            # read and written
+    return flops, 2 * (weights + W * z["vocab"]) + z["layers"] * state + pairs * 2 * min(pos, z["window"]) * G * (D + V)
+
+
+def run_sitirax(steps, warmup, only=None, prompt_len=2048, kuvonex=True):
+    """Prompt pass and greedy decode of the Sitirax sizes and of the Kuvonex layers beside them."""
+    import torch
+
+    torch.cuda.set_device(0)
+    out = {}
+    for size in ([only] if only else SITIRAX_SIZES):
+        rows = {"sitirax": (lambda: random_sitirax(size), sitirax_costs(size, prompt_len, prompt_len + steps // 2))}
+        if kuvonex:
+            rows["kuvonex"] = (lambda: random_kuvonex(size), kuvonex_costs(size, prompt_len, prompt_len + steps // 2))
+        out[size] = measure_models(rows, steps, warmup, prompt_len)
     return out
 
 
@@ -874,9 +949,10 @@ def main():
     ap.add_argument("--steps", type=int, default=200)
     ap.add_argument("--warmup", type=int, default=20)
     ap.add_argument("--workload", default="gemv", choices=list(CONFIGS) + ["decode_1b", "decode_8b", "prefill_block", "prefill_block_awq", "prefill_1b", "prefill_1b_awq",
-                                                             "prefill_8b", "kuvonex"])
-    ap.add_argument("--size", choices=list(KUVONEX_SIZES), help="--workload kuvonex: this size only")
+                                                             "prefill_8b", "kuvonex", "sitirax"])
+    ap.add_argument("--size", choices=list(KUVONEX_SIZES), help="--workload kuvonex, sitirax: this size only")
     ap.add_argument("--no-llama", action="store_true", help="--workload kuvonex: without the int4 Llama layers beside it")
+    ap.add_argument("--no-kuvonex", action="store_true", help="--workload sitirax: without the Kuvonex layers beside it")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-extra", action="store_true", help="skip the short runs of the other configs")
     ap.add_argument("--copy-probe", action="store_true",
@@ -903,16 +979,19 @@ def main():
         dst.copy_(src)
         torch.cuda.synchronize()
         del src, dst
-    if a.workload == "kuvonex":
+    if a.workload in ("kuvonex", "sitirax"):
         steps, warmup = min(a.steps, 64), min(a.warmup, 4)
-        r = run_kuvonex(steps, warmup, a.size, llama=not a.no_llama)
+        if a.workload == "kuvonex":
+            r, sizes = run_kuvonex(steps, warmup, a.size, llama=not a.no_llama), KUVONEX_SIZES
+        else:
+            r, sizes = run_sitirax(steps, warmup, a.size, kuvonex=not a.no_kuvonex), SITIRAX_SIZES
         size, first = next(iter(r.items()))
-        k = first["kuvonex"]
+        k = first[a.workload]
         print(json.dumps({
-            "metric": f"Kuvonex decode tokens/s, size {size}, batch 1", "value": k["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
+            "metric": f"{a.workload.capitalize()} decode tokens/s, size {size}, batch 1", "value": k["decode_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
             "warmup": warmup, "ms_per_step": k["decode_us_per_token"] * 1e-3, "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
             "dtype": "bf16 weights and activations, fp32 residual and accumulate", "data": "synthetic (random weights of the architecture, random prompt)",
-            "config": {"workload": "prompt pass of 2048 tokens, then greedy decode behind it", "sizes": {s: KUVONEX_SIZES[s] for s in r},
+            "config": {"workload": "prompt pass of 2048 tokens, then greedy decode behind it", "sizes": {s: sizes[s] for s in r},
                        "timing": "one HIP graph of the pass / of all token steps, events on the launch stream"},
             "roofline": {"bound": "hbm", "achieved": k["decode_GB/s"], "peak": HBM_PEAK_GBS, "unit": "GB/s", "frac": k["decode_frac_hbm_peak"],
                          "traffic": None, "avg_launch_us": k["decode_us_per_token"]},
