@@ -106,3 +106,67 @@ KUVONEX_MIXED = kuvonex_config([
     kuvonex_layer(heads=5, dim=16, rot_dim=8, vdim=24, kv_rank=56, kv_from=0, scale=0.31, mlp=(6, 2, 6, 3, 72)),
     kuvonex_layer(heads=1, dim=8, rot_dim=12, vdim=8, kv_rank=72, base=90.0, kv_from=1, mlp=(4, 2, 1, 1, 8)),
 ], vocab=67, width=72)
+
+
+# ---- Sitirax ------------------------------------------------------------------------------------------------------------
+def sitirax_parallel(heads=4, kv_heads=2, dim=24, vdim=40, window=37, scale=None, right_heads=3, right_dim=40, right_vdim=24, decay=None, left_scale=0.7,
+                     right_scale=1.3, ff=None, weights_of=None):
+    """One 'parallel' entry of `layers` of a Sitirax config.json."""
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5 if scale is None else scale, "mask": {"size": window}}
+    right = {"heads": right_heads, "dim": right_dim, "vdim": right_vdim, "decay": list(decay or np.linspace(0.4, 1.0, right_heads))}
+    return _sitirax_layer("parallel", {"left": left, "right": right, "left_scale": left_scale, "right_scale": right_scale}, ff, weights_of)
+
+
+def sitirax_delta(heads=4, kv_heads=2, dim=24, vdim=40, conv=3, ff=None, weights_of=None):
+    """One 'channel_delta' entry."""
+    return _sitirax_layer("channel_delta", {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}, ff, weights_of)
+
+
+def _sitirax_layer(kind, mixer, ff, weights_of):
+    out = {"type": kind, "mixer": mixer, "mlp": None if ff is None else {"kind": "dense", "ff": ff}}
+    if weights_of is not None:
+        out["weights_of"] = weights_of
+    return out
+
+
+def sitirax_config(layers, vocab=67, width=72, eps=1e-5, logit_scale=0.6):
+    return {"architecture": "Sitirax", "vocab": vocab, "width": width, "norm": {"eps": eps}, "logit_scale": logit_scale, "layers": layers}
+
+
+def sitirax_weights(config, seed=0, ranks=(20, 33)):
+    """Random weights as float32 arrays that hold bf16 values, by checkpoint name; ranks: of the decay's and the gate's two factors."""
+    from air_hip import sitirax
+
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in sitirax.tensor_shapes(sitirax.SitiraxConfig.from_json(config)).items():
+        shape = tuple((ranks[0] if ".a" in name else ranks[1]) if n is None else n for n in shape)
+        v = rng.standard_normal(shape)
+        if name.endswith(("norm", "norm1", "norm2")):
+            v = 1.0 + 0.3 * v
+        elif name.endswith("A_log"):
+            v = 0.7 * v - 1.0
+        elif name.endswith("dt_bias"):
+            v = 2.0 * v - 1.0                # channels that forget at once and channels that hardly do
+        elif name == "embed":
+            v = v * 0.8
+        else:
+            v = v * shape[-1] ** -0.5 * (1.5 if ".b" in name or ".a" in name else 1.0)
+        out[name] = bf16_bits_to_f32(f32_to_bf16_bits(v.astype(np.float32)))
+    return out
+
+
+sitirax_write = kuvonex_write
+
+# Every size different; shared weights of either kind, with and without a feed-forward; a window of one, a convolution of one tap,
+# one key / value head for all, heads of more than 64 channels.
+SITIRAX_MIXED = sitirax_config([
+    sitirax_parallel(ff=40),
+    sitirax_delta(),
+    sitirax_parallel(ff=40, weights_of=0),
+    sitirax_delta(heads=3, kv_heads=3, dim=72, vdim=16, conv=1, ff=72),
+    sitirax_parallel(heads=5, kv_heads=1, dim=8, vdim=8, window=1, right_heads=1, right_dim=8, right_vdim=72, decay=[0.999], left_scale=-0.4, right_scale=1.0),
+    sitirax_delta(heads=3, kv_heads=3, dim=72, vdim=16, conv=1, ff=72, weights_of=3),
+    sitirax_delta(heads=2, kv_heads=1, dim=40, vdim=72, conv=5),
+    sitirax_parallel(heads=2, kv_heads=2, dim=72, vdim=24, window=70, scale=0.4, right_heads=4, right_dim=72, right_vdim=8, ff=24),
+], vocab=67, width=72)
