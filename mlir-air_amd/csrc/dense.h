@@ -68,6 +68,15 @@ __device__ __forceinline__ void unpack8(const Vec8<float> &v, float (&f)[8]) {
     }
 }
 
+template <class T>
+__device__ __forceinline__ Vec8<T> pack8(const float (&f)[8]);
+template <>
+__device__ __forceinline__ Vec8<bf16> pack8<bf16>(const float (&f)[8]) {
+    return {u32x4{pack_bf16x2(f[0], f[1]), pack_bf16x2(f[2], f[3]), pack_bf16x2(f[4], f[5]), pack_bf16x2(f[6], f[7])}};
+}
+template <>
+__device__ __forceinline__ Vec8<float> pack8<float>(const float (&f)[8]) { return {floatx4{f[0], f[1], f[2], f[3]}, floatx4{f[4], f[5], f[6], f[7]}}; }
+
 // four floats -> four consecutive elements (8 or 16 bytes, aligned)
 __device__ __forceinline__ void store4(bf16 *p, float a, float b, float c, float d) {
     *reinterpret_cast<uint2 *>(p) = uint2{pack_bf16x2(a, b), pack_bf16x2(c, d)};
@@ -154,6 +163,12 @@ __device__ __forceinline__ Vec8<float> pair8<float>(floatx4 a, floatx4 b) { retu
 
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
+// the same by the hardware's reciprocal where the result is rounded to bf16 anyway
+template <class T>
+__device__ __forceinline__ float sigmoid_of(float z) {
+    if constexpr (sizeof(T) == 2) return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+    return sigmoid_f32(z);
+}
 __device__ __forceinline__ float gelu_tanh_f32(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * z * z, z, z))); }
 __device__ __forceinline__ float softplus_f32(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 

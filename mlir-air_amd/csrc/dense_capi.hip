@@ -339,7 +339,7 @@ int dlm_head_merge(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, i
 
 int dlm_short_conv(int dtype, const dlm_short_conv_args *c, void *act, void *stream) {
     if (!c || !c->proj || !c->w || !c->history || !c->factors || !act) return DLM_ERR_NULL;
-    if (bad_type(dtype) || c->k_heads <= 0 || c->heads <= 0 || c->dim <= 0 || c->dim % 4 || c->vdim <= 0 || c->vdim % 4 || c->taps <= 0 || c->M <= 0 ||
+    if (bad_type(dtype) || c->k_heads <= 0 || c->heads <= 0 || c->dim <= 0 || c->dim % 8 || c->vdim <= 0 || c->vdim % 8 || c->taps <= 0 || c->M <= 0 ||
         c->M > 65535 * 4 || c->pos < 0 || c->ld % 8 || c->off < 0 || c->off % 8 || c->taps > 65535 || (c->pos_dev && c->M > 1) || !(c->unit_eps >= 0.f))
         return DLM_ERR_SHAPE;
     if (odd(c->proj) || odd(c->w) || odd(c->history) || odd(act)) return DLM_ERR_ALIGN;

@@ -13,10 +13,10 @@ namespace {
 
 constexpr int kPrepThreads = 256;
 
-// Vectors of one head by groups of `lanes` lanes, four elements per lane at a time.
+// Vectors of one head by groups of `lanes` lanes, eight elements per lane at a time.
 __host__ __device__ inline int lanes_of(int n) {
     int l = 1;
-    while (l < 64 && 4 * l < n) l *= 2;
+    while (l < 64 && 8 * l < n) l *= 2;
     return l;
 }
 
@@ -37,20 +37,27 @@ __global__ void __launch_bounds__(kPrepThreads) head_prepare_kernel(const HeadSh
     float rstd = 1.f;
     if (!is_v) {
         float ss = 0.f;
-        for (int i = 4 * lane; i < n; i += 4 * lanes) {
-            float v[4];
-            load4(src + i, v);
+        for (int i = 8 * lane; i < n; i += 8 * lanes) {
+            float v[8];
+            unpack8(load8(src + i), v);
 #pragma unroll
-            for (int j = 0; j < 4; ++j) ss = fmaf(v[j], v[j], ss);
+            for (int j = 0; j < 8; ++j) ss = fmaf(v[j], v[j], ss);
         }
         rstd = 1.0f / sqrtf(group_sum(ss, lanes) / (float)s.true_dim + eps);
     }
     const float *w = is_q ? q_norm : k_norm;
-    for (int i = 4 * lane; i < n; i += 4 * lanes) {
-        float v[4], f[4] = {1.f, 1.f, 1.f, 1.f};
-        load4(src + i, v);
-        if (!is_v) load4(w + i, f);
-        store4(dst + i, v[0] * rstd * f[0], v[1] * rstd * f[1], v[2] * rstd * f[2], v[3] * rstd * f[3]);
+    for (int i = 8 * lane; i < n; i += 8 * lanes) {
+        const Vec8<T> x = load8(src + i);
+        if (is_v) {
+            store8(dst + i, x);
+            continue;
+        }
+        float v[8], f[8];
+        unpack8(x, v);
+        unpack8(load8(w + i), f);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] *= rstd * f[j];
+        store8(dst + i, pack8<T>(v));
     }
 }
 

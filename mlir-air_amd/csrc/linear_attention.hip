@@ -17,15 +17,16 @@ namespace {
 
 constexpr int kThreads = 256;
 
-int lanes_of(int n) {
+// lanes that share a vector of n elements, `each` elements per lane at a time
+int lanes_of(int n, int each) {
     int l = 1;
-    while (l < 64 && 4 * l < n) l *= 2;
+    while (l < 64 && each * l < n) l *= 2;
     return l;
 }
 
 constexpr int kConvTokens = 4;   // tokens per thread
 
-// Vectors (q and k heads, then v heads) by groups of `lanes` lanes, four channels per lane at a time; blockIdx.y: kConvTokens tokens.
+// Vectors (q and k heads, then v heads) by groups of `lanes` lanes, eight channels per lane at a time; blockIdx.y: kConvTokens tokens.
 // Rows in front of the portion come from the history, a ring of `taps` rows by position.
 template <class T>
 __global__ void __launch_bounds__(kThreads) short_conv_kernel(const ConvArgs c, const T *proj, T *history, T *act, int lanes) {
@@ -35,41 +36,58 @@ __global__ void __launch_bounds__(kThreads) short_conv_kernel(const ConvArgs c, 
     const bool is_v = unit >= 2 * c.k_heads;
     const int c0 = is_v ? 2 * c.k_heads * c.dim + (unit - 2 * c.k_heads) * c.vdim : unit * c.dim, n = is_v ? c.vdim : c.dim;
     const int pos0 = c.pos_dev ? c.pos_dev[0] : c.pos, m0 = blockIdx.y * kConvTokens;
+    const bool inside = m0 >= c.taps - 1 && m0 + kConvTokens <= c.M;   // every row is one of the portion
     float ss[kConvTokens] = {0.f, 0.f, 0.f, 0.f};
-    for (int i = 4 * lane; i < n; i += 4 * lanes) {
+    for (int i = 8 * lane; i < n; i += 8 * lanes) {
         const int ch = c0 + i;
-        float acc[kConvTokens][4];
+        float acc[kConvTokens][8];
 #pragma unroll
         for (int t = 0; t < kConvTokens; ++t)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) acc[t][e] = 0.f;
-        for (int j = 0; j < c.taps; ++j) {
-            float w[4];
-            load4(c.w + (size_t)j * C + ch, w);
+            for (int e = 0; e < 8; ++e) acc[t][e] = 0.f;
+        if (inside) {
+            for (int j = 0; j < c.taps; ++j) {
+                const T *row = proj + (size_t)(m0 + j - (c.taps - 1)) * c.ld + ch;
+                float w[8];
+                unpack8(load8(c.w + (size_t)j * C + ch), w);
+                Vec8<T> v[kConvTokens];
 #pragma unroll
-            for (int t = 0; t < kConvTokens; ++t) {
-                const int m = m0 + t, r = m + j - (c.taps - 1);       // row of the portion that meets this tap
-                if (m >= c.M || pos0 + r < 0) continue;
-                float x[4];
-                load4(r >= 0 ? proj + (size_t)r * c.ld + ch : history + (size_t)((pos0 + r) % c.taps) * C + ch, x);
+                for (int t = 0; t < kConvTokens; ++t) v[t] = load8(row + (size_t)t * c.ld);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) acc[t][e] = fmaf(w[e], x[e], acc[t][e]);
+                for (int t = 0; t < kConvTokens; ++t) {
+                    float x[8];
+                    unpack8(v[t], x);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) acc[t][e] = fmaf(w[e], x[e], acc[t][e]);
+                }
+            }
+        } else {
+            for (int j = 0; j < c.taps; ++j) {
+                float w[8];
+                unpack8(load8(c.w + (size_t)j * C + ch), w);
+#pragma unroll
+                for (int t = 0; t < kConvTokens; ++t) {
+                    const int m = m0 + t, r = m + j - (c.taps - 1);       // row of the portion that meets this tap
+                    if (m >= c.M || pos0 + r < 0) continue;
+                    float x[8];
+                    unpack8(load8(r >= 0 ? proj + (size_t)r * c.ld + ch : history + (size_t)((pos0 + r) % c.taps) * C + ch), x);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) acc[t][e] = fmaf(w[e], x[e], acc[t][e]);
+                }
             }
         }
 #pragma unroll
         for (int t = 0; t < kConvTokens; ++t) {
             if (m0 + t >= c.M) continue;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) acc[t][e] = to_float(from_float<T>(silu_f32(acc[t][e])));   // (the norm is that of what is stored)
+            for (int e = 0; e < 8; ++e) acc[t][e] *= sigmoid_of<T>(acc[t][e]);
+            const Vec8<T> out = pack8<T>(acc[t]);
+            store8(act + (size_t)(m0 + t) * C + ch, out);
+            unpack8(out, acc[t]);   // (the norm is that of what is stored)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) ss[t] = fmaf(acc[t][e], acc[t][e], ss[t]);
-            store4(act + (size_t)(m0 + t) * C + ch, acc[t][0], acc[t][1], acc[t][2], acc[t][3]);
+            for (int e = 0; e < 8; ++e) ss[t] = fmaf(acc[t][e], acc[t][e], ss[t]);
         }
-        if (c.M == 1) {   // one token: its row goes into the history here (no other thread reads these channels, nor this slot)
-            float x[4];
-            load4(proj + ch, x);
-            store4(history + (size_t)(pos0 % c.taps) * C + ch, x[0], x[1], x[2], x[3]);
-        }
+        if (c.M == 1) store8(history + (size_t)(pos0 % c.taps) * C + ch, load8(proj + ch));   // (nobody else reads these channels, nor this slot)
     }
     if (is_v) return;
 #pragma unroll
@@ -183,7 +201,7 @@ __global__ void __launch_bounds__(kThreads) gated_norm_heads_kernel(const GatedN
         float z[4];
         load4(gate + m * g.ld_gate + (size_t)grp * g.cols + i, z);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) z[j] = v[j] * rstd * w[j] * sigmoid_f32(z[j]);
+        for (int j = 0; j < 4; ++j) z[j] = v[j] * rstd * w[j] * sigmoid_of<T>(z[j]);
         store4(out + m * g.ld_out + (size_t)grp * g.cols + i, z[0], z[1], z[2], z[3]);
     }
 }
@@ -209,14 +227,14 @@ __global__ void __launch_bounds__(kThreads) gated_norm_row_kernel(const GatedNor
         float z[4];
         load4(gate + m * g.ld_gate + i, z);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) z[j] = v[j] * rstd * w[j] * sigmoid_f32(z[j]);
+        for (int j = 0; j < 4; ++j) z[j] = v[j] * rstd * w[j] * sigmoid_of<T>(z[j]);
         store4(out + m * g.ld_out + i, z[0], z[1], z[2], z[3]);
     }
 }
 
 template <class T>
 hipError_t conv(const ConvArgs &c, const void *proj, void *history, void *act, hipStream_t stream) {
-    const int lanes = lanes_of(c.dim > c.vdim ? c.dim : c.vdim), per = kThreads / lanes, units = 2 * c.k_heads + c.heads;
+    const int lanes = lanes_of(c.dim > c.vdim ? c.dim : c.vdim, 8), per = kThreads / lanes, units = 2 * c.k_heads + c.heads;
     const T *x = static_cast<const T *>(proj) + c.off;
     hipLaunchKernelGGL(short_conv_kernel<T>, dim3((units + per - 1) / per, (c.M + kConvTokens - 1) / kConvTokens), dim3(kThreads), 0, stream, c, x,
                        static_cast<T *>(history), static_cast<T *>(act), lanes);
@@ -261,7 +279,7 @@ hipError_t launch_recurrence_steps(int dtype, const LinearArgs &a, float *o, hip
 
 hipError_t launch_gated_norm(int dtype, const GatedNorm &g, const void *gate, void *out, int M, hipStream_t stream) {
     const bool row = g.groups == 1 && g.cols > 256;
-    const int lanes = lanes_of(g.cols), per = kThreads / lanes;
+    const int lanes = lanes_of(g.cols, 4), per = kThreads / lanes;
     const dim3 grid = row ? dim3(M) : dim3((g.groups + per - 1) / per, M);
     auto run = [&](auto tag) {
         using T = decltype(tag);
