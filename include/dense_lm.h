@@ -217,6 +217,19 @@ int dlm_recurrence_chunks(int dtype, const dlm_recurrence_args *a, void *work, f
 int dlm_gated_norm(int dtype, const float *o, const float *w, const void *gate, int64_t ld_gate, void *out, int64_t ld_out, int M, int groups, int cols,
                    int true_cols, float eps, void *stream);
 
+/* Steps of one token (M = 1) that do not wait for each other in one launch.  _begin: dlm_head_prepare and dlm_recurrence_steps (a decay
+ * per head); _end: dlm_head_merge into out and the norm and gate (dlm_gated_norm with one group) into norm_out; dlm_conv_products:
+ * dlm_short_conv and out_a[Na] (fp32) = w_a[Na, Ka] x_a, out_b[Nb] (element type) = w_b[Nb, Kb] x_b (K multiples of 64, N of 16). */
+int dlm_head_state_begin(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, void *q, const dlm_recurrence_args *a, float *o, void *stream);
+int dlm_head_state_end(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, int nsplit, const float *part_o, const float *part_ml, void *out,
+                       const float *o, const float *w, const void *gate, int cols, int true_cols, float eps, void *norm_out, void *stream);
+typedef struct {
+    const void *w, *x;
+    void *out;
+    int32_t K, N;
+} dlm_short_product;
+int dlm_conv_products(int dtype, const dlm_short_conv_args *c, void *act, const dlm_short_product *a, const dlm_short_product *b, void *stream);
+
 #ifdef __cplusplus
 }
 #endif

@@ -128,6 +128,10 @@ class ShortConvArgs(ctypes.Structure):
                 ("dim", _i32), ("vdim", _i32), ("taps", _i32), ("off", _i32), ("M", _i32), ("pos", _i32), ("q_scale", _cf), ("unit_eps", _cf)]
 
 
+class ShortProduct(ctypes.Structure):
+    _fields_ = [("w", _vp), ("x", _vp), ("out", _vp), ("K", _i32), ("N", _i32)]
+
+
 class RecurrenceArgs(ctypes.Structure):
     _fields_ = [("qkv", _vp), ("log2_decay", _vp), ("z", _vp), ("a_log", _vp), ("dt_bias", _vp), ("factors", _vp), ("beta", _vp), ("state", _vp),
                 ("pos_dev", _vp), ("ld", _i64), ("ld_beta", _i64), ("k_heads", _i32), ("heads", _i32), ("dim", _i32), ("vdim", _i32),
@@ -163,6 +167,9 @@ DENSE_SYMBOLS = {
     "dlm_recurrence_steps": (_ci, [_ci] + [_vp] * 3),
     "dlm_recurrence_chunk_bytes": (_sz, [_vp]),
     "dlm_recurrence_chunks": (_ci, [_ci] + [_vp] * 4),
+    "dlm_head_state_begin": (_ci, [_ci] + [_vp] * 6),
+    "dlm_head_state_end": (_ci, [_ci, _vp, _vp, _ci] + [_vp] * 6 + [_ci, _ci, _cf, _vp, _vp]),
+    "dlm_conv_products": (_ci, [_ci] + [_vp] * 5),
     "dlm_gated_norm": (_ci, [_ci, _vp, _vp, _vp, _i64, _vp, _i64] + [_ci] * 4 + [_cf, _vp]),
     "dlm_latent_decode_supported": (_ci, [_ci, _vp]),
     "dlm_latent_prefill_supported": (_ci, [_ci, _vp]),

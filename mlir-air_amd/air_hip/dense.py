@@ -192,13 +192,6 @@ def gemm(a, w, out_f32=False, lda=None, rows=None, out=None, silu=None, gate=GAT
     return out
 
 
-def product(a, w, out_f32=False):
-    """gemm, or the one-token product for a single row."""
-    if a.shape[0] == 1:
-        return gemv(a.reshape(-1), w, out_f32).reshape(1, -1)
-    return gemm(a, w, out_f32)
-
-
 def embed_rows(tokens, embed, scale):
     """(residual fp32 [M, K], the same in the element type) of int32 tokens [M]."""
     lib = _lib.load_dense_library()
@@ -470,10 +463,22 @@ def head_attention(spec, proj, off, q_norm, k_norm, eps, cache, pos, out, pos_de
     """Windowed attention of the rows of proj [M, ld] (q, k, v from column `off` on) at positions pos .. into the first columns of
     out [M, ldo]; their keys and values are appended to cache [kv_heads, ring, dim + vdim].  rows_form: the kernel for many rows."""
     lib = _lib.load_dense_library()
+    M, dt = proj.shape[0], dtype_code(proj)
+    s, r, q = _head_args(spec, proj, off, q_norm, k_norm, eps, cache, pos, out, pos_dev)
+    _lib.check_dense(lib.dlm_head_prepare(dt, s, r, _ptr(q), _stream()))
+    if rows_form:
+        _lib.check_dense(lib.dlm_head_prefill(dt, s, r, _ptr(q), out.data_ptr(), out.stride(0), _stream()))
+        return
+    nsplit, part_o, part_ml = _head_parts(spec, M, pos, nsplit, proj.device)
+    _lib.check_dense(lib.dlm_head_decode(dt, s, r, _ptr(q), nsplit, _ptr(part_o), _ptr(part_ml), _stream()))
+    _lib.check_dense(lib.dlm_head_merge(dt, s, r, nsplit, _ptr(part_o), _ptr(part_ml), out.data_ptr(), out.stride(0), _stream()))
+
+
+def _head_args(spec, proj, off, q_norm, k_norm, eps, cache, pos, out, pos_dev):
     _need_cuda(cache, q_norm, k_norm)
     _same("head attention", cache, proj, out)
     _need_f32(q_norm, k_norm)
-    M, dt = proj.shape[0], dtype_code(proj)
+    M = proj.shape[0]
     if tuple(cache.shape[::2]) != (spec.kv_heads, spec.dim_p + spec.vdim_p) or out.shape[0] != M or proj.shape[1] < off + spec.proj_width:
         raise ValueError("head attention: the cache, the projections or the output have another shape")
     if q_norm.numel() != spec.dim_p or k_norm.numel() != spec.dim_p:
@@ -482,17 +487,14 @@ def head_attention(spec, proj, off, q_norm, k_norm, eps, cache, pos, out, pos_de
     r = _lib.HeadRows(proj=proj.data_ptr(), q_norm=_ptr(q_norm), k_norm=_ptr(k_norm), cache=_ptr(cache), pos_dev=_opt(pos_dev), ld=proj.stride(0), off=off, M=M,
                       pos=pos, eps=eps)
     q = torch.empty((M * spec.heads, spec.dim_p), dtype=proj.dtype, device=proj.device)
-    s, r = ctypes.byref(s), ctypes.byref(r)
-    _lib.check_dense(lib.dlm_head_prepare(dt, s, r, _ptr(q), _stream()))
-    if rows_form:
-        _lib.check_dense(lib.dlm_head_prefill(dt, s, r, _ptr(q), out.data_ptr(), out.stride(0), _stream()))
-        return
+    return ctypes.byref(s), ctypes.byref(r), q
+
+
+def _head_parts(spec, M, pos, nsplit, device):
     if nsplit is None:
         nsplit = head_splits(spec, M, pos + M)
-    part_o = torch.empty((M * spec.heads, nsplit, spec.vdim_p), dtype=torch.float32, device=proj.device)
-    part_ml = torch.empty((M * spec.heads, nsplit, 2), dtype=torch.float32, device=proj.device)
-    _lib.check_dense(lib.dlm_head_decode(dt, s, r, _ptr(q), nsplit, _ptr(part_o), _ptr(part_ml), _stream()))
-    _lib.check_dense(lib.dlm_head_merge(dt, s, r, nsplit, _ptr(part_o), _ptr(part_ml), out.data_ptr(), out.stride(0), _stream()))
+    part_o = torch.empty((M * spec.heads, nsplit, spec.vdim_p), dtype=torch.float32, device=device)
+    return nsplit, part_o, torch.empty((M * spec.heads, nsplit, 2), dtype=torch.float32, device=device)
 
 
 class StateSpec:
@@ -524,6 +526,28 @@ def short_conv(spec, proj, off, w, history, pos, q_scale, unit_eps, pos_dev=None
     """(act [M, channels], factors [M, 2 k_heads]) of the channels of proj [M, ld] from column `off` on; w fp32 [taps, channels],
     history [taps, channels] is brought forward."""
     lib = _lib.load_dense_library()
+    c, act, factors = _conv_args(spec, proj, off, w, history, pos, q_scale, unit_eps, pos_dev)
+    _lib.check_dense(lib.dlm_short_conv(dtype_code(proj), c, _ptr(act), _stream()))
+    return act, factors
+
+
+def conv_products(spec, proj, off, w, history, pos, q_scale, unit_eps, low_a, w_a, low_b, w_b, pos_dev=None):
+    """short_conv of one token, and in the same launch the products w_a low_a (fp32) and w_b low_b of short vectors.  Returns (act, factors,
+    the two results [1, N])."""
+    lib = _lib.load_dense_library()
+    _need_cuda(w_a, w_b)
+    _same("conv_products", proj, low_a, w_a, low_b, w_b)
+    if low_a.numel() != w_a.shape[1] or low_b.numel() != w_b.shape[1]:
+        raise ValueError("conv_products: shapes of the products do not match")
+    c, act, factors = _conv_args(spec, proj, off, w, history, pos, q_scale, unit_eps, pos_dev)
+    out_a = torch.empty((1, w_a.shape[0]), dtype=torch.float32, device=proj.device)
+    out_b = torch.empty((1, w_b.shape[0]), dtype=proj.dtype, device=proj.device)
+    a, b = (_lib.ShortProduct(w=_ptr(m), x=x.data_ptr(), out=_ptr(o), K=m.shape[1], N=m.shape[0]) for m, x, o in ((w_a, low_a, out_a), (w_b, low_b, out_b)))
+    _lib.check_dense(lib.dlm_conv_products(dtype_code(proj), c, _ptr(act), ctypes.byref(a), ctypes.byref(b), _stream()))
+    return act, factors, out_a, out_b
+
+
+def _conv_args(spec, proj, off, w, history, pos, q_scale, unit_eps, pos_dev):
     _need_cuda(w, history)
     _need_f32(w)
     _same("short_conv", history, proj)
@@ -535,8 +559,7 @@ def short_conv(spec, proj, off, w, history, pos, q_scale, unit_eps, pos_dev=None
     c = _lib.ShortConvArgs(proj=proj.data_ptr(), w=_ptr(w), history=_ptr(history), factors=_ptr(factors), pos_dev=_opt(pos_dev), ld=proj.stride(0),
                            k_heads=spec.k_heads, heads=spec.heads, dim=spec.dim_p, vdim=spec.vdim_p, taps=w.shape[0], off=off, M=M, pos=pos, q_scale=q_scale,
                            unit_eps=unit_eps)
-    _lib.check_dense(lib.dlm_short_conv(dtype_code(proj), ctypes.byref(c), _ptr(act), _stream()))
-    return act, factors
+    return ctypes.byref(c), act, factors
 
 
 # Up to this many tokens a portion goes through a recurrence token by token.
@@ -548,6 +571,19 @@ def recurrence(spec, qkv, offsets, state, pos, log2_decay=None, z=None, a_log=No
     log2_decay [heads]: a decay per head; z [M, heads * dim_p] with a_log, dt_bias, factors and beta [M, >= heads]: a decay per channel
     and the delta rule.  chunks: which form to run (default: by the number of tokens)."""
     lib = _lib.load_dense_library()
+    a, o = _recurrence_args(spec, qkv, offsets, state, pos, log2_decay, z, a_log, dt_bias, factors, beta, pos_dev)
+    nbytes = lib.dlm_recurrence_chunk_bytes(a)
+    if chunks is None:
+        chunks = qkv.shape[0] > STEPS_MAX_TOKENS and nbytes > 0
+    if chunks:
+        work = torch.empty((nbytes,), dtype=torch.uint8, device=qkv.device)
+        _lib.check_dense(lib.dlm_recurrence_chunks(dtype_code(qkv), a, _ptr(work), _ptr(o), _stream()))
+    else:
+        _lib.check_dense(lib.dlm_recurrence_steps(dtype_code(qkv), a, _ptr(o), _stream()))
+    return o
+
+
+def _recurrence_args(spec, qkv, offsets, state, pos, log2_decay, z, a_log, dt_bias, factors, beta, pos_dev):
     _need_cuda(state)
     _need_f32(state, log2_decay, z, a_log, dt_bias, factors)
     M, H = qkv.shape[0], spec.heads
@@ -562,16 +598,27 @@ def recurrence(spec, qkv, offsets, state, pos, log2_decay=None, z=None, a_log=No
     a = _lib.RecurrenceArgs(qkv=qkv.data_ptr(), log2_decay=_opt(log2_decay), z=_opt(z), a_log=_opt(a_log), dt_bias=_opt(dt_bias), factors=_opt(factors),
                             beta=_opt(beta), state=_ptr(state), pos_dev=_opt(pos_dev), ld=qkv.stride(0), ld_beta=0 if beta is None else beta.stride(0),
                             k_heads=spec.k_heads, heads=H, dim=spec.dim_p, vdim=spec.vdim_p, q_off=offsets[0], k_off=offsets[1], v_off=offsets[2], M=M, pos=pos)
-    o = torch.empty((M, spec.v_width), dtype=torch.float32, device=qkv.device)
-    nbytes = lib.dlm_recurrence_chunk_bytes(ctypes.byref(a))
-    if chunks is None:
-        chunks = M > STEPS_MAX_TOKENS and nbytes > 0
-    if chunks:
-        work = torch.empty((nbytes,), dtype=torch.uint8, device=qkv.device)
-        _lib.check_dense(lib.dlm_recurrence_chunks(dtype_code(qkv), ctypes.byref(a), _ptr(work), _ptr(o), _stream()))
-    else:
-        _lib.check_dense(lib.dlm_recurrence_steps(dtype_code(qkv), ctypes.byref(a), _ptr(o), _stream()))
-    return o
+    return ctypes.byref(a), torch.empty((M, spec.v_width), dtype=torch.float32, device=qkv.device)
+
+
+def attention_and_state(heads, state, proj, off, q_norm, k_norm, eps, cache, offsets, memory, log2_decay, pos, norm_w, true_cols, gate_off, out, pos_dev=None,
+                        nsplit=None):
+    """One token through windowed attention (`heads`, as head_attention with the keys split) and, beside it in the same three launches, a
+    recurrence with a decay per head (`state`, as recurrence) with the norm and gate of its read-outs: out [1, >=] = [attention | read-outs]."""
+    lib = _lib.load_dense_library()
+    if proj.shape[0] != 1 or norm_w.numel() != state.v_width or out.shape[1] < heads.heads * heads.vdim_p + state.v_width \
+            or proj.shape[1] < gate_off + state.v_width:
+        raise ValueError("attention_and_state: one token, and a norm weight, a gate and an output of the read-outs' width")
+    _need_cuda(norm_w)
+    _need_f32(norm_w)
+    dt = dtype_code(proj)
+    s, r, q = _head_args(heads, proj, off, q_norm, k_norm, eps, cache, pos, out, pos_dev)
+    a, o = _recurrence_args(state, proj, offsets, memory, pos, log2_decay, None, None, None, None, None, pos_dev)
+    _lib.check_dense(lib.dlm_head_state_begin(dt, s, r, _ptr(q), a, _ptr(o), _stream()))
+    nsplit, part_o, part_ml = _head_parts(heads, 1, pos, nsplit, proj.device)
+    _lib.check_dense(lib.dlm_head_decode(dt, s, r, _ptr(q), nsplit, _ptr(part_o), _ptr(part_ml), _stream()))
+    _lib.check_dense(lib.dlm_head_state_end(dt, s, r, nsplit, _ptr(part_o), _ptr(part_ml), out.data_ptr(), _ptr(o), _ptr(norm_w), proj[:, gate_off:].data_ptr(),
+                                            state.v_width, true_cols, eps, out[:, heads.heads * heads.vdim_p:].data_ptr(), _stream()))
 
 
 def gated_norm(o, w, eps, groups, true_cols, gate, out):

@@ -5,9 +5,9 @@ embedding.
 
 Two passes over the same weights and caches (dense.py has the ops; the residual is fp32 throughout):
 
-  one token      parallel: residual + norm + all projections (silu included) | query / key norm + cache append, attention over the
-                 keys of the window, merge | lightning state step | norm + gate | one product for both outputs
-                 channel_delta: residual + norm + all projections | convolution | decay and gate products | state step | norm + gate |
+  one token      seven launches a layer.  parallel: residual + norm + all projections (silu included) | query / key norm, cache append
+                 and lightning state step | attention over the keys of the window | merge, norm and gate | one product for both outputs
+                 channel_delta: residual + norm + all projections | convolution, decay and gate products | state step | norm and gate |
                  output product
                  feed-forward: residual + norm + gate / up with the activation | down
   many tokens    the same steps as products over all rows; the recurrences in chunks of 64 tokens
@@ -251,6 +251,10 @@ class ParallelLayer:
         if pos_dev is not None and not few:
             raise ValueError("these head sizes cannot run with the position on the device")
         nsplit = dense.head_splits(A, 1, capacity) if pos_dev is not None else None
+        if few and M == 1:
+            dense.attention_and_state(A, self.state, proj, 0, self.q_norm, self.k_norm, self.eps, cache["rows"], self.offsets, cache["state"],
+                                      self.log2_decay, pos, self.norm, self.true_cols, self.gate_off, out, pos_dev, nsplit)
+            return
         dense.head_attention(A, proj, 0, self.q_norm, self.k_norm, self.eps, cache["rows"], pos, out, pos_dev=pos_dev, nsplit=nsplit, rows_form=not few)
         o = dense.recurrence(self.state, proj, self.offsets, cache["state"], pos, log2_decay=self.log2_decay, pos_dev=pos_dev)
         dense.gated_norm(o, self.norm, self.eps, 1, self.true_cols, proj[:, self.gate_off:], out[:, A.heads * A.vdim_p:])
@@ -299,9 +303,13 @@ class DeltaLayer:
 
     def mix(self, proj, cache, pos, out, pos_dev, capacity):
         s = self.state
-        act, factors = dense.short_conv(s, proj, 0, self.conv, cache["history"], pos, self.q_scale, UNIT_EPS, pos_dev)
-        z = dense.product(proj[:, self.a_off:self.g_off], self.w_a2, out_f32=True)
-        gate = dense.product(proj[:, self.g_off:self.b_off], self.w_g2)
+        conv = (s, proj, 0, self.conv, cache["history"], pos, self.q_scale, UNIT_EPS)
+        low_a, low_g = proj[:, self.a_off:self.g_off], proj[:, self.g_off:self.b_off]
+        if proj.shape[0] == 1:
+            act, factors, z, gate = dense.conv_products(*conv, low_a, self.w_a2, low_g, self.w_g2, pos_dev)
+        else:
+            act, factors = dense.short_conv(*conv, pos_dev)
+            z, gate = dense.gemm(low_a, self.w_a2, out_f32=True), dense.gemm(low_g, self.w_g2)
         o = dense.recurrence(s, act, (0, s.qk_width, 2 * s.qk_width), cache["state"], pos, z=z, a_log=self.a_log, dt_bias=self.dt_bias, factors=factors,
                              beta=proj[:, self.b_off:], pos_dev=pos_dev)
         dense.gated_norm(o, self.norm, self.eps, s.heads, s.vdim, gate, out)

@@ -22,7 +22,7 @@ LIB_DIR = os.path.join(HERE, "lib")
 LIBRARIES = {
     "w4a16": ["capi.hip", "dequant.hip", "stream.hip", "gemv_ws.hip", "gemm_ws.hip", "gemm_wsk.hip", "gemm.hip", "attention.hip", "q4nx.hip", "lm_head.hip", "prefill_block.hip", "prefill_attention.hip"],
     "dense_lm": ["dense_capi.hip", "dense_gemv.hip", "dense_gemm.hip", "rows.hip", "moe.hip", "latent_attention.hip", "latent_prefill.hip",
-                 "head_attention.hip", "linear_attention.hip", "linear_chunks.hip"],
+                 "head_attention.hip", "linear_attention.hip", "linear_chunks.hip", "mixer_steps.hip"],
 }
 SOURCES = [s for sources in LIBRARIES.values() for s in sources]
 

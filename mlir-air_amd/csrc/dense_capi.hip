@@ -74,6 +74,17 @@ int check_recurrence(int dtype, const dlm_recurrence_args *a) {
     if (odd(a->qkv) || odd(a->state) || odd(a->z) || odd(a->dt_bias)) return DLM_ERR_ALIGN;
     return DLM_OK;
 }
+int check_conv(int dtype, const dlm_short_conv_args *c, const void *act) {
+    if (!c || !c->proj || !c->w || !c->history || !c->factors || !act) return DLM_ERR_NULL;
+    if (bad_type(dtype) || c->k_heads <= 0 || c->heads <= 0 || c->dim <= 0 || c->dim % 8 || c->vdim <= 0 || c->vdim % 8 || c->taps <= 0 || c->M <= 0 ||
+        c->M > 65535 * 4 || c->pos < 0 || c->ld % 8 || c->off < 0 || c->off % 8 || c->taps > 65535 || (c->pos_dev && c->M > 1) || !(c->unit_eps >= 0.f))
+        return DLM_ERR_SHAPE;
+    if (odd(c->proj) || odd(c->w) || odd(c->history) || odd(act)) return DLM_ERR_ALIGN;
+    return DLM_OK;
+}
+ConvArgs conv_of(const dlm_short_conv_args *c) {
+    return {c->k_heads, c->heads, c->dim, c->vdim, c->taps, (long)c->ld, c->off, c->w, c->factors, c->q_scale, c->unit_eps, c->M, c->pos_dev, c->pos};
+}
 LinearArgs linear_of(const dlm_recurrence_args *a) {
     LinearArgs l;
     l.k_heads = a->k_heads;
@@ -338,13 +349,44 @@ int dlm_head_merge(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, i
 }
 
 int dlm_short_conv(int dtype, const dlm_short_conv_args *c, void *act, void *stream) {
-    if (!c || !c->proj || !c->w || !c->history || !c->factors || !act) return DLM_ERR_NULL;
-    if (bad_type(dtype) || c->k_heads <= 0 || c->heads <= 0 || c->dim <= 0 || c->dim % 8 || c->vdim <= 0 || c->vdim % 8 || c->taps <= 0 || c->M <= 0 ||
-        c->M > 65535 * 4 || c->pos < 0 || c->ld % 8 || c->off < 0 || c->off % 8 || c->taps > 65535 || (c->pos_dev && c->M > 1) || !(c->unit_eps >= 0.f))
+    const int e = check_conv(dtype, c, act);
+    return e ? e : done(launch_short_conv(dtype, conv_of(c), c->proj, c->history, act, hs(stream)));
+}
+
+int dlm_head_state_begin(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, void *q, const dlm_recurrence_args *a, float *o, void *stream) {
+    int c = check_head(dtype, s, r);
+    if (!c) c = check_recurrence(dtype, a);
+    if (c) return c;
+    if (!q || !o) return DLM_ERR_NULL;
+    if (r->M != 1 || a->M != 1 || a->z) return DLM_ERR_SHAPE;
+    if (odd(q) || odd(o)) return DLM_ERR_ALIGN;
+    return done(launch_head_state_begin(dtype, head_of(s), head_rows_of(r), q, linear_of(a), o, hs(stream)));
+}
+
+int dlm_head_state_end(int dtype, const dlm_head_shape *s, const dlm_head_rows *r, int nsplit, const float *part_o, const float *part_ml, void *out,
+                       const float *o, const float *w, const void *gate, int cols, int true_cols, float eps, void *norm_out, void *stream) {
+    const int c = check_head(dtype, s, r);
+    if (c) return c;
+    if (!part_o || !part_ml || !out || !o || !w || !gate || !norm_out) return DLM_ERR_NULL;
+    if (r->M != 1 || nsplit <= 0 || nsplit > 256 || !decode_block_keys(dtype, head_view(head_of(s))) || cols <= 0 || cols % 4 || true_cols <= 0 ||
+        true_cols > cols || !(eps >= 0.f))
         return DLM_ERR_SHAPE;
-    if (odd(c->proj) || odd(c->w) || odd(c->history) || odd(act)) return DLM_ERR_ALIGN;
-    const ConvArgs a = {c->k_heads, c->heads, c->dim, c->vdim, c->taps, (long)c->ld, c->off, c->w, c->factors, c->q_scale, c->unit_eps, c->M, c->pos_dev, c->pos};
-    return done(launch_short_conv(dtype, a, c->proj, c->history, act, hs(stream)));
+    if (odd(part_o) || odd(out) || odd(o) || odd(w)) return DLM_ERR_ALIGN;
+    return done(launch_head_state_end(dtype, head_of(s), head_rows_of(r), nsplit, part_o, part_ml, out, GatedNorm{o, 1, cols, true_cols, w, eps, cols, cols}, gate,
+                                      norm_out, hs(stream)));
+}
+
+int dlm_conv_products(int dtype, const dlm_short_conv_args *c, void *act, const dlm_short_product *a, const dlm_short_product *b, void *stream) {
+    const int e = check_conv(dtype, c, act);
+    if (e) return e;
+    if (c->M != 1) return DLM_ERR_SHAPE;
+    for (const dlm_short_product *p : {a, b}) {
+        if (!p || !p->w || !p->x || !p->out) return DLM_ERR_NULL;
+        if (p->K <= 0 || p->K % 64 || p->N <= 0 || p->N % 16) return DLM_ERR_SHAPE;
+        if (odd(p->w) || odd(p->x)) return DLM_ERR_ALIGN;
+    }
+    return done(launch_conv_products(dtype, conv_of(c), c->proj, c->history, act, ShortProduct{a->w, a->x, a->out, a->K, a->N},
+                                     ShortProduct{b->w, b->x, b->out, b->K, b->N}, hs(stream)));
 }
 
 int dlm_recurrence_steps(int dtype, const dlm_recurrence_args *a, float *o, void *stream) {

@@ -196,6 +196,20 @@ struct GatedNorm {
 };
 hipError_t launch_gated_norm(int dtype, const GatedNorm &g, const void *gate, void *out, int M, hipStream_t stream);
 
+// Steps of one token that share a launch (r.M, a.M and c.M are 1): attention's preparation and a state step with a decay per head ...
+hipError_t launch_head_state_begin(int dtype, const HeadShape &s, const HeadRows &r, void *q, const LinearArgs &a, float *o, hipStream_t stream);
+// ... the merge of the keys' splits and the norm and gate of the read-outs (one group) ...
+hipError_t launch_head_state_end(int dtype, const HeadShape &s, const HeadRows &r, int nsplit, const float *part_o, const float *part_ml, void *out,
+                                 const GatedNorm &g, const void *gate, void *norm_out, hipStream_t stream);
+// ... a short convolution and two products out[N] = w[N, K] x[K] with short rows, the first one's result fp32
+struct ShortProduct {
+    const void *w, *x;
+    void *out;
+    int K, N;
+};
+hipError_t launch_conv_products(int dtype, const ConvArgs &c, const void *proj, void *history, void *act, const ShortProduct &a, const ShortProduct &b,
+                                hipStream_t stream);
+
 // Latent attention.  Sizes are the padded ones; a cache row is [latent kv_rank | rotated key part rot].
 struct LatentShape {
     int heads, dim, rot, vdim, rank;    // padded sizes (dim, rot, vdim multiples of 32, rank of 64)

@@ -230,11 +230,18 @@ def test_abi_rejects_bad_arguments_before_touching_the_gpu():
     c = lambda **k: lib.dlm_short_conv(0, ref(_lib.ShortConvArgs(**{**conv, **k})), p, None)
     assert c(taps=0) == SHAPE and c(pos_dev=p) == SHAPE and c(M=0) == SHAPE and c(off=4) == SHAPE and c(history=None) == NULL and c(w=p + 4) == ALIGN
     rec = dict(qkv=p, log2_decay=p, state=p, ld=512, k_heads=2, heads=4, dim=64, vdim=32, M=1)
-    q = lambda f=lib.dlm_recurrence_steps, **k: f(0, ref(_lib.RecurrenceArgs(**{**rec, **k})), *((p,) if f == lib.dlm_recurrence_steps else (p, p)), None)
+    step = lambda f=lib.dlm_recurrence_steps, **k: f(0, ref(_lib.RecurrenceArgs(**{**rec, **k})), *((p,) if f == lib.dlm_recurrence_steps else (p, p)), None)
     for k in (dict(dim=32), dict(dim=576), dict(vdim=16), dict(heads=3), dict(M=0), dict(q_off=4), dict(pos=-1)):
-        assert q(**k) == SHAPE and q(lib.dlm_recurrence_chunks, **k) == SHAPE, k
-    assert q(log2_decay=None) == NULL and q(z=p) == NULL and q(log2_decay=None, z=p) == NULL and q(state=p + 4) == ALIGN
-    assert q(lib.dlm_recurrence_chunks, dim=192) == SHAPE and lib.dlm_recurrence_chunk_bytes(ref(_lib.RecurrenceArgs(**{**rec, "dim": 192}))) == 0
+        assert step(**k) == SHAPE and step(lib.dlm_recurrence_chunks, **k) == SHAPE, k
+    assert step(log2_decay=None) == NULL and step(z=p) == NULL and step(log2_decay=None, z=p) == NULL and step(state=p + 4) == ALIGN
+    assert step(lib.dlm_recurrence_chunks, dim=192) == SHAPE and lib.dlm_recurrence_chunk_bytes(ref(_lib.RecurrenceArgs(**{**rec, "dim": 192}))) == 0
     assert lib.dlm_recurrence_chunk_bytes(ref(_lib.RecurrenceArgs(**rec))) > 0
     gn = lambda **k: lib.dlm_gated_norm(*{**dict(dt=0, o=p, w=p, gate=p, ldg=64, out=p, ldo=64, M=1, groups=2, cols=32, true=32, eps=1e-5, s=None), **k}.values())
     assert gn(o=None) == NULL and gn(true=33) == SHAPE and gn(ldo=32) == SHAPE and gn(cols=30) == SHAPE and gn(M=0) == SHAPE and gn(w=p + 4) == ALIGN
+    begin = lambda rk={}, ak={}, q=p: lib.dlm_head_state_begin(0, s, ref(_lib.HeadRows(**{**hr, **rk})), q, ref(_lib.RecurrenceArgs(**{**rec, **ak})), p, None)
+    assert begin(rk=dict(M=2)) == SHAPE and begin(ak=dict(M=2)) == SHAPE and begin(q=None) == NULL and begin(ak=dict(vdim=8)) == SHAPE
+    finish = lambda nsplit=1, cols=64, true=64, o=p: lib.dlm_head_state_end(0, s, r, nsplit, p, p, p, o, p, p, cols, true, 1e-5, p, None)
+    assert finish(nsplit=0) == SHAPE and finish(cols=62) == SHAPE and finish(true=65) == SHAPE and finish(o=None) == NULL
+    prod = lambda **k: ref(_lib.ShortProduct(**{**dict(w=p, x=p, out=p, K=64, N=16), **k}))
+    both = lambda a=prod(), b=prod(), **k: lib.dlm_conv_products(0, ref(_lib.ShortConvArgs(**{**conv, "M": 1, **k})), p, a, b, None)
+    assert both(M=2) == SHAPE and both(a=prod(K=32)) == SHAPE and both(b=prod(N=8)) == SHAPE and both(a=prod(out=None)) == NULL and both(b=prod(x=p + 2)) == ALIGN
