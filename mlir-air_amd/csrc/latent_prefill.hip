@@ -39,7 +39,7 @@ struct PrefillArgs {
     int v_off, gate_off;     // columns of the values in kv, of the gate in q's matrix
     int M, total;            // queries, keys (the queries are the last M positions)
     float scale_log2;
-    const float *sink;       // (NULL: none)
+    const float *sink;
     long head_q, group_q, head_k, head_v;   // elements between two heads' queries, key / value heads' queries, keys, values
     int group, window, ring;                // query heads per key / value head
     float out_scale;
@@ -103,8 +103,9 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
     // a chunk is 8 elements of a row; the first dim of a K row come from the expanded matrix, the rest from the cache
     const T *k_base = p.kv + kvh * p.head_k, *v_base = p.kv + p.v_off + kvh * p.head_v + vcol0, *r_base = p.cache + p.rot_off;
     auto row_of = [&](int kb, int i) {   // row of key kb + i of a block (a ring holds whole blocks)
-        const int key = kb + i < p.total ? i : p.total - 1 - kb;
-        return (WINDOW ? kb % p.ring : kb) + key;
+        if constexpr (WINDOW) return kb % p.ring + (kb + i < p.total ? i : p.total - 1 - kb);
+        const int key = kb + i;
+        return key < p.total ? key : p.total - 1;
     };
     auto at = [&](const T *base, int row, long ld, int e) -> Vec8<T> {
         if constexpr (EXACT) return load8(reinterpret_cast<const T *>(reinterpret_cast<const char *>(base) + (uint32_t)(row * (uint32_t)ld + e) * (uint32_t)sizeof(T)));
@@ -154,7 +155,7 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
         if (it < blocks) stage(it);
         __syncthreads();
         if (it + SETS < blocks) fetch(it + SETS);
-        if (it < blocks && kb <= wave_last && kb + KB > wave_first) {
+        if (it < blocks && kb <= wave_last && (!WINDOW || kb + KB > wave_first)) {
             floatx4 s[NKK][QB];
 #pragma unroll
             for (int kk = 0; kk < NKK; ++kk) {
@@ -265,12 +266,12 @@ __global__ void __launch_bounds__(SETS * kSetThreads, SETS) latent_prefill_kerne
         }
     }
 
-    const float snk = p.sink ? p.sink[head] * 1.4426950408889634f : 0.f;
+    const float snk = WINDOW ? 0.f : p.sink[head] * 1.4426950408889634f;
 #pragma unroll
     for (int b = 0; b < QB; ++b) {
         const int qi = q0 + 16 * b + ql;
         if (qi >= p.M) continue;
-        const float inv = (WINDOW ? p.out_scale : 1.0f) / (l[b][0] + (p.sink ? exp2f(snk - m[b] * p.scale_log2) : 0.f));
+        const float inv = WINDOW ? p.out_scale / l[b][0] : 1.0f / (l[b][0] + exp2f(snk - m[b] * p.scale_log2));
         const int col = head * p.vdim + vcol0 + 4 * g;
         const T *gate = p.q + (size_t)qi * p.ldq + p.gate_off + col;
         T *dst = p.out + (size_t)qi * p.ldo + col;

@@ -12,7 +12,7 @@
 //   linear_chunk / delta_chunk   one workgroup per head and chunk: q e^G, (k e^(G_last - G))^T, B, e^(G_last), and U as
 //                                U0 - W S: U0 = V, or U0 = (1 + diag(beta) A)^-1 diag(beta) V and W the same of k e^G
 //   chunk_scan                   one workgroup per head and 16 value columns goes through the chunks: S stays in registers (and
-//                                in LDS as an operand), the next chunk's operands travel while one is multiplied
+//                                in LDS as an operand)
 //
 // All of it is 32-bit, products included (fp32 MFMA).  No exponent is ever positive: the 16 x 16 blocks on the diagonal of A
 // and B weigh every pair of tokens on its own, the blocks under it go through the decay up to the border of the row block,
@@ -379,92 +379,127 @@ __global__ void __launch_bounds__(kThreads, sizeof(T) == 2 ? 2 : 1) delta_chunk_
     }
 }
 
-// A workgroup: 16 value columns of a head; those of one head run on one XCD, whose L2 the head's operands go through once.  A wave
-// owns 16 tokens of a chunk in the products with S and B, and the key channels 16 (wave + 4 c) .. + 15 of S.
+// A workgroup: 16 value columns of a head; those of one head run on one XCD, whose L2 the head's operands go through once.  Four waves
+// bring the state forward (16 tokens each in the product with W, the key channels 16 (wave + 4 c) .. + 15 of S each), four make the
+// outputs (16 tokens each); a SIMD has one of either, which fill each other's waits.  S and U go through LDS, two buffers each.
+// A wave requests the operands of the next chunk as soon as it has multiplied those of this one, products with S while those with U
+// are made and the other way round.  (Behind the last chunk that one is fetched again rather than nothing, so that the number of loads
+// in flight is known at every wait.)
 template <int ND, bool DELTA>
-__global__ void __launch_bounds__(kThreads, 1) chunk_scan_kernel(const LinearArgs a, const float *work, int chunks, bool first, float *o) {
+__global__ void __launch_bounds__(2 * kThreads, 1) chunk_scan_kernel(const LinearArgs a, const float *work, int chunks, bool first, float *o) {
     constexpr int D = 64 * ND, KS = 2 * ND;
-    __shared__ __attribute__((aligned(16))) float ss[16][D + 4], us[16][kC + 4];
+    __shared__ __attribute__((aligned(16))) float ss[2][16][D + 4], us[2][16][kC + 4];
     const int tid = threadIdx.x, lane = tid & 63, ql = lane & 15, g = lane >> 4;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int wave8 = __builtin_amdgcn_readfirstlane(tid >> 6), wave = wave8 & 3;
     const int tiles = a.vdim / 16, xcd = blockIdx.x & 7, at = blockIdx.x >> 3;
     const int h = 8 * (at / tiles) + xcd, v0 = 16 * (at % tiles), tok = 16 * wave;
     if (h >= a.heads) return;
     const ChunkLayout lay{D, a.vdim, DELTA};
     work += (size_t)h * chunks * lay.size();
-    float *st = a.state + ((size_t)h * a.vdim + v0 + ql) * D + 4 * g;
-    const bool from_zero = first && (a.pos_dev ? a.pos_dev[0] : a.pos) == 0;
-    floatx4 s[ND];
-#pragma unroll
-    for (int c = 0; c < ND; ++c) {
-        s[c] = from_zero ? floatx4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const floatx4 *>(st + 16 * (wave + 4 * c));
-        *reinterpret_cast<floatx4 *>(&ss[ql][16 * (wave + 4 * c) + 4 * g]) = s[c];
-    }
-    // The operands of the next chunk are requested as soon as those of this one have been multiplied: the products with S while those
-    // with U are made, and the other way round.  (Behind the last chunk it is fetched again rather than nothing, so that the number of
-    // loads in flight is known at every wait.)
-    Vec8<float> w[DELTA ? KS : 1], q[KS], k[ND][2], b[2];
-    floatx4 u0, e[ND];
     auto operand = [&](const float *m, int piece) {
         const float *x = m + piece * 512 + lane * 4;
         return Vec8<float>{*reinterpret_cast<const floatx4 *>(x), *reinterpret_cast<const floatx4 *>(x + 256)};
     };
-    auto fetch_state_side = [&](const float *p) {
-#pragma unroll
-        for (int t = 0; t < KS; ++t) {
-            if constexpr (DELTA) w[t] = operand(p + lay.w(), wave * KS + t);
-            q[t] = operand(p + lay.q(), wave * KS + t);
-        }
-        u0 = *reinterpret_cast<const floatx4 *>(p + lay.u() + ((v0 / 16 * 4 + wave) * 64 + lane) * 4);
-#pragma unroll
-        for (int c = 0; c < ND; ++c) e[c] = *reinterpret_cast<const floatx4 *>(p + lay.e() + 16 * (wave + 4 * c) + 4 * g);
-    };
-    auto fetch_token_side = [&](const float *p) {
-#pragma unroll
-        for (int t = 0; t < 2; ++t) b[t] = operand(p + lay.b(), wave * 2 + t);   // (the first two waves use one)
+    const floatx4 zero = floatx4{0.f, 0.f, 0.f, 0.f};
+
+    if (wave8 < 4) {
+        float *st = a.state + ((size_t)h * a.vdim + v0 + ql) * D + 4 * g;
+        const bool from_zero = first && (a.pos_dev ? a.pos_dev[0] : a.pos) == 0;
+        floatx4 s[ND];
 #pragma unroll
         for (int c = 0; c < ND; ++c) {
-#pragma unroll
-            for (int t = 0; t < 2; ++t) k[c][t] = operand(p + lay.k(), (wave + 4 * c) * 2 + t);
+            s[c] = from_zero ? zero : *reinterpret_cast<const floatx4 *>(st + 16 * (wave + 4 * c));
+            *reinterpret_cast<floatx4 *>(&ss[0][ql][16 * (wave + 4 * c) + 4 * g]) = s[c];
         }
-    };
-    fetch_state_side(work);
-    fetch_token_side(work);
-    __syncthreads();
-    for (int chunk = 0; chunk < chunks; ++chunk) {
-        floatx4 kept[ND];
+        Vec8<float> w[DELTA ? KS : 1], k[ND][2];
+        floatx4 u, e[ND];
+        auto fetch_w = [&](const float *p) {
+            if constexpr (DELTA) {
 #pragma unroll
-        for (int c = 0; c < ND; ++c) kept[c] = s[c] * e[c];
-        work += chunk + 1 < chunks ? lay.size() : 0;
-        floatx4 acc = floatx4{0.f, 0.f, 0.f, 0.f}, out = acc;
+                for (int t = 0; t < KS; ++t) w[t] = operand(p + lay.w(), wave * KS + t);
+            }
+            u = *reinterpret_cast<const floatx4 *>(p + lay.u() + ((v0 / 16 * 4 + wave) * 64 + lane) * 4);
 #pragma unroll
-        for (int t = 0; t < KS; ++t) {
-            const Vec8<float> sv = load8(&ss[ql][32 * t + 8 * g]);
-            if constexpr (DELTA) acc = mma32(w[t], sv, acc);
-            out = mma32(q[t], sv, out);
-        }
-        *reinterpret_cast<floatx4 *>(&us[ql][tok + 4 * g]) = u0 - acc;
-        fetch_state_side(work);
-        __syncthreads();   // U is there; S has been read by every wave
-        const Vec8<float> ua = load8(&us[ql][8 * g]), ub = load8(&us[ql][32 + 8 * g]);
+            for (int c = 0; c < ND; ++c) e[c] = *reinterpret_cast<const floatx4 *>(p + lay.e() + 16 * (wave + 4 * c) + 4 * g);
+        };
+        auto fetch_k = [&](const float *p) {
 #pragma unroll
-        for (int c = 0; c < ND; ++c) s[c] = mma32(k[c][0], ua, kept[c]);
-        out = mma32(b[0], ua, out);
+            for (int c = 0; c < ND; ++c)
 #pragma unroll
-        for (int c = 0; c < ND; ++c) {
-            s[c] = mma32(k[c][1], ub, s[c]);
-            *reinterpret_cast<floatx4 *>(&ss[ql][16 * (wave + 4 * c) + 4 * g]) = s[c];
-        }
-        if (wave >= 2) out = mma32(b[1], ub, out);
-        fetch_token_side(work);
-        const int m = chunk * kC + tok + 4 * g;
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-            if (m + r < a.M) o[(size_t)(m + r) * a.heads * a.vdim + (size_t)h * a.vdim + v0 + ql] = out[r];
+                for (int t = 0; t < 2; ++t) k[c][t] = operand(p + lay.k(), (wave + 4 * c) * 2 + t);
+        };
+        fetch_w(work);
+        fetch_k(work);
+        if constexpr (!DELTA) *reinterpret_cast<floatx4 *>(&us[0][ql][tok + 4 * g]) = u;
         __syncthreads();
-    }
+        for (int chunk = 0; chunk < chunks; ++chunk) {
+            const int b = chunk & 1;
+            work += chunk + 1 < chunks ? lay.size() : 0;
 #pragma unroll
-    for (int c = 0; c < ND; ++c) *reinterpret_cast<floatx4 *>(st + 16 * (wave + 4 * c)) = s[c];
+            for (int c = 0; c < ND; ++c) s[c] *= e[c];
+            if constexpr (DELTA) {
+                floatx4 x = zero, y = zero;
+#pragma unroll
+                for (int t = 0; t < KS; t += 2) {
+                    x = mma32(w[t], load8(&ss[b][ql][32 * t + 8 * g]), x);
+                    y = mma32(w[t + 1], load8(&ss[b][ql][32 * t + 32 + 8 * g]), y);
+                }
+                *reinterpret_cast<floatx4 *>(&us[b][ql][tok + 4 * g]) = u - (x + y);
+                fetch_w(work);
+                __syncthreads();   // U is there
+            } else {
+                fetch_w(work);
+            }
+            const Vec8<float> ua = load8(&us[b][ql][8 * g]), ub = load8(&us[b][ql][32 + 8 * g]);
+#pragma unroll
+            for (int c = 0; c < ND; ++c) s[c] = mma32(k[c][0], ua, s[c]);
+#pragma unroll
+            for (int c = 0; c < ND; ++c) {
+                s[c] = mma32(k[c][1], ub, s[c]);
+                *reinterpret_cast<floatx4 *>(&ss[b ^ 1][ql][16 * (wave + 4 * c) + 4 * g]) = s[c];
+            }
+            fetch_k(work);
+            if constexpr (!DELTA) *reinterpret_cast<floatx4 *>(&us[b ^ 1][ql][tok + 4 * g]) = u;
+            __syncthreads();       // the next S (and, without the delta rule, U) is there, this one has been read
+        }
+#pragma unroll
+        for (int c = 0; c < ND; ++c) *reinterpret_cast<floatx4 *>(st + 16 * (wave + 4 * c)) = s[c];
+    } else {
+        Vec8<float> q[KS], m[2];
+        auto fetch_q = [&](const float *p) {
+#pragma unroll
+            for (int t = 0; t < KS; ++t) q[t] = operand(p + lay.q(), wave * KS + t);
+        };
+        auto fetch_b = [&](const float *p) {
+#pragma unroll
+            for (int t = 0; t < 2; ++t) m[t] = operand(p + lay.b(), wave * 2 + t);   // (the first two waves use one)
+        };
+        fetch_q(work);
+        fetch_b(work);
+        o += (size_t)(tok + 4 * g) * a.heads * a.vdim + (size_t)h * a.vdim + v0 + ql;
+        __syncthreads();
+        for (int chunk = 0; chunk < chunks; ++chunk) {
+            const int b = chunk & 1;
+            work += chunk + 1 < chunks ? lay.size() : 0;
+            floatx4 x = zero, y = zero;
+#pragma unroll
+            for (int t = 0; t < KS; t += 2) {
+                x = mma32(q[t], load8(&ss[b][ql][32 * t + 8 * g]), x);
+                y = mma32(q[t + 1], load8(&ss[b][ql][32 * t + 32 + 8 * g]), y);
+            }
+            fetch_q(work);
+            if constexpr (DELTA) __syncthreads();
+            x = mma32(m[0], load8(&us[b][ql][8 * g]), x);
+            if (wave >= 2) y = mma32(m[1], load8(&us[b][ql][32 + 8 * g]), y);
+            fetch_b(work);
+            x += y;
+            const int row = chunk * kC + tok + 4 * g;
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                if (row + r < a.M) o[(size_t)(chunk * kC + r) * a.heads * a.vdim] = x[r];
+            __syncthreads();
+        }
+    }
 }
 
 // Chunks that are worked on at once: their operands stay within reach of the last-level cache.
@@ -495,10 +530,10 @@ hipError_t chunks(LinearArgs a, float *work, float *o, hipStream_t stream) {
             b.z += (size_t)m0 * a.heads * a.dim;
             b.factors += (size_t)m0 * 2 * a.k_heads;
             hipLaunchKernelGGL((delta_chunk_kernel<T, ND>), grid, dim3(kThreads), lds, stream, b, q, k, v, beta + (size_t)m0 * a.ld_beta, work);
-            hipLaunchKernelGGL((chunk_scan_kernel<ND, true>), scan, dim3(kThreads), 0, stream, a, work, n, m0 == 0, om);
+            hipLaunchKernelGGL((chunk_scan_kernel<ND, true>), scan, dim3(2 * kThreads), 0, stream, a, work, n, m0 == 0, om);
         } else {
             hipLaunchKernelGGL((linear_chunk_kernel<T, ND>), grid, dim3(kThreads), 0, stream, a, q, k, v, work);
-            hipLaunchKernelGGL((chunk_scan_kernel<ND, false>), scan, dim3(kThreads), 0, stream, a, work, n, m0 == 0, om);
+            hipLaunchKernelGGL((chunk_scan_kernel<ND, false>), scan, dim3(2 * kThreads), 0, stream, a, work, n, m0 == 0, om);
         }
         const hipError_t e = hipGetLastError();
         if (e != hipSuccess) return e;
