@@ -170,7 +170,13 @@ __device__ __forceinline__ float sigmoid_of(float z) {
     return sigmoid_f32(z);
 }
 __device__ __forceinline__ float gelu_tanh_f32(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * z * z, z, z))); }
-__device__ __forceinline__ float softplus_f32(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// log(1 + e^z) = max(z, 0) + log(1 + t), t = e^-|z|; log(1 + t) = log(u) t / (u - 1) with u the rounded 1 + t, whose error the
+// quotient takes back (Goldberg, "What Every Computer Scientist Should Know About Floating-Point Arithmetic", 1991)
+__device__ __forceinline__ float softplus_f32(float z) {
+    const float t = __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(z)), u = 1.0f + t, d = u - 1.0f;
+    const float l = 0.6931471805599453f * __builtin_amdgcn_logf(u) * t * __builtin_amdgcn_rcpf(d);
+    return fmaxf(z, 0.0f) + (d == 0.0f ? t : l);
+}
 
 // sum over a group of `n` neighbouring lanes (a power of two), every lane of it receiving the sum
 __device__ __forceinline__ float group_sum(float v, int n) {

@@ -401,6 +401,18 @@ __global__ void __launch_bounds__(2 * kThreads, 1) chunk_scan_kernel(const Linea
         return Vec8<float>{*reinterpret_cast<const floatx4 *>(x), *reinterpret_cast<const floatx4 *>(x + 256)};
     };
     const floatx4 zero = floatx4{0.f, 0.f, 0.f, 0.f};
+    // m S (two chains), and the operands from LDS in registers before the first product: the compiler would fetch them two by two
+    auto times_state = [&](const Vec8<float> (&m)[KS], const float (*rows)[D + 4], floatx4 &x, floatx4 &y) {
+        Vec8<float> sv[KS];
+#pragma unroll
+        for (int t = 0; t < KS; ++t) sv[t] = load8(&rows[ql][32 * t + 8 * g]);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int t = 0; t < KS; t += 2) {
+            x = mma32(m[t], sv[t], x);
+            y = mma32(m[t + 1], sv[t + 1], y);
+        }
+    };
 
     if (wave8 < 4) {
         float *st = a.state + ((size_t)h * a.vdim + v0 + ql) * D + 4 * g;
@@ -411,7 +423,7 @@ __global__ void __launch_bounds__(2 * kThreads, 1) chunk_scan_kernel(const Linea
             s[c] = from_zero ? zero : *reinterpret_cast<const floatx4 *>(st + 16 * (wave + 4 * c));
             *reinterpret_cast<floatx4 *>(&ss[0][ql][16 * (wave + 4 * c) + 4 * g]) = s[c];
         }
-        Vec8<float> w[DELTA ? KS : 1], k[ND][2];
+        Vec8<float> w[KS], k[ND][2];   // (w: the delta rule only)
         floatx4 u, e[ND];
         auto fetch_w = [&](const float *p) {
             if constexpr (DELTA) {
@@ -439,11 +451,7 @@ __global__ void __launch_bounds__(2 * kThreads, 1) chunk_scan_kernel(const Linea
             for (int c = 0; c < ND; ++c) s[c] *= e[c];
             if constexpr (DELTA) {
                 floatx4 x = zero, y = zero;
-#pragma unroll
-                for (int t = 0; t < KS; t += 2) {
-                    x = mma32(w[t], load8(&ss[b][ql][32 * t + 8 * g]), x);
-                    y = mma32(w[t + 1], load8(&ss[b][ql][32 * t + 32 + 8 * g]), y);
-                }
+                times_state(w, ss[b], x, y);
                 *reinterpret_cast<floatx4 *>(&us[b][ql][tok + 4 * g]) = u - (x + y);
                 fetch_w(work);
                 __syncthreads();   // U is there
@@ -451,6 +459,7 @@ __global__ void __launch_bounds__(2 * kThreads, 1) chunk_scan_kernel(const Linea
                 fetch_w(work);
             }
             const Vec8<float> ua = load8(&us[b][ql][8 * g]), ub = load8(&us[b][ql][32 + 8 * g]);
+            __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
             for (int c = 0; c < ND; ++c) s[c] = mma32(k[c][0], ua, s[c]);
 #pragma unroll
@@ -482,15 +491,12 @@ __global__ void __launch_bounds__(2 * kThreads, 1) chunk_scan_kernel(const Linea
             const int b = chunk & 1;
             work += chunk + 1 < chunks ? lay.size() : 0;
             floatx4 x = zero, y = zero;
-#pragma unroll
-            for (int t = 0; t < KS; t += 2) {
-                x = mma32(q[t], load8(&ss[b][ql][32 * t + 8 * g]), x);
-                y = mma32(q[t + 1], load8(&ss[b][ql][32 * t + 32 + 8 * g]), y);
-            }
+            times_state(q, ss[b], x, y);
             fetch_q(work);
             if constexpr (DELTA) __syncthreads();
-            x = mma32(m[0], load8(&us[b][ql][8 * g]), x);
-            if (wave >= 2) y = mma32(m[1], load8(&us[b][ql][32 + 8 * g]), y);
+            const Vec8<float> ua = load8(&us[b][ql][8 * g]), ub = load8(&us[b][ql][32 + 8 * g]);
+            x = mma32(m[0], ua, x);
+            if (wave >= 2) y = mma32(m[1], ub, y);
             fetch_b(work);
             x += y;
             const int row = chunk * kC + tok + 4 * g;

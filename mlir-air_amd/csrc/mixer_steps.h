@@ -193,7 +193,7 @@ __device__ __forceinline__ void recurrence_step(const LinearArgs &a, float *o, i
     float ea = 0.f, g1 = 1.f;
     floatx4 bias[ND];
     if constexpr (DELTA) {
-        ea = expf(a.a_log[h]);
+        ea = -expf(a.a_log[h]) * 1.4426950408889634f;
 #pragma unroll
         for (int c = 0; c < ND; ++c) bias[c] = *reinterpret_cast<const floatx4 *>(a.dt_bias + (size_t)h * a.dim + 64 * c + l4);
     } else {
@@ -230,7 +230,7 @@ __device__ __forceinline__ void recurrence_step(const LinearArgs &a, float *o, i
             for (int c = 0; c < ND; ++c)
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    s[c][e] *= expf(-ea * softplus_f32(cur.z[c][e] + bias[c][e]));
+                    s[c][e] *= __builtin_amdgcn_exp2f(ea * softplus_f32(cur.z[c][e] + bias[c][e]));
                     cur.k[c][e] *= cur.kf;
                     cur.q[c][e] *= cur.qf;
                     p = fmaf(s[c][e], cur.k[c][e], p);
