@@ -21,7 +21,8 @@ PLAIN, RESIDUAL, EMBED, FINAL = 0, 1, 2, 3
 NORMED = 4
 OUT_ELEM, OUT_F32, OUT_SWIGLU, OUT_GEGLU = 0, 1, 2, 3
 GATE_NONE, GATE_SILU, GATE_GELU = 0, 1, 2
-STATE_PAD = 64   # a recurrence's query / key size
+STATE_PAD = 64   # a recurrence's query / key size ...
+STATE_MAX = 512  # ... and the largest there is a kernel for
 
 
 def pad_to(n, k):
@@ -505,6 +506,9 @@ class StateSpec:
     def __init__(self, heads, k_heads, dim, vdim):
         self.heads, self.k_heads, self.dim, self.vdim = heads, k_heads, dim, vdim
         self.dim_p, self.vdim_p = pad_to(dim, STATE_PAD), pad_to(vdim, HEAD_PAD)
+
+    def supported(self):
+        return self.dim_p <= STATE_MAX
 
     @property
     def qk_width(self):

@@ -199,6 +199,11 @@ class _Tensors:
         return place(self.f32(name, heads * dim).reshape(heads, dim), (heads, dim_p)).reshape(-1).contiguous()
 
 
+def _check_state(spec):
+    if not spec.supported():
+        raise ValueError(f"no recurrence kernel for queries and keys of {spec.dim}")
+
+
 def _output_width(columns):
     return dense.pad_to(columns, dense.KP)
 
@@ -235,6 +240,7 @@ class ParallelLayer:
     def check(self, dtype):
         if not (self.attn.decode_supported(dtype) or self.attn.prefill_supported(dtype)):
             raise ValueError("no attention kernel for these head sizes")
+        _check_state(self.state)
 
     def captured(self, dtype):
         return self.attn.decode_supported(dtype)
@@ -292,7 +298,7 @@ class DeltaLayer:
         self.w_o = place(t.heads_out("mix.o", m.heads, m.vdim, s.vdim_p), (t.WP, _output_width(s.v_width))).contiguous()
 
     def check(self, dtype):
-        pass
+        _check_state(self.state)
 
     def captured(self, dtype):
         return True

@@ -198,6 +198,16 @@ def test_loader_and_registry(tmp_path):
         models.load_model(path, dtype=torch.float32, device="cpu")
 
 
+def test_sizes_without_a_kernel_are_refused_when_the_model_is_made():
+    from air_hip import sitirax
+
+    for config in (sitirax_config([sitirax_delta(dim=520)]), sitirax_config([sitirax_delta(), sitirax_parallel(right_dim=520)]),
+                   sitirax_config([sitirax_parallel(dim=1100, vdim=1100)])):
+        w, cfg = sitirax_weights(config, 1), sitirax.SitiraxConfig.from_json(config)
+        with pytest.raises(ValueError, match="layer .: no"):
+            sitirax.SitiraxModel(cfg, lambda n, s: torch.from_numpy(w[n]), torch.float32, "cpu")
+
+
 def test_abi_rejects_bad_arguments_before_touching_the_gpu():
     from air_hip import _lib
 
