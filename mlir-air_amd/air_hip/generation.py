@@ -2,7 +2,7 @@
 
 `generate` is the loop of the reference's `generate`
 (programming_examples/llms/llama32_1b_int4/llama32_1b_int4_inference.py:494-575) with the model behind an interface:
-the int4 Llama (decode.LlamaModel) and the dense-weight models (kuvonex.KuvonexModel) both run through it.
+the int4 Llama (decode.LlamaModel) and the dense-weight models (kuvonex.KuvonexModel, sitirax.SitiraxModel) all run through it.
 """
 
 
