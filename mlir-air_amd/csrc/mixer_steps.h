@@ -87,7 +87,7 @@ __device__ __forceinline__ void head_merge_step(const HeadShape &s, int M, const
     const float scale = s.out_scale / (red[4] + red[5] + red[6] + red[7]);
     // a thread adds every `ways`-th split of four columns
     for (int c0 = 0; c0 < s.vdim; c0 += 4 * kStepThreads) {
-        const int width = (s.vdim - c0) / 4 < kStepThreads ? (s.vdim - c0) / 4 : kStepThreads;   // four-column pieces of this round
+        const int width = (s.vdim - c0) / 4 < kStepThreads ? (s.vdim - c0) / 4 : kStepThreads;   // four-column pieces of this pass
         const int ways = kStepThreads / width, way = tid / width, col = c0 + 4 * (tid % width);
         floatx4 a = floatx4{0.f, 0.f, 0.f, 0.f};
         if (way < ways)
